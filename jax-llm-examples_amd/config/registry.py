@@ -93,3 +93,4 @@ def _ensure_builtin() -> None:
     from ..parts import tiradra as _tiradra  # noqa: F401
     from ..parts import mazotar as _mazotar  # noqa: F401
     from ..parts import sudilorn as _sudilorn  # noqa: F401
+    from ..parts import folivik as _folivik  # noqa: F401

@@ -236,8 +236,10 @@ class ReferenceOps:
         return logits.copy_(torch.tanh(logits / cap) * cap)
 
     def sigmoid_mul(self, o, gate):
-        """``o * sigmoid(gate)`` element by element (``gate``: a view with the same shape), float32 inside."""
-        return (o.float() * torch.sigmoid(gate.float())).to(o.dtype)
+        """``o * sigmoid(gate)``, float32 inside: element by element, or (``gate`` narrower than ``o``) one gate for as many
+        neighbouring elements of ``o`` as it is narrower."""
+        g = torch.sigmoid(gate.float())
+        return (o.float() * g.repeat_interleave(o.shape[1] // g.shape[1], dim=1)).to(o.dtype)
 
     def conv_attention(self, proj, bias, conv_w, taps: int, state, num_heads: int, num_kv_heads: int, head_dim: int,
                        value_dim: int, page_dim: int, prep, ctx, kv_cache, writes: bool, slot_mapping, block_table,
@@ -295,18 +297,20 @@ class ReferenceOps:
             values_t(kv_cache)[page, :, :, off] = pad(v).to(kv_cache.dtype)
         return pad(q).to(dt).contiguous()
 
-    def conv_rows(self, proj, bias, conv_w, taps: int, state, ctx, activation=None):
+    def conv_rows(self, proj, bias, conv_w, taps: int, state, ctx, activation=None, conv_bias=None):
         """``u = proj + bias`` rounded to the run dtype; ``y[t] = sum_j conv_w[j] * u[t - taps + 1 + j]`` per channel
         (``conv_w``: float32 ``[taps, channels]``; without taps ``y = u``), the rows before a segment's start from
         the request's state (``state[slot, phase]``: ``[taps - 1, channels]``, oldest first; zeros before the
         sequence's start), whose other half gets the last ``taps - 1`` rows of ``u``; ``activation = "silu"``:
-        ``y * sigmoid(y)``; ``[N, channels]`` rounded to the run dtype."""
+        ``y * sigmoid(y)``; ``[N, channels]`` rounded to the run dtype.  ``conv_bias`` (float32
+        ``[channels]``): what the sum over the taps starts from (``bias`` is part of ``u``, and of the state).  ``proj``
+        may be a view of wider rows."""
         dt = ctx.dtype
         u = proj.float() if bias is None else (proj.float() + bias.float())
         u = u.to(dt).float()
         y = u
         if taps:
-            y = torch.zeros_like(u)
+            y = torch.zeros_like(u) if conv_bias is None else conv_bias.float().expand_as(u).clone()
             cu = ctx.cu_seqlens.tolist()
             slots, phase = ctx.state_slots.tolist(), ctx.state_phase.tolist()
             w = conv_w.float()
@@ -373,6 +377,40 @@ class ReferenceOps:
         if gate is not None:
             d = d * torch.sigmoid(gate.float())
         return d.to(o.dtype)
+
+    def mamba2(self, proj, rows, dt_bias, a_log, skip, norm_weight, num_heads: int, value_dim: int, state_dim: int,
+               num_groups: int, norm_groups: int, eps: float, state, ctx):
+        """``proj``: ``[N, 2 H P + 2 G S + H]`` = gate z | (values x | write keys B | read keys C before their convolution) |
+        step sizes, run dtype; ``rows``: ``[N, H P + 2 G S]`` = x | B | C behind convolution and activation, run dtype.
+        Per head, with the B and C of its group, token by token from the request's memory (``state[slot, phase]``:
+        ``[H, S, P]``; the new one goes to ``state[slot, 1 - phase]``)::
+
+            d = softplus(dt + dt_bias);  M <- exp(-exp(a_log) d) M + d B x^T;  y = M^T C + skip x
+
+        then ``y * silu(z)`` divided by the root mean square (``eps``) of each of ``norm_groups`` equal parts, times
+        ``norm_weight``; ``[N, H P]`` in the run dtype."""
+        n = rows.shape[0]
+        H, P, S, G = num_heads, value_dim, state_dim, num_groups
+        inner = H * P
+        r = rows.float()
+        x = r[:, :inner].reshape(n, H, P)
+        B = r[:, inner: inner + G * S].reshape(n, G, S).repeat_interleave(H // G, dim=1)
+        C = r[:, inner + G * S:].reshape(n, G, S).repeat_interleave(H // G, dim=1)
+        d = torch.nn.functional.softplus(proj[:, proj.shape[1] - H:].float() + dt_bias.float())
+        decay = torch.exp(-torch.exp(a_log.float()) * d)
+        y = torch.empty(n, H, P, dtype=torch.float32, device=rows.device)
+        cu = ctx.cu_seqlens.tolist()
+        slots, phase = ctx.state_slots.tolist(), ctx.state_phase.tolist()
+        for s in range(len(cu) - 1):
+            M = state[slots[s], phase[s]].float().clone()
+            for t in range(cu[s], cu[s + 1]):
+                M = decay[t][:, None, None] * M + (d[t][:, None] * B[t])[:, :, None] * x[t][:, None, :]
+                y[t] = torch.einsum("hsp,hs->hp", M, C[t]) + skip.float()[:, None] * x[t]
+            state[slots[s], 1 - phase[s]] = M.to(state.dtype)
+        y = y.reshape(n, inner) * torch.nn.functional.silu(proj[:, :inner].float())
+        y = y.reshape(n, norm_groups, inner // norm_groups)
+        y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)
+        return (y.reshape(n, inner) * norm_weight.float()).to(rows.dtype)
 
     def gated_delta(self, rows, gates, a_log, dt_bias, norm_weight, out_gate, num_heads: int, num_kv_heads: int,
                     head_dim: int, value_dim: int, eps: float, floor: float, state, ctx):
@@ -454,8 +492,9 @@ class ReferenceOps:
         into their pages at ``slot = page * page_size + offset``."""
         n = rows.shape[0]
         H, dn, dr = num_heads, nope_dim, rope_dim
-        q = rows[:, : H * (dn + dr)].view(n, H, dn + dr)
-        q[:, :, dn:] = self._turn(q[:, :, dn:].float(), positions, rotation).to(rows.dtype)
+        if H:
+            q = rows[:, : H * (dn + dr)].view(n, H, dn + dr)
+            q[:, :, dn:] = self._turn(q[:, :, dn:].float(), positions, rotation).to(rows.dtype)
         if writes:
             c = rows[:, H * (dn + dr): H * (dn + dr) + kv_rank].float()
             c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps)
@@ -468,6 +507,24 @@ class ReferenceOps:
             rope_pages[page, off] = kr.to(rope_pages.dtype)
             if latent_t_pages is not None:  # a second copy, per page [kv_rank, page_size]
                 latent_t_pages.view(latent_t_pages.shape[0], kv_rank, ps)[page, :, off] = c.to(latent_t_pages.dtype)
+
+    def latent_down_prepare(self, rows, query_rank: int, query_norm, query_eps: float, rope_dim: int, kv_rank: int,
+                            positions, rotation, latent_norm, eps: float, latent_pages, rope_pages, slot_mapping,
+                            writes: bool, latent_t_pages=None):
+        """``rows``: ``[N, query_rank + kv_rank + rope (+ anything else)]``.  Returns the queries' latent (the first
+        ``query_rank`` numbers) RMS-normed with ``query_norm``, ``[N, query_rank]``; norms, turns and writes the
+        cached latent and the shared key part behind it as :meth:`latent_prepare` does."""
+        cq = rows[:, :query_rank].float()
+        cq = cq * torch.rsqrt(cq.pow(2).mean(-1, keepdim=True) + query_eps) * query_norm.float()
+        if writes:
+            self.latent_prepare(rows[:, query_rank:], 0, 0, rope_dim, kv_rank, positions, rotation, latent_norm, eps,
+                                latent_pages, rope_pages, slot_mapping, True, latent_t_pages)
+        return cq.to(rows.dtype)
+
+    def rotate_heads_(self, q, num_heads: int, nope_dim: int, rope_dim: int, positions, rotation) -> None:
+        """Turns the last ``rope_dim`` numbers of every head's query ``[unrotated, rotated]`` in place."""
+        v = q.view(q.shape[0], num_heads, nope_dim + rope_dim)
+        v[:, :, nope_dim:] = self._turn(v[:, :, nope_dim:].float(), positions, rotation).to(q.dtype)
 
     def latent_attention(self, q_lat, q, nope_dim: int, latent_pages, rope_pages, block_table, positions,
                          token_segment, window, scale: float, meta=None, latent_t_pages=None, sink=None):
@@ -594,11 +651,13 @@ class ReferenceOps:
         return self.paged_attention(q, kv_cache, block_table, positions, token_segment, retention, scale, meta)
 
     def paged_attention(self, q, kv_cache, block_table, positions, token_segment, retention, scale: float, meta=None,
-                        bias=None, sink=None):
+                        bias=None, sink=None, penalty=None):
         """For each token: softmax over the keys of its own request at positions
         ``[start(pos), pos]``, read from the pages its block table names.  ``bias``: float32 ``[Hq, L]``; a key ``n``
         places back adds ``bias[h, min(n, L - 1)]`` to head ``h``'s scaled score.  ``sink``: float32 ``[Hq]``;
-        ``exp(sink[h])`` is one more term of head ``h``'s denominator (no key, no value, not scaled, no bias)."""
+        ``exp(sink[h])`` is one more term of head ``h``'s denominator (no key, no value, not scaled, no bias).
+        ``penalty``: float32 ``[Hq, 2]``; ``penalty[h, 0] * ln(1 + penalty[h, 1] * n)`` is taken off head ``h``'s scaled
+        score of a key ``n`` places back."""
         n, hq, dh = q.shape
         hk, ps = kv_cache.shape[2], kv_cache.shape[3]
         g = hq // hk
@@ -624,6 +683,9 @@ class ReferenceOps:
             if bias is not None:
                 back = (p - kpos).clamp_max(bias.shape[1] - 1)
                 sc = sc + bias.float()[:, back].reshape(hk, g, -1)
+            if penalty is not None:
+                r1, r2 = penalty[:, :1].float(), penalty[:, 1:].float()
+                sc = sc - (r1 * torch.log1p(r2 * (p - kpos).float())).reshape(hk, g, -1)
             if sink is None:
                 pr = torch.softmax(sc, dim=-1)
             else:
@@ -673,15 +735,20 @@ class ReferenceOps:
             out += shared.float()
         return out
 
-    def moe_choose(self, h32, router, correction, top_k: int, groups=None, keep_groups=None, group_terms: int = 2):
-        """Router logits ``z`` in float32, scores ``s = sigmoid(z)``, choice scores ``c = s + correction``
+    def moe_choose(self, h32, router, correction, top_k: int, groups=None, keep_groups=None, group_terms: int = 2,
+                   scores: str = "sigmoid", normalize=None, weight_scale: float = 1.0, num_experts=None,
+                   extra_group: bool = False):
+        """Router logits ``z`` in float32, scores ``s = sigmoid(z)`` (``scores = "softmax"``: over all of the router's
+        rows), choice scores ``c = s + correction``
         (``correction``: float32 ``[E]`` or ``None``).  With ``groups``: the experts form that many equal groups of
         neighbours, a group's score is the sum of its ``group_terms`` largest ``c``, the ``keep_groups`` best groups
         (lowest index first among equals) stay and the others' experts cannot be chosen.  The ``top_k`` largest ``c``
-        among those that can, lowest index first among equals.  Returns ``(ids int32 [N, top_k], their s float32,
-        None)`` (the third: the grouping by expert that a kernel set may make in the same call)."""
+        among those that can, lowest index first among equals.  The weights are the chosen ``s``, with ``normalize``
+        divided by their sum plus that number, times ``weight_scale``.  Returns ``(ids int32 [N, top_k], weights
+        float32, None)`` (the third: the grouping by expert that a kernel set may make in the same call, of the first
+        ``num_experts`` of the router's rows)."""
         z = h32.float() @ router.float().t()
-        s = torch.sigmoid(z)
+        s = torch.softmax(z, dim=-1) if scores == "softmax" else torch.sigmoid(z)
         c = s if correction is None else s + correction.float()
         n, e = c.shape
         if groups is not None:
@@ -692,24 +759,37 @@ class ReferenceOps:
             allowed.scatter_(1, kept, True)
             c = c.masked_fill(~allowed.repeat_interleave(per, dim=1), float("-inf"))
         ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top_k]
-        return ids.to(torch.int32), torch.gather(s, 1, ids), None
+        w = torch.gather(s, 1, ids)
+        if normalize is not None:
+            w = w / (w.sum(dim=-1, keepdim=True) + normalize)
+        return ids.to(torch.int32), w * weight_scale, None
 
     def moe_experts_scored(self, h, expert_ids, weights, w_up, w_down, activation: str = "relu2", tiled: bool = False,
-                           grouping=None):
+                           grouping=None, shared_weights=None):
         """``sum_j weights[j] * W_down[e_j] act(W_up[e_j] h)`` per token, float32 result; ``w_up`` ``[E, F, D]``,
-        ``w_down`` ``[E, D, F]``; ``act = relu2``: the square of relu.  Activations between the two products and
+        ``w_down`` ``[E, D, F]``; ``act = relu2``: the square of relu.  ``swiglu``: ``w_up`` is ``[E, 2F, D]`` (gate
+        rows, then up rows) and ``act`` gives ``silu(gate) * up``.  A choice ``e_j >= E`` is an identity expert: its
+        output is ``h`` itself.  ``shared_weights``: a SwiGLU expert that is added unweighted.  Activations between the two products and
         every expert's weighted output are rounded to the run dtype, as the kernels store them."""
         assert not tiled, "the plain ops read row-major weights"
-        if activation != "relu2":
+        if activation not in ("relu2", "swiglu"):
             raise ValueError(f"unknown activation {activation!r}")
         n, d = h.shape
+        f = w_down.shape[2]
         out = torch.zeros(n, d, dtype=torch.float32, device=h.device)
         hf = h.float()
         for j in range(expert_ids.shape[1]):
             for e in torch.unique(expert_ids[:, j]).tolist():
                 rows = (expert_ids[:, j] == e).nonzero().squeeze(-1)
-                act = (torch.relu(hf[rows] @ w_up[e].float().t()) ** 2).to(h.dtype).float()
+                if e >= w_up.shape[0]:
+                    out[rows] += hf[rows] * weights[rows, j: j + 1].float()
+                    continue
+                up = hf[rows] @ w_up[e].float().t()
+                act = torch.relu(up) ** 2 if activation == "relu2" else torch.nn.functional.silu(up[:, :f]) * up[:, f:]
+                act = act.to(h.dtype).float()
                 out[rows] += ((act @ w_down[e].float().t()) * weights[rows, j: j + 1].float()).to(h.dtype).float()
+        if shared_weights is not None:
+            out += self.linear(self.swiglu_linear(h, shared_weights[0]), shared_weights[1]).float()
         return out
 
     # ------------------------------------------------------------------ sampling

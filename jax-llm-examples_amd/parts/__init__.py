@@ -1,4 +1,4 @@
-from . import (attention, embedding, feed_forward, gated_delta, latent_attention, mlstm, norm, position,  # noqa: F401
+from . import (attention, embedding, feed_forward, gated_delta, latent_attention, mamba2, mlstm, norm, position,  # noqa: F401
                side_by_side)  # noqa: F401  (register the built-in parts)
 from .base import (CacheNeed, Embedding, FeedForward, Mixer, Norm, OutputHead, ParamSpec, Part, PositionEncoding,
                    build_embedding, build_feed_forward, build_head, register_embedding, register_head,

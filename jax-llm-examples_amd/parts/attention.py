@@ -24,7 +24,10 @@ same values; with ``lam = exp(lq1 . lk1) - exp(lq2 . lk2) + diff`` from four lea
 ``a1 - lam a2``, divided by its root mean square and multiplied by ``1 - diff``; q and k rows lie head by head as
 ``[map 1, map 2]``), ``output_gate`` (the heads side by side times ``sigmoid(W_g h)`` before the output projection),
 a weighted q/k norm before the rotation together with a convolution, half-split pairs with a stretch, and the
-retention rule ``window_keep`` (a window plus the sequence's first tokens).  With any of these the projected rows go
+retention rule ``window_keep`` (a window plus the sequence's first tokens), ``head_temperature`` (a learned number per
+head that its scaled scores are multiplied by: it rides in the query norm's weight) and the ``distance_bias`` kind
+``log_distance`` (two learned numbers per head: ``r1 ln(1 + r2 n)`` is taken off the score of a key ``n`` places back;
+formed inside the attention kernels).  With any of these the projected rows go
 through ``conv_rows`` (bias, convolution, state), ``heads_prepare`` (norm, rotation, pages with filled-up heads; a
 value head written once per score map, so that the attention kernels see ``maps * kv_heads`` key/value heads, the
 queries re-ordered at load so that those of a key head lie together) and, for two maps, ``diff_combine``.  Formulas:
@@ -75,8 +78,12 @@ class Attention(Mixer):
         if self.qk_norm_span not in ("head", "projection"):
             raise ValueError(f"a q/k norm spans a head or the projection, not {self.qk_norm_span!r}")
         db = spec.get("distance_bias")
-        if db is not None and db.kind != "log_buckets":
+        if db is not None and db.kind not in ("log_buckets", "log_distance"):
             raise ValueError(f"unknown distance_bias kind {db.kind!r}")
+        self.log_distance = db is not None and db.kind == "log_distance"
+        if self.log_distance:
+            db = None  # (no table: two numbers per head)
+        self.head_temperature = bool(spec.get("head_temperature", False))
         self.bias_rows = None if db is None else int(db.rows)
         self.bias_max = None if db is None else int(db.max_distance)
         if db is not None and not 2 <= self.bias_rows // 2 < self.bias_max:
@@ -103,7 +110,8 @@ class Attention(Mixer):
         self.head_norm_eps = None if maps is None else float(maps.eps)
         self.output_gate = bool(spec.get("output_gate", False))
         # the path through conv_rows and heads_prepare (see the module's text)
-        self.general = (self.maps > 1 or self.output_gate or self.retention[0] == "window_keep"
+        self.general = (self.maps > 1 or self.output_gate or self.retention[0] == "window_keep" or self.log_distance
+                        or self.head_temperature
                         or (not self.spanned and (self.conv_taps > 0 or self.biased or self.value_dim != self.head_dim)
                             and (self.qk_norm_weighted or self.qk_norm_first
                                  or (rot is not None and rot.pairing != "adjacent"))))
@@ -117,6 +125,10 @@ class Attention(Mixer):
         if self.general and (self.spanned or self.query_scale is not None or self.qk_norm_span != "head"):
             raise ValueError("score maps, an output gate, the window_keep rule and a weighted norm with a convolution "
                              "come without a norm over the projection, a distance table, sinks and a query scale")
+        if self.log_distance and (self.maps > 1 or self.retention[0] == "window_keep"):
+            raise ValueError("a log_distance penalty comes without score maps and the window_keep rule")
+        if self.head_temperature and not (self.qk_norm_weighted and self.qk_norm_first and self.maps == 1):
+            raise ValueError("a head temperature comes with a weighted q/k norm before the rotation and one score map")
         # the path through the convolution kernel, which also rotates, norms, fills up and writes the pages
         self.convolved = not self.spanned and not self.general and (self.conv_taps > 0 or self.value_dim != self.head_dim or self.biased
                                                or (rot is not None and rot.magnitude != 1.0))
@@ -150,6 +162,11 @@ class Attention(Mixer):
             extra["conv"] = ParamSpec((channels, self.conv_taps), policy="float32", init=("normal", 0.6))
         if self.output_gate:
             extra["wg"] = ParamSpec((hq * dv, d), init=("normal", d ** -0.5))
+        if self.head_temperature:
+            extra["head_temp"] = ParamSpec((hq,), policy="float32", init=("uniform", 0.5, 1.5))
+        if self.log_distance:
+            extra["dist_mul"] = ParamSpec((hq,), policy="float32", init=("uniform", 0.0, 2.0))
+            extra["dist_rate"] = ParamSpec((hq,), policy="float32", init=("uniform", 0.05, 0.5))
         if self.maps > 1:
             for name in ("lam_q1", "lam_k1", "lam_q2", "lam_k2"):
                 extra[name] = ParamSpec((dh,), policy="float32", init=("normal", 0.3))
@@ -203,6 +220,11 @@ class Attention(Mixer):
         self.prep.rotation = rot
         self.prep.norm_weight_q = self.params.get("q_norm")
         self.prep.norm_weight_k = self.params.get("k_norm")
+        if self.head_temperature:  # (the score is linear in q: [heads, head_dim], a head's weights times its number)
+            self.prep.norm_weight_q = self.params["head_temp"][:, None] * self.params["q_norm"][None, :]
+        self.penalty = None
+        if self.log_distance:  # [heads, 2]
+            self.penalty = torch.stack([self.params["dist_mul"], self.params["dist_rate"]], dim=1).contiguous()
         self.prep.norm_span = self.qk_norm_span
         self.bias_run = None
         if self.biased:  # (the library's product adds a bias of its operands' dtype)
@@ -242,12 +264,14 @@ class Attention(Mixer):
             mp = self.maps
             proj, bias = ops.linear_bias(h, self.params["wqkv"], self.params.get("bqkv"), self.bias_run)
             gate = ops.linear(h, self.params["wg"]) if self.output_gate else None
-            rows = ops.conv_rows(proj, bias, self.conv_by_tap, self.conv_taps, cache.state, ctx)
+            rows = proj
+            if self.conv_taps or bias is not None or proj.dtype != ctx.dtype:
+                rows = ops.conv_rows(proj, bias, self.conv_by_tap, self.conv_taps, cache.state, ctx)
             q = ops.heads_prepare(rows, self.num_heads * mp, self.num_kv_heads * mp, self.num_kv_heads, self.head_dim,
                                   self.value_dim, self.page_dim, self.prep, ctx.positions,
                                   cache.kv if cache.writes else None, cache.slot_mapping)
             o = ops.paged_attention(q, cache.kv, cache.block_table, ctx.positions, ctx.token_segment, self.retention,
-                                    self.softmax_scale, cache.attn_meta)
+                                    self.softmax_scale, cache.attn_meta, penalty=self.penalty)
             if mp > 1:
                 o = ops.diff_combine(o, self.lam, 1.0 - self.diff, self.head_norm_eps, gate, self.num_heads,
                                      self.num_kv_heads, self.page_dim, self.value_dim)

@@ -259,7 +259,7 @@ class QKPreparation:
 
     rotation: Optional[Rotation] = None
     norm_eps: Optional[float] = None  # None: no norm
-    norm_weight_q: Optional[torch.Tensor] = None  # float32 [head_dim]; None: weightless
+    norm_weight_q: Optional[torch.Tensor] = None  # float32 [head_dim] or (one for every head) [heads, head_dim]; None: weightless
     norm_weight_k: Optional[torch.Tensor] = None
     norm_first: bool = False  # the norm comes before the rotation
     query_scale: Optional[tuple] = None  # (floor_scale, attn_scale): q *= 1 + attn_scale * ln(1 + floor((pos + 1) / floor_scale))

@@ -129,10 +129,17 @@ class MoEScored(FeedForward):
     s_e expert_e(h)`` with the scores as they are (no renormalisation).  With ``groups``: the experts form that many
     equal groups of neighbours, a group's score is the sum of its ``group_score_terms`` largest choice scores, and
     only experts of the ``keep_groups`` best groups can be chosen.  An expert is ``W_down act(W_up h)`` without
-    biases; ``activation``: ``relu2`` (the square of relu)."""
+    biases; ``activation``: ``relu2`` (the square of relu) or ``swiglu`` (``W_down (silu(W_gate h) * W_up h)``).
+    Further options: ``scores`` (``sigmoid`` or ``softmax``: over all of the router's rows), ``normalize`` (the chosen
+    scores are divided by their sum plus this number), ``weight_scale`` (then multiplied by it), ``identity_experts``
+    (so many more rows of the router, behind the experts': choosing one adds ``h`` itself, weighted; groups are formed
+    over experts and identity experts together) and ``shared_intermediate_size`` (a SwiGLU expert of that width whose
+    output every token gets, unweighted)."""
 
     wants_float32_input = True
     graph_safe = True
+    # (h and h32 go to the kernel set's router and expert products only)
+    accepts_deferred_norm = True
 
     def __init__(self, spec) -> None:
         super().__init__()
@@ -141,47 +148,64 @@ class MoEScored(FeedForward):
         self.top_k = int(spec.top_k)
         self.inter = int(spec.intermediate_size)
         self.activation = str(spec.get("activation") or "relu2")
-        if self.activation != "relu2":
-            raise ValueError(f"unknown activation {self.activation!r} (relu2)")
+        if self.activation not in ("relu2", "swiglu"):
+            raise ValueError(f"unknown activation {self.activation!r} (relu2, swiglu)")
+        self.scores = str(spec.get("scores") or "sigmoid")
+        if self.scores not in ("sigmoid", "softmax"):
+            raise ValueError(f"unknown scores {self.scores!r} (sigmoid, softmax)")
+        self.normalize = None if spec.get("normalize") is None else float(spec.normalize)
+        self.weight_scale = float(spec.get("weight_scale", 1.0))
+        self.identity = int(spec.get("identity_experts") or 0)
+        self.outputs = self.num_experts + self.identity
+        self.shared_inter = int(spec.get("shared_intermediate_size") or 0)
+        self.up_name = "w_gate_up" if self.activation == "swiglu" else "w_up"
         self.has_correction = bool(spec.get("correction", False))
         g = spec.get("groups")
         self.groups = None if g is None else int(g)
         self.keep_groups = None if g is None else int(spec.keep_groups)
         self.group_terms = int(spec.get("group_score_terms") or 2)
-        if self.groups is not None and (self.num_experts % self.groups or not 1 <= self.keep_groups <= self.groups
-                                        or self.keep_groups * (self.num_experts // self.groups) < self.top_k):
+        if self.groups is not None and (self.outputs % self.groups or not 1 <= self.keep_groups <= self.groups
+                                        or self.keep_groups * (self.outputs // self.groups) < self.top_k):
             raise ValueError("groups of equal size, 1 <= keep_groups <= groups, and top_k experts within the kept groups")
         self.tiled = False
 
     def param_specs(self):
         e, f, d = self.num_experts, self.inter, self.hidden
         specs = {
-            "router": ParamSpec((e, d), policy="float32", init=("normal", d ** -0.5)),
-            "w_up": ParamSpec((e, f, d), init=("normal", d ** -0.5)),  # per expert [out, in]
+            "router": ParamSpec((self.outputs, d), policy="float32", init=("normal", d ** -0.5)),
+            # per expert [out, in]; swiglu: gate rows, then up rows
+            self.up_name: ParamSpec((e, 2 * f if self.activation == "swiglu" else f, d), init=("normal", d ** -0.5)),
             "w_down": ParamSpec((e, d, f), init=("normal", f ** -0.5)),
         }
         if self.has_correction:
-            specs["correction"] = ParamSpec((e,), policy="float32", init=("normal", 0.3))
+            specs["correction"] = ParamSpec((self.outputs,), policy="float32", init=("normal", 0.3))
+        if self.shared_inter:
+            specs["shared_gate_up"] = ParamSpec((2 * self.shared_inter, d), init=("normal", d ** -0.5))
+            specs["shared_down"] = ParamSpec((d, self.shared_inter), init=("normal", self.shared_inter ** -0.5))
         return specs
 
     def step_weight_bytes(self, observed=None) -> int:
-        n = self.num_experts if observed is None else int(torch.unique(observed[0]).numel())
+        n = self.num_experts
+        if observed is not None:
+            n = int((torch.unique(observed[0]) < self.num_experts).sum())
         total = 0
         for name, t in self.params.items():
             b = t.numel() * t.element_size()
-            total += b // self.num_experts * n if name in ("w_up", "w_down") else b
+            total += b // self.num_experts * n if name in (self.up_name, "w_down") else b
         return total
 
     def flops_per_token(self) -> float:
+        """(With identity experts: as many of the chosen experts as their share of the router's rows.)"""
         per = 0
+        chosen = self.top_k * self.num_experts / self.outputs
         for name, t in self.params.items():
-            per += t.numel() // self.num_experts * self.top_k if name in ("w_up", "w_down") else t.numel()
+            per += t.numel() / self.num_experts * chosen if name in (self.up_name, "w_down") else t.numel()
         return 2.0 * per
 
     def finalize(self) -> None:
         from ..ops.layout import can_tile, tile_
 
-        up, dn = self.params["w_up"], self.params["w_down"]
+        up, dn = self.params[self.up_name], self.params["w_down"]
         if not self.tiled and can_tile(up) and can_tile(dn) and self.inter % 16 == 0:
             tile_(up)
             tile_(dn)
@@ -189,16 +213,21 @@ class MoEScored(FeedForward):
 
     def forward(self, h: torch.Tensor, h32: Optional[torch.Tensor], ctx) -> torch.Tensor:
         ops = ctx.ops
+        shared = (self.params["shared_gate_up"], self.params["shared_down"]) if self.shared_inter else None
         expert_ids, weights, grouping = ops.moe_choose(h32, self.params["router"], self.params.get("correction"),
-                                                       self.top_k, self.groups, self.keep_groups, self.group_terms)
+                                                       self.top_k, self.groups, self.keep_groups, self.group_terms,
+                                                       scores=self.scores, normalize=self.normalize,
+                                                       weight_scale=self.weight_scale, num_experts=self.num_experts,
+                                                       extra_group=shared is not None)
         tap = getattr(ctx, "tap", None)
         if tap is not None:  # whoever watches the step sees the choice and may replace it
             replaced = tap(self, "routing", (expert_ids, weights))
             if replaced is not None:
                 expert_ids, weights = replaced
                 grouping = None
-        return ops.moe_experts_scored(h, expert_ids, weights, self.params["w_up"], self.params["w_down"],
-                                      activation=self.activation, tiled=self.tiled, grouping=grouping)
+        return ops.moe_experts_scored(h, expert_ids, weights, self.params[self.up_name], self.params["w_down"],
+                                      activation=self.activation, tiled=self.tiled, grouping=grouping,
+                                      shared_weights=shared)
 
 
 @register_feed_forward("dense_polynorm")

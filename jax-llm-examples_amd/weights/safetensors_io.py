@@ -89,5 +89,5 @@ def write_safetensors(path: str, tensors: Iterable[tuple[str, torch.Tensor]], sp
         for (name, t), (sname, dt, shape) in zip(tensors, specs):
             assert name == sname and t.dtype == dt and tuple(t.shape) == tuple(shape), (name, sname)
             t = t.contiguous().cpu()
-            f.write(t.view(torch.uint8).numpy().tobytes() if t.numel() else b"")
+            f.write(t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")
     os.replace(tmp, path)
