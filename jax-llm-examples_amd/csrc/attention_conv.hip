@@ -1,6 +1,7 @@
 // Behind a fused q|k|v projection whose rows pass a short causal convolution over time before anything else:
 //     u[t]   = proj[t] + bias                                   (rounded to the run dtype: what the state keeps)
-//     y[t,c] = sum_j w[j, c] * u[t - taps + 1 + j, c]           (zeros before the sequence's start)
+//     y[t,c] = sum_j w[j, c] * u[t - taps + 1 + j, c]           (zeros before the sequence's start; conv_rows may start
+//                                                                the sum from a bias of the convolution's own)
 // then, per head, the rotation of q and k (adjacent pairs of the leading rotary_dim elements, sines and cosines
 // times a magnitude), their division by the root mean square over the head, and the write of k and v into their
 // page.  Queries and keys have dk elements a head, values dv; the pages (and the queries handed on) hold heads of
@@ -38,6 +39,8 @@ struct ConvArgs {
   float magnitude, norm_eps;  // norm_eps < 0: no norm
   int taps, C, Hq, Hkv, dk, dv, D, ps, rotary_dim;
   int act;  // (the convolution alone) 1: y * sigmoid(y) before the rounding
+  int ld;   // from one projected row to the next (C, or more where the rows are part of wider ones)
+  const float* conv_bias;  // (the convolution alone) [C] or null: what the sum over the taps starts from
 };
 
 __device__ __forceinline__ float conv_act(float y, int act) { return act == 1 ? y / (1.0f + expf(-y)) : y; }
@@ -45,7 +48,7 @@ __device__ __forceinline__ float conv_act(float y, int act) { return act == 1 ? 
 // the projected value of channel c in row `row`, with its bias, as the run dtype holds it
 template <typename PT, typename T>
 __device__ __forceinline__ float projected(const ConvArgs<PT, T>& a, size_t row, int c) {
-  float v = Num<PT>::load(a.proj + row * a.C + c);
+  float v = Num<PT>::load(a.proj + row * a.ld + c);
   if (a.bias != nullptr) v += a.bias[c];
   return Num<T>::round(v);
 }
@@ -183,7 +186,7 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(ConvArgs<PT, T> a, T* __
     const int t = n - a.cu_seqlens[seg];
     const T* old = nullptr;
     if (K > 1) old = a.state + ((size_t)a.state_slots[seg] * 2 + a.state_phase[seg]) * (K - 1) * a.C;
-    float acc = 0.f;
+    float acc = a.conv_bias != nullptr ? a.conv_bias[c] : 0.f;
     for (int j = 0; j < K; ++j) {  // (the same sum, in the same order, as conv_qk_prepare_kernel's)
       const int back = K - 1 - j;
       const float u = t - back >= 0 ? projected(a, (size_t)(n - back), c)
@@ -229,7 +232,7 @@ struct Row8<bf16_t> {
 
 template <typename PT, typename T>
 __device__ __forceinline__ void projected8(const ConvArgs<PT, T>& a, size_t row, int c, const float* bias8, float* u) {
-  Row8<PT>::load(a.proj + row * a.C + c, u);
+  Row8<PT>::load(a.proj + row * a.ld + c, u);
 #pragma unroll
   for (int i = 0; i < 8; ++i) u[i] = Num<T>::round(u[i] + bias8[i]);
 }
@@ -251,6 +254,10 @@ __global__ __launch_bounds__(256) void conv_rows_vec_kernel(ConvArgs<PT, T> a, T
 #pragma unroll
   for (int i = 0; i < 8; ++i) bias8[i] = 0.f;
   if (a.bias != nullptr) Row8<float>::load(a.bias + c, bias8);
+  float start8[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) start8[i] = 0.f;
+  if (a.conv_bias != nullptr) Row8<float>::load(a.conv_bias + c, start8);
   float u[8];
   if ((int)blockIdx.x >= token_blocks) {  // a segment's state
     if (K <= 1) return;
@@ -287,7 +294,7 @@ __global__ __launch_bounds__(256) void conv_rows_vec_kernel(ConvArgs<PT, T> a, T
       const T* old = nullptr;
       if (K > 1) old = a.state + ((size_t)a.state_slots[seg] * 2 + a.state_phase[seg]) * (K - 1) * a.C;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) y[i] = 0.f;
+      for (int i = 0; i < 8; ++i) y[i] = start8[i];
 #pragma unroll
       for (int j = 0; j < kTapsInRegisters; ++j) {  // (the taps ascending, as in every kernel of this file)
         if (j < K) {
@@ -316,8 +323,9 @@ __global__ __launch_bounds__(256) void conv_rows_vec_kernel(ConvArgs<PT, T> a, T
 
 template <typename PT, typename T>
 int launch_conv_rows(const ConvArgs<PT, T>& a, void* y_out, int N, int R, hipStream_t s) {
-  const uintptr_t all = (uintptr_t)a.proj | (uintptr_t)a.bias | (uintptr_t)a.w | (uintptr_t)a.state | (uintptr_t)y_out;
-  if (a.C % 8 == 0 && all % 16 == 0)  // (by the sizes alone: the same kernel for every step of a model)
+  const uintptr_t all = (uintptr_t)a.proj | (uintptr_t)a.bias | (uintptr_t)a.w | (uintptr_t)a.state | (uintptr_t)y_out |
+                        (uintptr_t)a.conv_bias;
+  if (a.C % 8 == 0 && a.ld % 8 == 0 && all % 16 == 0)  // (by the sizes alone: the same kernel for every step of a model)
   {
     const int per = N >= 512 ? kRowsPerBlock : 1;
     const int token_blocks = (N + per - 1) / per;
@@ -368,7 +376,7 @@ JLE_API int jle_conv_qk_prepare(const void* proj, int proj_f32, const float* bia
 #define JLE_CONV_ARGS(PT, T)                                                                                        \
   ConvArgs<PT, T> a{(const PT*)proj, bias, conv_w, (T*)state, token_segment, cu_seqlens, state_slots, state_phase, \
                     positions, slot_mapping, inv_freq, (T*)q_out, (T*)kv_cache, magnitude, norm_eps, taps, C, Hq,  \
-                    Hkv, dk, dv, D, ps, rotary_dim}
+                    Hkv, dk, dv, D, ps, rotary_dim, 0, C, nullptr}
   if (!is_bf16) {
     JLE_CONV_ARGS(float, float);
     return launch_conv(a, N, R, s);
@@ -382,19 +390,23 @@ JLE_API int jle_conv_qk_prepare(const void* proj, int proj_f32, const float* bia
 #undef JLE_CONV_ARGS
 }
 
-// The convolution alone: y [N, C] in the run dtype, C channels of any meaning; the state as above.
-static int conv_rows_act(const void* proj, int proj_f32, const float* bias, const float* conv_w, int taps,
-                         void* state, const int* token_segment, const int* cu_seqlens, const int* state_slots,
-                         const int* state_phase, void* y_out, int is_bf16, int N, int R, int C, int act, hipStream_t s) {
+// The convolution alone: y [N, C] in the run dtype, C channels of any meaning, the state as above.  ld: from one
+// projected row to the next (C, or more where the rows are part of wider ones); conv_bias: [C] or null, what the sum
+// over the taps starts from; act 1: y * sigmoid(y) on the result, float32, before the rounding.
+JLE_API int jle_conv_rows(const void* proj, int proj_f32, int ld, const float* bias, const float* conv_w,
+                          const float* conv_bias, int taps, void* state, const int* token_segment, const int* cu_seqlens,
+                          const int* state_slots, const int* state_phase, void* y_out, int is_bf16, int N, int R, int C,
+                          int act, hipStream_t s) {
   if (N <= 0) return 0;
-  if (act < 0 || act > 1) return JLE_BAD_ARG;
+  if (act < 0 || act > 1 || ld < C || (conv_bias != nullptr && taps < 1)) return JLE_BAD_ARG;
   if (C <= 0 || taps < 0 || R <= 0 || (C + 255) / 256 > 65535 || y_out == nullptr) return JLE_BAD_ARG;
   if ((taps > 0 && conv_w == nullptr) || (taps > 1 && (state == nullptr || state_slots == nullptr || state_phase == nullptr)))
     return JLE_BAD_ARG;
   if (!is_bf16 && !proj_f32) return JLE_BAD_ARG;
 #define JLE_ROWS_ARGS(PT, T)                                                                                        \
   ConvArgs<PT, T> a{(const PT*)proj, bias, conv_w, (T*)state, token_segment, cu_seqlens, state_slots, state_phase, \
-                    nullptr, nullptr, nullptr, nullptr, nullptr, 1.f, -1.f, taps, C, 0, 0, 0, 0, 0, 0, 0, act}
+                    nullptr, nullptr, nullptr, nullptr, nullptr, 1.f, -1.f, taps, C, 0, 0, 0, 0, 0, 0, 0, act,      \
+                    ld, conv_bias}
   if (!is_bf16) {
     JLE_ROWS_ARGS(float, float);
     return launch_conv_rows(a, y_out, N, R, s);
@@ -406,20 +418,4 @@ static int conv_rows_act(const void* proj, int proj_f32, const float* bias, cons
   JLE_ROWS_ARGS(bf16_t, bf16_t);
   return launch_conv_rows(a, y_out, N, R, s);
 #undef JLE_ROWS_ARGS
-}
-
-JLE_API int jle_conv_rows(const void* proj, int proj_f32, const float* bias, const float* conv_w, int taps,
-                          void* state, const int* token_segment, const int* cu_seqlens, const int* state_slots,
-                          const int* state_phase, void* y_out, int is_bf16, int N, int R, int C, hipStream_t s) {
-  return conv_rows_act(proj, proj_f32, bias, conv_w, taps, state, token_segment, cu_seqlens, state_slots, state_phase,
-                       y_out, is_bf16, N, R, C, 0, s);
-}
-
-// The same with an activation on the convolution's result (act 1: y * sigmoid(y), float32, before the rounding).
-JLE_API int jle_conv_rows_act(const void* proj, int proj_f32, const float* bias, const float* conv_w, int taps,
-                              void* state, const int* token_segment, const int* cu_seqlens, const int* state_slots,
-                              const int* state_phase, void* y_out, int is_bf16, int N, int R, int C, int act,
-                              hipStream_t s) {
-  return conv_rows_act(proj, proj_f32, bias, conv_w, taps, state, token_segment, cu_seqlens, state_slots, state_phase,
-                       y_out, is_bf16, N, R, C, act, s);
 }

@@ -101,7 +101,9 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
         }
         s = dot * scale;
         // a learned number per head and distance; every key further back than the table is long takes its last entry
-        if (bias != nullptr) s += bias[(size_t)h * bias_len + min(pos - key, bias_len - 1)];
+        // (a negative length: a penalty that grows with the distance, two numbers per head)
+        if (bias_len < 0) s -= bias[2 * h] * log1pf(bias[2 * h + 1] * (float)(pos - key));
+        else if (bias != nullptr) s += bias[(size_t)h * bias_len + min(pos - key, bias_len - 1)];
       }
     }
     const float m_new = fmaxf(m, wave_max(s));
@@ -251,7 +253,7 @@ __global__ __launch_bounds__(256) void paged_attention_generic_merge_kernel(cons
 // tiles_per_split tiles of 64 keys each, and merged by a second kernel; ws_ml: [N * Hq * splits * 2] float32,
 // ws_o: [N * Hq * splits * dh] float32.  splits * tiles_per_split must cover the longest range of keys.
 // bias: float32 [Hq][bias_len] or null: a key n places back adds bias[h][min(n, bias_len - 1)] to head h's scaled
-// score; sink: float32 [Hq] or null: exp(sink[h]) is one more term of head h's denominator.
+// score (bias_len < 0: bias is [Hq][2], and bias[h][0] * ln(1 + bias[h][1] * n) is taken off it); sink: float32 [Hq] or null: exp(sink[h]) is one more term of head h's denominator.
 static int launch_generic(const void* q, const void* kv, void* out, const int* positions, const int* token_segment,
                           const int* block_table, int table_width, int ret_mode, int ret_param, float scale,
                           int is_bf16, int N, int Hq, int Hkv, int dh, int ps, int splits, int tiles_per_split,
@@ -259,7 +261,7 @@ static int launch_generic(const void* q, const void* kv, void* out, const int* p
                           hipStream_t s, int keep = 0) {
   if (N <= 0) return 0;
   if (keep < 0) return JLE_BAD_ARG;
-  if (bias != nullptr && bias_len < 1) return JLE_BAD_ARG;
+  if ((bias == nullptr) != (bias_len == 0)) return JLE_BAD_ARG;
   if (dh % 8 || dh > 256 || Hkv <= 0 || Hq % Hkv || ps <= 0) return JLE_BAD_ARG;
   if ((ret_mode == 1 || ret_mode == 2) && ret_param <= 0) return JLE_BAD_ARG;
   if (splits < 1 || (splits > 1 && (tiles_per_split < 1 || ws_ml == nullptr || ws_o == nullptr))) return JLE_BAD_ARG;

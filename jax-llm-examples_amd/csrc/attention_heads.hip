@@ -23,12 +23,13 @@ struct HeadsArgs {
   const int* positions;
   const int* slot_mapping;
   const float* inv_freq;  // [rotary_dim / 2] or null
-  const float* wq;        // [dk] or null
+  const float* wq;        // [dk], or [Hq][dk] (wq_stride = dk), or null
   const float* wk;
   T* q_out;
   T* kv_cache;  // or null
   float magnitude, norm_eps;  // norm_eps < 0: no norm
   int rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps;
+  int wq_stride;  // from one query head's norm weights to the next's (0: one for all)
 };
 
 template <typename T>
@@ -48,7 +49,7 @@ __global__ __launch_bounds__(64) void heads_prepare_kernel(HeadsArgs<T> a) {
     x[i] = e < dim ? Num<T>::load(src + e) : 0.f;
   }
   if (!is_v) {
-    const float* w = is_q ? a.wq : a.wk;
+    const float* w = is_q ? (a.wq == nullptr ? nullptr : a.wq + (size_t)h * a.wq_stride) : a.wk;
     if (a.norm_eps >= 0.f && a.norm_first) {
       float ss = 0.f;
 #pragma unroll
@@ -160,7 +161,7 @@ __global__ __launch_bounds__(64) void diff_combine_kernel(const T* __restrict__ 
 
 JLE_API int jle_heads_prepare(const void* rows, const int* positions, const int* slot_mapping, const float* inv_freq,
                               int rotary_dim, int half_pairs, float magnitude, float norm_eps, int norm_first,
-                              const float* wq, const float* wk, void* q_out, void* kv_cache, int is_bf16, int N, int Hq,
+                              const float* wq, int wq_stride, const float* wk, void* q_out, void* kv_cache, int is_bf16, int N, int Hq,
                               int Hk, int Hv, int dk, int dv, int D, int ps, hipStream_t s) {
   if (N <= 0) return 0;
   if (rows == nullptr || q_out == nullptr || Hq <= 0 || Hk <= 0 || Hv <= 0 || Hk % Hv || dk <= 0 || dv <= 0 ||
@@ -169,14 +170,15 @@ JLE_API int jle_heads_prepare(const void* rows, const int* positions, const int*
   if (rotary_dim < 0 || rotary_dim % 2 || rotary_dim > dk || (rotary_dim > 0 && (inv_freq == nullptr || positions == nullptr)))
     return JLE_BAD_ARG;
   if (kv_cache != nullptr && slot_mapping == nullptr) return JLE_BAD_ARG;
+  if (wq_stride != 0 && wq_stride != dk) return JLE_BAD_ARG;
   const dim3 grid(N, Hq + Hk + Hv);
   if (is_bf16) {
     HeadsArgs<bf16_t> a{(const bf16_t*)rows, positions, slot_mapping, inv_freq, wq, wk, (bf16_t*)q_out, (bf16_t*)kv_cache,
-                        magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps};
+                        magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, wq_stride};
     hipLaunchKernelGGL(heads_prepare_kernel<bf16_t>, grid, dim3(64), 0, s, a);
   } else {
     HeadsArgs<float> a{(const float*)rows, positions, slot_mapping, inv_freq, wq, wk, (float*)q_out, (float*)kv_cache,
-                       magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps};
+                       magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, wq_stride};
     hipLaunchKernelGGL(heads_prepare_kernel<float>, grid, dim3(64), 0, s, a);
   }
   JLE_LAUNCH_CHECK();

@@ -58,9 +58,22 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(T* __restrict__ row
                                                              const float* __restrict__ norm_w, float eps,
                                                              T* __restrict__ latent_pages, T* __restrict__ rope_pages,
                                                              T* __restrict__ latent_t_pages, int ps,
-                                                             const int* __restrict__ slot_mapping, int writes) {
+                                                             const int* __restrict__ slot_mapping, int writes,
+                                                             int QR = 0, const float* __restrict__ qnorm_w = nullptr,
+                                                             float q_eps = 0.f, T* __restrict__ cq = nullptr) {
+  // QR > 0: a row begins with QR numbers of the queries' own latent, normed into cq (and H is 0)
   __shared__ float red[4];
   const size_t n = blockIdx.x;
+  if (QR > 0) {
+    const T* c = rows + n * ld;
+    float ss = 0.f;
+    for (int d = threadIdx.x; d < QR; d += 256) {
+      const float v = Num<T>::load(c + d);
+      ss = __builtin_fmaf(v, v, ss);
+    }
+    const float inv = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)QR + q_eps);
+    for (int d = threadIdx.x; d < QR; d += 256) Num<T>::store(cq + n * QR + d, Num<T>::load(c + d) * inv * qnorm_w[d]);
+  }
   T* row = rows + n * ld;
   const float pos = (float)positions[n];
   const int half = rd / 2;
@@ -79,7 +92,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(T* __restrict__ row
     Num<T>::store(q + ib, v * cs + u * sn);
   }
   if (!writes) return;
-  const T* c = row + (size_t)H * (dn + dr);
+  const T* c = row + (size_t)H * (dn + dr) + QR;
   const T* kr = c + R;
   float ss = 0.f;
   for (int d = threadIdx.x; d < R; d += 256) {
@@ -842,6 +855,31 @@ JLE_API int jle_latent_prepare(void* rows, int ld, int H, int dn, int dr, int R,
     hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(N), dim3(256), 0, s, (float*)rows, ld, H, dn, dr, R,
                        positions, inv_freq, pairing, rd, magnitude, norm_w, eps, (float*)latent_pages, (float*)rope_pages,
                        (float*)latent_t_pages, ps, slot_mapping, writes);
+  JLE_LAUNCH_CHECK();
+  return 0;
+}
+
+// The rows' first QR numbers are the queries' latent: normed with qnorm_w into cq [N, QR]; the cached latent and the
+// shared key part behind it are normed, turned and written into their pages as by jle_latent_prepare.
+JLE_API int jle_latent_down_prepare(void* rows, int ld, int QR, const float* qnorm_w, float q_eps, void* cq, int dr, int R,
+                                    const int* positions, const float* inv_freq, int pairing, int rd, float magnitude,
+                                    const float* norm_w, float eps, void* latent_pages, void* rope_pages,
+                                    void* latent_t_pages, int ps, const int* slot_mapping, int writes, int is_bf16, int N,
+                                    hipStream_t s) {
+  if (N <= 0) return 0;
+  if (QR <= 0 || qnorm_w == nullptr || cq == nullptr || dr <= 0 || R <= 0 || rd % 2 || rd < 0 || rd > dr ||
+      (rd > 0 && inv_freq == nullptr) || ld < QR + (writes ? R + dr : 0))
+    return JLE_BAD_ARG;
+  if (writes && (latent_pages == nullptr || rope_pages == nullptr || slot_mapping == nullptr || ps <= 0))
+    return JLE_BAD_ARG;
+  if (is_bf16)
+    hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, dim3(N), dim3(256), 0, s, (bf16_t*)rows, ld, 0, 0, dr, R, positions,
+                       inv_freq, pairing, rd, magnitude, norm_w, eps, (bf16_t*)latent_pages, (bf16_t*)rope_pages,
+                       (bf16_t*)latent_t_pages, ps, slot_mapping, writes, QR, qnorm_w, q_eps, (bf16_t*)cq);
+  else
+    hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(N), dim3(256), 0, s, (float*)rows, ld, 0, 0, dr, R, positions,
+                       inv_freq, pairing, rd, magnitude, norm_w, eps, (float*)latent_pages, (float*)rope_pages,
+                       (float*)latent_t_pages, ps, slot_mapping, writes, QR, qnorm_w, q_eps, (float*)cq);
   JLE_LAUNCH_CHECK();
   return 0;
 }

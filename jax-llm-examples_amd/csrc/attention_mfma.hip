@@ -52,10 +52,17 @@ struct Columns {  // per lane, for each of its column tiles
 };
 
 // A learned number per (query head, distance) added to the scaled score: table[h][min(pos - key, L - 1)], float32.
+// Or (L < 0) a penalty that grows with the distance: table[h] = (r1, r2), r1 ln(1 + r2 (pos - key)) taken off.
 struct Biasing {
   const float* table;
   int L;
 };
+constexpr int kNoBias = 0, kBiasTable = 1, kBiasPenalty = 2;  // what a kernel is compiled for
+
+// the penalty in the exponent's base-2 units: r1 ln(x) log2(e) = r1 log2(x)
+__device__ __forceinline__ float penalty_log2(float r1, float r2, float back) {
+  return r1 * __builtin_amdgcn_logf(fmaf(r2, back, 1.0f));
+}
 
 // Maximum / sum over the four lanes that hold one column (equal lane % 16), in all of them.  The two swaps
 // exchange the halves of the wavefront and neighbouring rows of 16 lanes: no trip through shared memory.
@@ -84,11 +91,12 @@ __device__ __forceinline__ float column_sum(float v) {
 //   st[ct][tt]: scores of key tile tt (keys kb + 16 tt + 4 g + i in element i); act0 / act1: the tile exists
 //   vraw[dt]: for element row 16 dt + (lane % 16): keys 4 g .. 4 g + 3 of tile 0 (x, y) and of tile 1 (z, w)
 //   l: each lane's own part of the column's sum (column_sum at the end gives the whole)
-//   BIASED: a distance bias is added to every scaled score (far: every key of the step is so far behind every
+//   BIASED (kBiasTable): a distance bias is added to every scaled score (far: every key of the step is so far behind every
 //   live column that the table's last entry holds, far_b[ct], already in the exponent's base-2 units), and the
 //   probabilities enter the second product as two bfloat16 terms (leading part and remainder) instead of one
-//   rounded term, which keeps about 16 bits of them.
-template <int DH, int CT, bool MASKED, typename V4, bool BIASED = false>
+//   rounded term, which keeps about 16 bits of them.  kBiasPenalty: the penalty is taken off every scaled score
+//   (far_b[ct] = r1, far_b[CT + ct] = r2), one rounded term.
+template <int DH, int CT, bool MASKED, typename V4, int BIASED = kNoBias>
 __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], bool act0, bool act1,
                                                    const V4 (&vraw)[DH / 16], int kb, const Columns (&col)[CT],
                                                    int k_lo, int k_hi, float scale_log2, float (&m)[CT],
@@ -99,7 +107,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
   const int g = (threadIdx.x & 63) >> 4;
   const float sc = BIASED ? 1.0f : scale_log2;  // (biased scores are scaled where the bias is added)
   bf16x8 pb[CT];
-  bf16x8 pb_lo[BIASED ? CT : 1];
+  bf16x8 pb_lo[BIASED == kBiasTable ? CT : 1];
   float corr[CT];
   bool unchanged = true;
 #pragma unroll
@@ -111,7 +119,9 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         float v = st[ct][tt][i];
-        if (BIASED) {
+        if (BIASED == kBiasPenalty)
+          v = fmaf(v, scale_log2, -penalty_log2(far_b[ct], far_b[CT + ct], (float)(col[ct].pos - kb - 4 * g) - (float)(16 * tt + i)));
+        if (BIASED == kBiasTable) {
           float b = far_b[ct];
           if (!far) {
             const int back = col[ct].pos - (kb + 16 * tt + 4 * g + i);
@@ -143,7 +153,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
     m[ct] = m_new;
     const uint4 pk = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]), pack_bf16(p[6], p[7])};
     pb[ct] = __builtin_bit_cast(bf16x8, pk);
-    if (BIASED) {  // what the rounding left out, as a second term
+    if (BIASED == kBiasTable) {  // what the rounding left out, as a second term
       float r[8];
 #pragma unroll
       for (int j = 0; j < 8; j += 2) {
@@ -190,7 +200,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
       const bf16x8 a = __builtin_bit_cast(bf16x8, vv);
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
-        if (BIASED) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct], acc[ct][dt], 0, 0, 0);
+        if (BIASED == kBiasTable) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct], acc[ct][dt], 0, 0, 0);
         acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[ct], acc[ct][dt], 0, 0, 0);
       }
     }
@@ -200,7 +210,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
       const bf16x8 a = __builtin_bit_cast(bf16x8, vraw[dt]);
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
-        if (BIASED) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct], acc[ct][dt], 0, 0, 0);
+        if (BIASED == kBiasTable) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct], acc[ct][dt], 0, 0, 0);
         acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[ct], acc[ct][dt], 0, 0, 0);
       }
     }
@@ -252,7 +262,7 @@ __device__ __forceinline__ void load_queries(const bf16_t* __restrict__ q, const
   }
 }
 
-template <int DH, int CT, bool ONCE, bool BIASED = false>
+template <int DH, int CT, bool ONCE, int BIASED = kNoBias>
 __device__ __forceinline__ void attend_with(const bf16x8 (&qb)[CT][DH / 32], const bf16_t* __restrict__ kv,
                                             const int* __restrict__ table, const Columns (&col)[CT], int k_lo,
                                             int k_hi, int hk, int Hkv, int ps, float scale_log2, float (&m)[CT],
@@ -345,9 +355,17 @@ __device__ __forceinline__ void attend_with(const bf16x8 (&qb)[CT][DH / 32], con
   common_range<CT>(col, all_lo, all_hi);
   // with a distance bias: the table's last entry per column, and the last key that is that far behind every
   // live column of the wavefront
-  float far_b[CT];
+  // (with a penalty: its two numbers per column)
+  float far_b[2 * CT];
   int far_until = INT_MIN;
-  if (BIASED) {
+  if (BIASED == kBiasPenalty) {
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+      far_b[ct] = bias.table[2 * col[ct].head];
+      far_b[CT + ct] = bias.table[2 * col[ct].head + 1];
+    }
+  }
+  if (BIASED == kBiasTable) {
     int min_pos = INT_MAX;
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
@@ -384,10 +402,10 @@ __device__ __forceinline__ void attend_with(const bf16x8 (&qb)[CT][DH / 32], con
     if (BIASED) {
       const bool far = kb + 31 <= far_until;
       if (__all(act0 && act1 && kb >= all_lo && kb + 31 <= all_hi))
-        softmax_and_values<DH, CT, false, u32x4, true>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l,
+        softmax_and_values<DH, CT, false, u32x4, BIASED>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l,
                                                        acc, bias, far, far_b);
       else
-        softmax_and_values<DH, CT, true, u32x4, true>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l,
+        softmax_and_values<DH, CT, true, u32x4, BIASED>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l,
                                                       acc, bias, far, far_b);
       continue;
     }
@@ -402,7 +420,7 @@ __device__ __forceinline__ void attend_with(const bf16x8 (&qb)[CT][DH / 32], con
   }
 }
 
-template <int DH, int CT, bool ONCE, bool BIASED = false>
+template <int DH, int CT, bool ONCE, int BIASED = kNoBias>
 __device__ __forceinline__ void attend(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv,
                                        const int* __restrict__ table, const Columns (&col)[CT], int k_lo, int k_hi,
                                        int hk, int Hq, int Hkv, int ps, float scale_log2, float (&m)[CT],
@@ -420,7 +438,7 @@ __device__ __forceinline__ void attend(const bf16_t* __restrict__ q, const bf16_
 // (launch bounds: with one column tile and head sizes up to 128 the registers are held to what lets two wavefronts share a SIMD)
 // BIASED: a distance bias (see Biasing) on every score and, with `sink`, one more term exp(sink[h]) in head h's
 // denominator.
-template <int DH, int CT, bool BIASED = false>
+template <int DH, int CT, int BIASED = kNoBias>
 __global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && !BIASED) ? 2 : 1) void attention_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, bf16_t* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
@@ -807,7 +825,7 @@ __device__ __forceinline__ void load_to_lds16(const void* base, uint32_t byte_of
 // half h are those of keys 8 g .. 8 g + 7, and the values are read half by half as one 16-byte piece per element
 // (sv points at the step's value tiles, v_rd is the lane's offset in a tile, tile_bytes the distance between
 // tiles).  halves: 1 if the second half holds nothing for this wavefront.
-template <int DH, int CT, bool MASKED, bool BIASED = false>
+template <int DH, int CT, bool MASKED, int BIASED = kNoBias>
 __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int halves,
                                                      const unsigned char* sv, uint32_t v_rd, int tile_bytes, int kb,
                                                      const Columns (&col)[CT], int k_lo, int k_hi, float scale_log2,
@@ -818,7 +836,7 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
   const int g = (threadIdx.x & 63) >> 4;
   const float sc = BIASED ? 1.0f : scale_log2;  // (biased scores are scaled where the bias is added)
   bf16x8 pb[CT][2];
-  bf16x8 pb_lo[BIASED ? CT : 1][2];  // (see softmax_and_values)
+  bf16x8 pb_lo[BIASED == kBiasTable ? CT : 1][2];  // (see softmax_and_values)
   float corr[CT];
   bool unchanged = true;
 #pragma unroll
@@ -829,7 +847,12 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         float v = st[ct][tt][i];
-        if (BIASED) {
+        if (BIASED == kBiasPenalty) {
+          v = fmaf(v, scale_log2, -penalty_log2(far_b[ct], far_b[CT + ct], (float)(col[ct].pos - kb - 8 * g) -
+                                                                               (float)(32 * (tt >> 1) + 4 * (tt & 1) + i)));
+          st[ct][tt][i] = v;
+        }
+        if (BIASED == kBiasTable) {
           float b = far_b[ct];
           if (!far) {
             const int back = col[ct].pos - (kb + 32 * (tt >> 1) + 8 * g + 4 * (tt & 1) + i);
@@ -862,7 +885,7 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
       }
       const uint4 pk = {pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]), pack_bf16(p[4], p[5]), pack_bf16(p[6], p[7])};
       pb[ct][hf] = __builtin_bit_cast(bf16x8, pk);
-      if (BIASED) {  // what the rounding left out, as a second term
+      if (BIASED == kBiasTable) {  // what the rounding left out, as a second term
         float r[8];
 #pragma unroll
         for (int j = 0; j < 8; j += 2) {
@@ -921,7 +944,7 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
       const bf16x8 a = __builtin_bit_cast(bf16x8, vraw[dt]);
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
-        if (BIASED) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct][hf], acc[ct][dt], 0, 0, 0);
+        if (BIASED == kBiasTable) acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb_lo[ct][hf], acc[ct][dt], 0, 0, 0);
         acc[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[ct][hf], acc[ct][dt], 0, 0, 0);
       }
     }
@@ -930,7 +953,7 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
 
 // BIASED: a distance bias on every score and, with `sink`, one more term in every head's denominator (two blocks a
 // compute unit all the same: 86 us against 99 with one, at 2,048 tokens, 16 heads on 8 kv heads).
-template <bool BIASED>
+template <int BIASED>
 __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, bf16_t* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
@@ -995,9 +1018,16 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
   }
   int all_lo, all_hi;
   common_range<CT>(col, all_lo, all_hi);
-  float far_b[CT];         // with a distance bias: the table's last entry, and the last key that is that far behind
+  float far_b[2 * CT];     // with a distance bias: the table's last entry, and the last key that is that far behind
   int far_until = INT_MIN;  // every live column of the wavefront (its columns' positions ascend: the first is the least)
-  if (BIASED) {
+  if (BIASED == kBiasPenalty) {
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+      far_b[ct] = bias.table[2 * h];
+      far_b[CT + ct] = bias.table[2 * h + 1];
+    }
+  }
+  if (BIASED == kBiasTable) {
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) far_b[ct] = bias.table[(size_t)h * bias.L + bias.L - 1] * kLog2e;
     far_until = p_first - (bias.L - 1);
@@ -1103,10 +1133,10 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
       if (BIASED) {
         const bool far = kb + 63 <= far_until;
         if (kb >= all_lo && kb + 63 <= all_hi)
-          softmax64_and_values<DH, CT, false, true>(st, 2, sb + 4 * TILE, v_rd, TILE, kb, col, k_lo, k_hi, scale_log2, m,
+          softmax64_and_values<DH, CT, false, BIASED>(st, 2, sb + 4 * TILE, v_rd, TILE, kb, col, k_lo, k_hi, scale_log2, m,
                                                     l, acc, bias, far, far_b);
         else
-          softmax64_and_values<DH, CT, true, true>(st, halves, sb + 4 * TILE, v_rd, TILE, kb, col, k_lo, k_hi,
+          softmax64_and_values<DH, CT, true, BIASED>(st, halves, sb + 4 * TILE, v_rd, TILE, kb, col, k_lo, k_hi,
                                                    scale_log2, m, l, acc, bias, far, far_b);
       } else if (kb >= all_lo && kb + 63 <= all_hi)  // the same for the whole wavefront
         softmax64_and_values<DH, CT, false>(st, 2, sb + 4 * TILE, v_rd, TILE, kb, col, k_lo, k_hi, scale_log2, m, l, acc);
@@ -1140,7 +1170,7 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
 // dec_tokens: [num_dec] rows of q that are single decode tokens.  One wavefront per
 // (decode token, kv head, key range); ws_ml: [item][16 * CT][2], ws_o: [item][16 * CT][DH],
 // item = (d * Hkv + hk) * max_splits + split.
-template <int DH, int CT, bool BIASED = false>
+template <int DH, int CT, int BIASED = kNoBias>
 __global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && !BIASED) ? 2 : 1) void attention_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, float* __restrict__ ws_ml, float* __restrict__ ws_o,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
@@ -1557,7 +1587,7 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
                                   int bias_len, const float* sink, hipStream_t s) {
   if (num_tiles <= 0) return 0;
   if (!jle_attention_mfma_supported(dh, Hq, Hkv, ps)) return JLE_BAD_ARG;
-  // bias: [Hq][bias_len] (with a sink and no bias: a table of zeros); the kernels that share keys take neither
+  // bias: [Hq][bias_len] (with a sink and no bias: a table of zeros), or bias_len < 0: a penalty's [Hq][2]; the kernels that share keys take neither
   if ((bias == nullptr) != (bias_len == 0) || (sink != nullptr && bias == nullptr)) return JLE_BAD_ARG;
   if (bias != nullptr && groups != nullptr && dh != 128) return JLE_BAD_ARG;  // (of those, the kernel for 128 alone)
   const Biasing bs = {bias, bias_len};
@@ -1579,12 +1609,16 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
       case 64: PICK_S(64); break;
       case 96: PICK_S(96); break;
       case 128:  // (the kernel whose loads go straight into shared memory)
-        if (bias != nullptr)
-          hipLaunchKernelGGL(attention_prefill_lds_kernel<true>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
+        if (bias_len < 0)
+          hipLaunchKernelGGL(attention_prefill_lds_kernel<kBiasPenalty>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
+                             (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,
+                             groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink);
+        else if (bias != nullptr)
+          hipLaunchKernelGGL(attention_prefill_lds_kernel<kBiasTable>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
                              (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,
                              groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink);
         else
-          hipLaunchKernelGGL(attention_prefill_lds_kernel<false>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
+          hipLaunchKernelGGL(attention_prefill_lds_kernel<kNoBias>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
                              (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,
                              groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink);
         break;
@@ -1602,11 +1636,13 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
 #define LAUNCH(DH)                                                                                                   \
   do {                                                                                                               \
     if (tile_tokens == 32) {                                                                                         \
-      if (bias != nullptr) LAUNCH_B(DH, 2, true);                                                                    \
-      else LAUNCH_B(DH, 2, false);                                                                                   \
+      if (bias_len < 0) LAUNCH_B(DH, 2, kBiasPenalty);                                                               \
+      else if (bias != nullptr) LAUNCH_B(DH, 2, kBiasTable);                                                         \
+      else LAUNCH_B(DH, 2, kNoBias);                                                                                 \
     } else {                                                                                                         \
-      if (bias != nullptr) LAUNCH_B(DH, 1, true);                                                                    \
-      else LAUNCH_B(DH, 1, false);                                                                                   \
+      if (bias_len < 0) LAUNCH_B(DH, 1, kBiasPenalty);                                                               \
+      else if (bias != nullptr) LAUNCH_B(DH, 1, kBiasTable);                                                         \
+      else LAUNCH_B(DH, 1, kNoBias);                                                                                 \
     }                                                                                                                \
   } while (0)
   switch (dh) {
@@ -1679,12 +1715,15 @@ JLE_API int jle_attention_decode(const void* q, const void* kv, void* out, float
                      max_splits, split, ret_mode, ret_param, sl, Hq, Hkv, ps, bs)
 #define PICK(DH)                             \
   do {                                       \
-    if (bias != nullptr) {                   \
-      if (ct == 1) LAUNCH(DH, 1, true);      \
-      else LAUNCH(DH, 2, true);              \
+    if (bias_len < 0) {                      \
+      if (ct == 1) LAUNCH(DH, 1, kBiasPenalty); \
+      else LAUNCH(DH, 2, kBiasPenalty);      \
+    } else if (bias != nullptr) {            \
+      if (ct == 1) LAUNCH(DH, 1, kBiasTable); \
+      else LAUNCH(DH, 2, kBiasTable);        \
     } else {                                 \
-      if (ct == 1) LAUNCH(DH, 1, false);     \
-      else LAUNCH(DH, 2, false);             \
+      if (ct == 1) LAUNCH(DH, 1, kNoBias);   \
+      else LAUNCH(DH, 2, kNoBias);           \
     }                                        \
   } while (0)
   switch (dh) {

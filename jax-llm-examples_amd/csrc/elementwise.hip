@@ -193,7 +193,7 @@ static void launch_add_rmsnorm(float* x, Delta<DT> delta, const float* w, float 
   dim3 g(N);
   // (which kernel: by the width and the arrays' alignment only, so a row's result is the same in any batch)
   const uintptr_t all = (uintptr_t)x | (uintptr_t)delta.plain | (uintptr_t)delta.routed | (uintptr_t)delta.shared |
-                        (uintptr_t)w | (uintptr_t)out | (uintptr_t)out32;
+                        (uintptr_t)delta.self | (uintptr_t)w | (uintptr_t)out | (uintptr_t)out32;
   if (D % 8 == 0 && (all & 15) == 0 && D > 1024 && D <= 8192) {  // (rows of any of the arrays then start 16-byte aligned)
     // (the same arithmetic either way: only where the data are kept differs)
     if ((size_t)N * D >= ((size_t)4 << 20))
@@ -213,15 +213,17 @@ static void launch_add_rmsnorm(float* x, Delta<DT> delta, const float* w, float 
     hipLaunchKernelGGL((add_rmsnorm_wide_kernel<DT, OT>), g, dim3(256), 0, s, x, delta, w, eps, (OT*)out, out32, D);
 }
 
-// delta_kind: 0 none, 1 plain (delta), 2 expert sum (routed, inv, k, shared)
+// delta_kind: 0 none, 1 plain (delta), 2 expert sum (routed, inv, k, shared; self, self_w, self_k: see Delta)
 JLE_API int jle_add_rmsnorm(float* x, int delta_kind, const void* delta, const void* routed, const int* inv, int k,
                             const void* shared, int delta_is_bf16, const float* w, float eps, void* out,
-                            int out_is_bf16, float* out32, int N, int D, hipStream_t s) {
+                            int out_is_bf16, float* out32, int N, int D, const void* self, const float* self_w,
+                            int self_k, hipStream_t s) {
   if (N <= 0) return 0;
 #define GO(DT, OT)                                                                              \
   do {                                                                                          \
     Delta<DT> dl = {delta_kind == 1 ? (const DT*)delta : nullptr,                               \
-                    delta_kind == 2 ? (const DT*)routed : nullptr, inv, (const DT*)shared, k}; \
+                    delta_kind == 2 ? (const DT*)routed : nullptr, inv, (const DT*)shared, k,  \
+                    (const DT*)self, self_w, self_k};                                           \
     launch_add_rmsnorm<DT, OT>(x, dl, w, eps, out, out32, N, D, s);                             \
   } while (0)
   if (delta_is_bf16) {
@@ -357,52 +359,50 @@ JLE_API int jle_softcap(float* x, long long n, float cap, hipStream_t s) {
 // out[n, c] = o[n, c] * sigmoid(gate[n * gate_ld + c]): the gate's rows are a slice of wider rows.
 template <typename T>
 __global__ void sigmoid_mul_kernel(const T* __restrict__ o, const T* __restrict__ gate, int gate_ld,
-                                   T* __restrict__ out, int C) {
+                                   T* __restrict__ out, int C, int share) {
   const size_t row = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
-  const float g = Num<T>::load(gate + row * gate_ld + c);
+  const float g = Num<T>::load(gate + row * gate_ld + (share == 1 ? c : c / share));
   Num<T>::store(out + row * C + c, Num<T>::load(o + row * C + c) / (1.0f + expf(-g)));
 }
 
+// share: so many neighbouring elements of o have one gate (1: a gate each)
 JLE_API int jle_sigmoid_mul(const void* o, const void* gate, int gate_ld, void* out, int is_bf16, int N, int C,
-                            hipStream_t s) {
+                            int share, hipStream_t s) {
   if (N <= 0 || C <= 0) return 0;
-  if (gate_ld < C || (C + 255) / 256 > 65535) return JLE_BAD_ARG;
+  if (share < 1 || C % share || gate_ld < C / share || (C + 255) / 256 > 65535) return JLE_BAD_ARG;
   dim3 g(N, (C + 255) / 256), b(256);
   if (is_bf16)
     hipLaunchKernelGGL(sigmoid_mul_kernel<bf16_t>, g, b, 0, s, (const bf16_t*)o, (const bf16_t*)gate, gate_ld,
-                       (bf16_t*)out, C);
+                       (bf16_t*)out, C, share);
   else
     hipLaunchKernelGGL(sigmoid_mul_kernel<float>, g, b, 0, s, (const float*)o, (const float*)gate, gate_ld,
-                       (float*)out, C);
+                       (float*)out, C, share);
   JLE_LAUNCH_CHECK();
   return 0;
 }
 
 // ------------------------------------------------------------------ combine expert outputs
-// out[n] = sum_j routed[inv[n * k + j]] + shared[n]   (float32 result)
+// out[n] = sum_j routed[inv[n * k + j]] + shared[n]   (float32 result; see Delta for negative rows)
 template <typename T>
 __global__ void moe_combine_kernel(const T* __restrict__ routed, const int* __restrict__ inv,
-                                   const T* __restrict__ shared, float* __restrict__ out, int k, int D) {
+                                   const T* __restrict__ shared, float* __restrict__ out, int k, int D,
+                                   const T* __restrict__ self, const float* __restrict__ self_w, int self_k) {
   const size_t n = blockIdx.x;
-  for (int d = threadIdx.x; d < D; d += blockDim.x) {
-    float acc = 0.f;
-    for (int j = 0; j < k; ++j) acc += Num<T>::load(routed + (size_t)inv[n * k + j] * D + d);
-    if (shared != nullptr) acc += Num<T>::load(shared + n * D + d);
-    out[n * D + d] = acc;
-  }
+  const Delta<T> delta = {nullptr, routed, inv, shared, k, self, self_w, self_k};
+  for (int d = threadIdx.x; d < D; d += blockDim.x) out[n * D + d] = delta.at(n, d, D);
 }
 
 JLE_API int jle_moe_combine(const void* routed, const int* inv, const void* shared, float* out, int is_bf16, int N,
-                            int k, int D, hipStream_t s) {
+                            int k, int D, const void* self, const float* self_w, int self_k, hipStream_t s) {
   if (N <= 0) return 0;
   if (is_bf16)
     hipLaunchKernelGGL(moe_combine_kernel<bf16_t>, dim3(N), dim3(256), 0, s, (const bf16_t*)routed, inv,
-                       (const bf16_t*)shared, out, k, D);
+                       (const bf16_t*)shared, out, k, D, (const bf16_t*)self, self_w, self_k);
   else
     hipLaunchKernelGGL(moe_combine_kernel<float>, dim3(N), dim3(256), 0, s, (const float*)routed, inv,
-                       (const float*)shared, out, k, D);
+                       (const float*)shared, out, k, D, (const float*)self, self_w, self_k);
   JLE_LAUNCH_CHECK();
   return 0;
 }

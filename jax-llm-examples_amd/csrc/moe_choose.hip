@@ -1,96 +1,56 @@
-// The choice of experts by scores: s = sigmoid(z), choice scores c = s + correction; with groups, the experts form
-// equal groups of neighbours, a group's score is the sum of its `terms` largest c, the `keep` best groups stay; the
-// top_k largest c among the experts that stay, lowest index first among equals; the weights are the chosen s.
-// A thread per token walks through the experts (their number is small beside a token's other work).  And the
-// experts' activation relu(x)^2, element by element.
+// The choice of experts by scores (see Choice, route.h): a wavefront per token; in steps of few tokens one block chooses
+// for all of them and groups the choices by expert in the same launch.  And the experts' activation relu(x)^2,
+// element by element.
 #include "common.h"
+#include "route.h"
 
 using namespace jle;
 
 namespace {
 
-constexpr int kMaxGroups = 64, kMaxTerms = 4, kMaxTop = 16, kCached = 64;
+constexpr int kFewTokens = 64;  // up to here one block chooses and groups
 
-__device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
+__global__ __launch_bounds__(256) void moe_choose_kernel(const float* __restrict__ logits, Choice a, int* __restrict__ ids,
+                                                         float* __restrict__ weights, int N) {
+  extern __shared__ float lds[];  // [waves][2 E]
+  const int wave = wave_index(), lane = threadIdx.x & 63;
+  const int n = blockIdx.x * (blockDim.x >> 6) + wave;
+  if (n >= N) return;  // (no barrier below)
+  float* scores = lds + (size_t)wave * 2 * a.E;
+  int id;
+  float weight;
+  choose_by_wave<false>(logits + (size_t)n * a.E, a, scores, scores + a.E, id, weight);
+  if (lane < a.top_k) {
+    ids[(size_t)n * a.top_k + lane] = id;
+    weights[(size_t)n * a.top_k + lane] = weight;
+  }
+}
 
-__global__ __launch_bounds__(64) void moe_choose_kernel(const float* __restrict__ logits,
-                                                        const float* __restrict__ correction, int* __restrict__ ids,
-                                                        float* __restrict__ weights, int N, int E, int top_k,
-                                                        int groups, int keep, int terms) {
-  // (a thread's lists lie in shared memory: indexed by values that are known only when the kernel runs, they would
-  // otherwise be kept in scratch memory)
-  __shared__ float score_all[kMaxGroups][64];
-  __shared__ int chosen_all[kMaxTop][64];
-  const int n = blockIdx.x * 64 + threadIdx.x;
-  if (n >= N) return;
-  const int me = threadIdx.x;
-  const float* z = logits + (size_t)n * E;
-  // the choice scores of up to kCached experts are formed once and kept in shared memory (a thread walks through them
-  // top_k + 1 times); with more experts they are formed anew each time
-  __shared__ float cached[kCached][64];
-  const bool in_lds = E <= kCached;
-  if (in_lds)
-    for (int e = 0; e < E; ++e) cached[e][me] = sigmoidf_(z[e]) + (correction != nullptr ? correction[e] : 0.f);
-  auto choice = [&](int e) {
-    return in_lds ? cached[e][me] : sigmoidf_(z[e]) + (correction != nullptr ? correction[e] : 0.f);
-  };
-  unsigned long long kept = ~0ull;  // bit gi: group gi's experts can be chosen
-  const int per = groups > 0 ? E / groups : E;
-  if (groups > 0) {
-    for (int gi = 0; gi < groups; ++gi) {
-      float best[kMaxTerms];
-#pragma unroll
-      for (int i = 0; i < kMaxTerms; ++i) best[i] = -INFINITY;
-      for (int e = gi * per; e < (gi + 1) * per; ++e) {
-        float c = choice(e);
-#pragma unroll
-        for (int i = 0; i < kMaxTerms; ++i) {  // (kept in descending order)
-          if (i < terms && c > best[i]) {
-            const float t = best[i];
-            best[i] = c;
-            c = t;
-          }
-        }
-      }
-      float sum = 0.f;
-#pragma unroll
-      for (int i = 0; i < kMaxTerms; ++i)
-        if (i < terms && i < per) sum += best[i];
-      score_all[gi][me] = sum;
-    }
-    kept = 0ull;
-    for (int r = 0; r < keep; ++r) {
-      int at = -1;
-      float top = 0.f;
-      for (int gi = 0; gi < groups; ++gi) {
-        if ((kept >> gi) & 1ull) continue;
-        const float sc = score_all[gi][me];
-        if (at < 0 || sc > top) {
-          at = gi;
-          top = sc;
-        }
-      }
-      kept |= 1ull << at;
+__global__ __launch_bounds__(1024) void moe_choose_align_kernel(const float* __restrict__ logits, Choice a,
+                                                                int* __restrict__ ids, float* __restrict__ weights,
+                                                                int* __restrict__ offsets, int* __restrict__ sorted_token,
+                                                                float* __restrict__ sorted_weight, int* __restrict__ inv,
+                                                                int N, int experts, int extra, int inv_ld) {
+  extern __shared__ int smem[];  // counts[experts], starts[experts + 1], ids[N k], weights[N k], [waves][2 E] floats
+  const int k = a.top_k, M = N * k;
+  int* ids_s = smem + 2 * experts + 1;
+  float* weights_s = reinterpret_cast<float*>(ids_s + M);
+  const int wave = wave_index(), lane = threadIdx.x & 63;
+  float* scores = weights_s + M + (size_t)wave * 2 * a.E;
+  for (int n = wave; n < N; n += (int)(blockDim.x >> 6)) {
+    int id;
+    float weight;
+    choose_by_wave<false>(logits + (size_t)n * a.E, a, scores, scores + a.E, id, weight);
+    if (lane < k) {
+      ids[n * k + lane] = id;
+      weights[n * k + lane] = weight;
+      ids_s[n * k + lane] = id;
+      weights_s[n * k + lane] = weight;
     }
   }
-  for (int r = 0; r < top_k; ++r) {
-    int at = -1;
-    float top = 0.f;
-    for (int e = 0; e < E; ++e) {
-      if (groups > 0 && !((kept >> (e / per)) & 1ull)) continue;
-      bool taken = false;
-      for (int i = 0; i < r; ++i) taken |= chosen_all[i][me] == e;
-      if (taken) continue;
-      const float c = choice(e);
-      if (at < 0 || c > top) {
-        at = e;
-        top = c;
-      }
-    }
-    chosen_all[r][me] = at;
-    ids[(size_t)n * top_k + r] = at;
-    weights[(size_t)n * top_k + r] = sigmoidf_(z[at]);
-  }
+  __syncthreads();
+  align_by_block(ids_s, weights_s, smem, smem + experts, offsets, sorted_token, sorted_weight, inv, M, experts, k, extra,
+                 inv_ld);
 }
 
 template <typename T>
@@ -103,18 +63,34 @@ __global__ __launch_bounds__(256) void relu2_kernel(const T* __restrict__ x, T* 
 
 }  // namespace
 
-// groups == 0: no groups.  logits float32 [N, E]; correction float32 [E] or null.
+// groups == 0: no groups; correction null: none; floor_ < 0: the weights are not divided by their sum.  logits float32
+// [N, E].  experts > 0 (and few tokens: see jle_moe_choose_groups): also the grouping of the choices among the first
+// `experts` of the router's rows, as by jle_moe_align.
+JLE_API int jle_moe_choose_groups(int N, int E, int top_k, int experts) {
+  const size_t words = (size_t)2 * experts + 1 + (size_t)2 * N * top_k + (size_t)32 * E;
+  return N <= kFewTokens && words * sizeof(int) <= 64 * 1024;
+}
+
 JLE_API int jle_moe_choose(const float* logits, const float* correction, int* ids, float* weights, int N, int E,
-                           int top_k, int groups, int keep, int terms, hipStream_t s) {
+                           int top_k, int groups, int keep, int terms, int softmax, float floor_, float scale, int experts,
+                           int* offsets, int* sorted_token, float* sorted_weight, int* inv, int extra_group, int inv_ld,
+                           hipStream_t s) {
   if (N <= 0) return 0;
-  if (logits == nullptr || ids == nullptr || weights == nullptr || E <= 0 || top_k < 1 || top_k > kMaxTop || top_k > E)
-    return JLE_BAD_ARG;
-  if (groups < 0 || groups > kMaxGroups ||
-      (groups > 0 && (E % groups || keep < 1 || keep > groups || terms < 1 || terms > kMaxTerms ||
-                      keep * (E / groups) < top_k)))
-    return JLE_BAD_ARG;
-  hipLaunchKernelGGL(moe_choose_kernel, dim3((N + 63) / 64), dim3(64), 0, s, logits, correction, ids, weights, N, E,
-                     top_k, groups, keep, terms);
+  const Choice a = {correction, E, top_k, groups, keep, terms, softmax, floor_, scale};
+  if (logits == nullptr || ids == nullptr || weights == nullptr || !choice_ok(a)) return JLE_BAD_ARG;
+  if (experts > 0) {
+    if (experts > E || !jle_moe_choose_groups(N, E, top_k, experts) || offsets == nullptr || sorted_token == nullptr ||
+        sorted_weight == nullptr || inv == nullptr || inv_ld < top_k || inv_ld > top_k + 1)
+      return JLE_BAD_ARG;
+    const size_t words = (size_t)2 * experts + 1 + (size_t)2 * N * top_k + (size_t)32 * E;
+    hipLaunchKernelGGL(moe_choose_align_kernel, dim3(1), dim3(1024), words * sizeof(int), s, logits, a, ids, weights,
+                       offsets, sorted_token, sorted_weight, inv, N, experts, extra_group ? N : 0, inv_ld);
+    JLE_LAUNCH_CHECK();
+    return 0;
+  }
+  const int waves = E <= 1024 ? 4 : 1;
+  hipLaunchKernelGGL(moe_choose_kernel, dim3((N + waves - 1) / waves), dim3(64 * waves),
+                     (size_t)waves * 2 * E * sizeof(float), s, logits, a, ids, weights, N);
   JLE_LAUNCH_CHECK();
   return 0;
 }

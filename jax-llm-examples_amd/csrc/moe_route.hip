@@ -3,6 +3,7 @@
 #include <limits.h>
 
 #include "common.h"
+#include "route.h"
 #include "rows.h"
 
 using namespace jle;
@@ -78,15 +79,6 @@ __global__ __launch_bounds__(256) void moe_logits_kernel(const float* __restrict
       const float v = wave_sum(acc[t][j]);
       if (lane == 0 && n0 + t < N && e0 + j < E) logits[(size_t)(n0 + t) * E + e0 + j] = v;
     }
-}
-
-// A float written to / read from where all compute units of the GPU see it at once (the caches of one die are
-// written through and read past): for data that blocks on different dies hand each other within a launch.
-__device__ __forceinline__ void put_shared(float* p, float v) {
-  __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-}
-__device__ __forceinline__ float get_shared(const float* p) {
-  return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
 
 // The k largest logits of token n (lowest index first among equals) and their sigmoids.
@@ -187,56 +179,6 @@ __global__ void moe_topk_kernel(const float* __restrict__ logits, int* __restric
   }
 }
 
-// Stable counting sort of the M = N * k pairs by expert, by one block.
-//   offsets[e] .. offsets[e + 1]: rows of expert e in sorted order
-//   sorted_token[s]: the token of sorted row s;  sorted_gate[s]: its gate;  inv[r]: sorted row of pair r
-// ids and gates may lie in shared memory; counts[E] and starts[E + 1] do.
-// extra > 0: one more group behind the experts' that holds every token once, in order, with gate 1
-// (offsets[E + 1] = M + extra; rows M .. M + extra - 1): the rows of a shared expert.
-__device__ __forceinline__ void align_by_block(const int* ids, const float* gates, int* counts, int* starts,
-                                               int* __restrict__ offsets, int* __restrict__ sorted_token,
-                                               float* __restrict__ sorted_gate, int* __restrict__ inv, int M, int E,
-                                               int k, int extra) {
-  if (extra > 0) {
-    if (threadIdx.x == 0) offsets[E + 1] = M + extra;
-    for (int i = threadIdx.x; i < extra; i += blockDim.x) {
-      sorted_token[M + i] = i;
-      sorted_gate[M + i] = 1.0f;
-    }
-  }
-  for (int e = threadIdx.x; e < E; e += blockDim.x) counts[e] = 0;
-  __syncthreads();
-  for (int r = threadIdx.x; r < M; r += blockDim.x) atomicAdd(&counts[ids[r]], 1);
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    int run = 0;
-    for (int e = 0; e < E; ++e) {
-      starts[e] = run;
-      run += counts[e];
-    }
-    starts[E] = run;
-  }
-  __syncthreads();
-  for (int e = threadIdx.x; e <= E; e += blockDim.x) offsets[e] = starts[e];
-  const int lane = threadIdx.x & 63, wave = wave_index(), waves = blockDim.x >> 6;
-  for (int e = wave; e < E; e += waves) {
-    if (counts[e] == 0) continue;
-    int run = starts[e];
-    for (int base = 0; base < M; base += 64) {
-      const int r = base + lane;
-      const bool match = r < M && ids[r] == e;
-      const unsigned long long bal = __ballot(match);
-      if (match) {
-        const int pos = run + __popcll(bal & ((1ull << lane) - 1ull));
-        sorted_token[pos] = r / k;
-        sorted_gate[pos] = gates[r];
-        inv[r] = pos;
-      }
-      run += __popcll(bal);
-    }
-  }
-}
-
 // The same grouping for any number of pairs that lie in memory, a piece of the pairs at a time: all threads bring
 // the piece's experts into shared memory (whole lines); every wavefront looks through the piece for its experts
 // and notes each pair's row there; then all threads write the rows' tokens and gates.  Nothing in a wavefront's
@@ -245,23 +187,17 @@ __device__ __forceinline__ void align_by_block(const int* ids, const float* gate
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids, const float* __restrict__ gates,
                                                          int* __restrict__ offsets, int* __restrict__ sorted_token,
                                                          float* __restrict__ sorted_gate, int* __restrict__ inv,
-                                                         int M, int E, int k, int extra, int piece_len) {
+                                                         int M, int E, int k, int extra, int piece_len, int inv_ld) {
   extern __shared__ int smem[];  // counts[E], starts[E + 1], runs[E], piece[piece_len], rows[piece_len]
   int* counts = smem;
   int* starts = smem + E;
   int* runs = smem + 2 * E + 1;
   int* piece = smem + 3 * E + 1;
   int* rows = piece + piece_len;
-  if (extra > 0) {
-    if (threadIdx.x == 0) offsets[E + 1] = M + extra;
-    for (int i = threadIdx.x; i < extra; i += blockDim.x) {
-      sorted_token[M + i] = i;
-      sorted_gate[M + i] = 1.0f;
-    }
-  }
   for (int e = threadIdx.x; e < E; e += blockDim.x) counts[e] = 0;
   __syncthreads();
-  for (int r = threadIdx.x; r < M; r += blockDim.x) atomicAdd(&counts[ids[r]], 1);
+  for (int r = threadIdx.x; r < M; r += blockDim.x)
+    if (ids[r] < E) atomicAdd(&counts[ids[r]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int run = 0;
@@ -273,11 +209,15 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
     starts[E] = run;
   }
   __syncthreads();
+  extra_group(starts[E], offsets, sorted_token, sorted_gate, inv, E, k, extra, inv_ld);
   for (int e = threadIdx.x; e <= E; e += blockDim.x) offsets[e] = starts[e];
   const int lane = threadIdx.x & 63, wave = wave_index(), waves = blockDim.x >> 6;
   for (int c0 = 0; c0 < M; c0 += piece_len) {
     const int n = min(piece_len, M - c0);
-    for (int i = threadIdx.x; i < n; i += blockDim.x) piece[i] = ids[c0 + i];
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+      piece[i] = ids[c0 + i];
+      rows[i] = -1;
+    }
     __syncthreads();
     for (int e = wave; e < E; e += waves) {
       if (counts[e] == 0) continue;
@@ -293,10 +233,11 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
     }
     __syncthreads();
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-      const int pos = rows[i];
-      sorted_token[pos] = (c0 + i) / k;
+      const int pos = rows[i], t = (c0 + i) / k;
+      inv[t * inv_ld + (c0 + i) - t * k] = pos;
+      if (pos < 0) continue;
+      sorted_token[pos] = t;
       sorted_gate[pos] = gates[c0 + i];
-      inv[c0 + i] = pos;
     }
     __syncthreads();
   }
@@ -329,7 +270,7 @@ __global__ __launch_bounds__(1024) void moe_topk_align_kernel(const float* __res
     }
   }
   __syncthreads();
-  align_by_block(ids_s, gates_s, smem, smem + E, offsets, sorted_token, sorted_gate, inv, M, E, k, extra);
+  align_by_block(ids_s, gates_s, smem, smem + E, offsets, sorted_token, sorted_gate, inv, M, E, k, extra, k);
 }
 
 // Steps of few tokens: the addition of the pending branch output to the residual, the norm of the sum, the
@@ -339,7 +280,9 @@ __global__ __launch_bounds__(1024) void moe_topk_align_kernel(const float* __res
 // expert's logit (the arithmetic of moe_logits_kernel<1, 1, true>).  The block of a token's first four experts
 // also writes the new residual and the normed row.  The block that finishes last (a ticket counter, zero between
 // launches) chooses and groups for all tokens.  N <= 256, D a multiple of 8 in (1024, 8192].
-template <typename DT, typename OT>
+// SCORED: the choice is made by scores (see Choice, route.h); `experts` of the router's E rows have matrices and are
+// grouped, a token's row in the extra group is noted behind its choices' (inv_ld = k + 1 then).
+template <typename DT, typename OT, bool SCORED>
 __global__ __launch_bounds__(256) void norm_route_kernel(const float* __restrict__ x, Delta<DT> delta,
                                                          const float* __restrict__ w, float eps,
                                                          float* __restrict__ x_out, OT* __restrict__ h_out,
@@ -349,7 +292,7 @@ __global__ __launch_bounds__(256) void norm_route_kernel(const float* __restrict
                                                          int* __restrict__ sorted_token,
                                                          float* __restrict__ sorted_gate, int* __restrict__ inv,
                                                          int* __restrict__ ticket, int N, int D, int E, int k,
-                                                         int extra) {
+                                                         int extra, Choice choice, int experts) {
   constexpr int THREADS = 256, CPT = 8;
   extern __shared__ int smem[];  // the normed row [D] (floats); afterwards the grouping's counters and pairs
   float* row = reinterpret_cast<float*>(smem);
@@ -454,6 +397,24 @@ __global__ __launch_bounds__(256) void norm_route_kernel(const float* __restrict
   const int M = N * k;
   int* ids_s = ismem + 2 * E + 1;
   float* gates_s = reinterpret_cast<float*>(ids_s + M);
+  if (SCORED) {
+    float* scores = gates_s + M + (size_t)wave_index() * 2 * E;
+    for (int t = wave_index(); t < N; t += THREADS / 64) {
+      int id;
+      float weight;
+      choose_by_wave<true>(logits + (size_t)t * E, choice, scores, scores + E, id, weight);
+      if (lane < k) {
+        ids[t * k + lane] = id;
+        gates[t * k + lane] = weight;
+        ids_s[t * k + lane] = id;
+        gates_s[t * k + lane] = weight;
+      }
+    }
+    __syncthreads();
+    align_by_block(ids_s, gates_s, ismem, ismem + E, offsets, sorted_token, sorted_gate, inv, M, experts, k, extra,
+                   extra > 0 ? k + 1 : k);
+    return;
+  }
   if (E >= 64 && E <= 64 * kWaveTopKPerLane) {
     // many experts: a wavefront per token, the token's logits fetched in one trip
     for (int t = wave_index(); t < N; t += THREADS / 64) {
@@ -490,7 +451,7 @@ __global__ __launch_bounds__(256) void norm_route_kernel(const float* __restrict
     }
   }
   __syncthreads();
-  align_by_block(ids_s, gates_s, ismem, ismem + E, offsets, sorted_token, sorted_gate, inv, M, E, k, extra);
+  align_by_block(ids_s, gates_s, ismem, ismem + E, offsets, sorted_token, sorted_gate, inv, M, E, k, extra, k);
 }
 
 static int launch_logits(const float* h, const float* w, float* logits, int N, int D, int E, hipStream_t s) {
@@ -530,13 +491,13 @@ static int launch_logits(const float* h, const float* w, float* logits, int N, i
 }
 
 static int launch_align(const int* ids, const float* gates, int* offsets, int* sorted_token, float* sorted_gate,
-                        int* inv, int M, int E, int k, int extra, hipStream_t s) {
+                        int* inv, int M, int E, int k, int extra, int inv_ld, hipStream_t s) {
   // (shared memory: 64 KB; the pieces take what the experts' counters leave, at most 2,048 pairs)
   int piece = (16384 - (3 * E + 1)) / 2;
   piece = piece > 2048 ? 2048 : piece / 64 * 64;
   if (piece < 64) return JLE_BAD_ARG;
   hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), (3 * E + 1 + 2 * piece) * sizeof(int), s, ids, gates, offsets,
-                     sorted_token, sorted_gate, inv, M, E, k, extra, piece);
+                     sorted_token, sorted_gate, inv, M, E, k, extra, piece, inv_ld);
   JLE_LAUNCH_CHECK();
   return 0;
 }
@@ -576,18 +537,22 @@ JLE_API int jle_moe_route_align(const float* h, const float* w, int* ids, float*
   }
   hipLaunchKernelGGL(moe_topk_kernel, dim3((N + 127) / 128), dim3(128), 0, s, logits, ids, gates, N, E, k);
   JLE_LAUNCH_CHECK();
-  return launch_align(ids, gates, offsets, sorted_token, sorted_gate, inv, N * k, E, k, extra_group ? N : 0, s);
+  return launch_align(ids, gates, offsets, sorted_token, sorted_gate, inv, N * k, E, k, extra_group ? N : 0, k, s);
 }
 
+// inv_ld: k, or k + 1 to note a token's row in the extra group behind its choices' rows; choices of E and beyond get
+// no row (see route.h).
 JLE_API int jle_moe_align(const int* ids, const float* gates, int* offsets, int* sorted_token, float* sorted_gate,
-                          int* inv, int M, int E, int k, int extra_group, hipStream_t s) {
+                          int* inv, int M, int E, int k, int extra_group, int inv_ld, hipStream_t s) {
   if (M <= 0) return 0;
-  if (E < 1 || E > 4096 || k < 1 || M % k) return JLE_BAD_ARG;
-  return launch_align(ids, gates, offsets, sorted_token, sorted_gate, inv, M, E, k, extra_group ? M / k : 0, s);
+  if (E < 1 || E > 4096 || k < 1 || M % k || inv_ld < k || inv_ld > k + 1) return JLE_BAD_ARG;
+  return launch_align(ids, gates, offsets, sorted_token, sorted_gate, inv, M, E, k, extra_group ? M / k : 0, inv_ld, s);
 }
 
 // add + norm + router + choice + grouping in one launch, for steps of at most 256 tokens (see norm_route_kernel).
-// delta_kind: 0 none, 1 plain (delta), 2 expert sum (routed, inv_in, k_in, shared), as for jle_add_rmsnorm.
+// delta_kind: 0 none, 1 plain (delta), 2 expert sum (routed, inv_in, k_in, shared, self, self_w, self_k), as for
+// jle_add_rmsnorm.  experts > 0: the choice is made by scores (correction .. scale: see Choice, route.h), E counts the
+// router's rows, the first `experts` of them have matrices; with the extra group inv has k + 1 entries a token.
 // x_out: the residual after the addition (another array than x: the blocks of a token read x while one writes).
 // ticket: one counter, zero before the first launch and after every launch.
 // Returns JLE_BAD_ARG for sizes the fused kernel does not take (the caller then uses the separate kernels).
@@ -595,23 +560,34 @@ JLE_API int jle_norm_route(const float* x, int delta_kind, const void* delta, co
                            int k_in, const void* shared, int delta_is_bf16, const float* w, float eps, float* x_out,
                            void* h_out, int out_is_bf16, const float* router, float* logits, int* ids, float* gates,
                            int* offsets, int* sorted_token, float* sorted_gate, int* inv, int* ticket, int N, int D,
-                           int E, int k, int extra_group, hipStream_t s) {
+                           int E, int k, int extra_group, const void* self, const float* self_w, int self_k,
+                           int experts, const float* correction, int groups, int keep, int terms, int softmax,
+                           float floor_, float scale, hipStream_t s) {
   if (N <= 0) return 0;
-  if (N > 256 || D % 8 || D <= 1024 || D > 8192 || k < 1 || k > kMaxTopK || k > E || E > 4096) return JLE_BAD_ARG;
-  const uintptr_t all = (uintptr_t)x | (uintptr_t)delta | (uintptr_t)routed | (uintptr_t)shared | (uintptr_t)w |
+  const bool scored = experts > 0;
+  const Choice choice = {correction, E, k, groups, keep, terms, softmax, floor_, scale};
+  if (N > 256 || D % 8 || D <= 1024 || D > 8192 || k < 1 || k > E || E > 4096) return JLE_BAD_ARG;
+  if (scored ? (!choice_ok(choice) || experts > E) : k > kMaxTopK) return JLE_BAD_ARG;
+  const uintptr_t all = (uintptr_t)x | (uintptr_t)delta | (uintptr_t)routed | (uintptr_t)shared | (uintptr_t)w | (uintptr_t)self |
                         (uintptr_t)x_out | (uintptr_t)h_out | (uintptr_t)router;
   if ((all & 15) != 0 || ticket == nullptr || logits == nullptr || x_out == x) return JLE_BAD_ARG;
-  const size_t words = (size_t)2 * E + 1 + (size_t)2 * N * k;
+  const size_t words = (size_t)2 * E + 1 + (size_t)2 * N * k + (scored ? (size_t)8 * E : 0);
   const size_t lds = (words > (size_t)D ? words : (size_t)D) * sizeof(float);
   if (lds > 48 * 1024) return JLE_BAD_ARG;
   dim3 g(N, (E + 3) / 4), b(256);
 #define GO(DT, OT)                                                                                               \
   do {                                                                                                           \
     Delta<DT> dl = {delta_kind == 1 ? (const DT*)delta : nullptr,                                                \
-                    delta_kind == 2 ? (const DT*)routed : nullptr, inv_in, (const DT*)shared, k_in};             \
-    hipLaunchKernelGGL((norm_route_kernel<DT, OT>), g, b, lds, s, x, dl, w, eps, x_out, (OT*)h_out, router,      \
-                       logits, ids, gates, offsets, sorted_token, sorted_gate, inv, ticket, N, D, E, k,          \
-                       extra_group ? N : 0);                                                                     \
+                    delta_kind == 2 ? (const DT*)routed : nullptr, inv_in, (const DT*)shared, k_in,              \
+                    (const DT*)self, self_w, self_k};                                                            \
+    if (scored)                                                                                                  \
+      hipLaunchKernelGGL((norm_route_kernel<DT, OT, true>), g, b, lds, s, x, dl, w, eps, x_out, (OT*)h_out,      \
+                         router, logits, ids, gates, offsets, sorted_token, sorted_gate, inv, ticket, N, D, E,   \
+                         k, extra_group ? N : 0, choice, experts);                                               \
+    else                                                                                                         \
+      hipLaunchKernelGGL((norm_route_kernel<DT, OT, false>), g, b, lds, s, x, dl, w, eps, x_out, (OT*)h_out,     \
+                         router, logits, ids, gates, offsets, sorted_token, sorted_gate, inv, ticket, N, D, E,   \
+                         k, extra_group ? N : 0, choice, experts);                                               \
   } while (0)
   if (delta_is_bf16) {
     if (out_is_bf16) GO(bf16_t, bf16_t); else GO(bf16_t, float);

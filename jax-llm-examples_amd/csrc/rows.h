@@ -9,6 +9,8 @@ typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 
 // delta is either a plain tensor or the sum of a token's expert outputs and the shared expert's:
 //   delta[n] = sum_j routed[inv[n * k + j]] + shared[n]
+// A negative inv[n * k + j] stands for a choice whose output is the expert layer's own input row (an identity
+// expert): self_w[n * self_k + j] * self[n] is added for it.
 template <typename DT>
 struct Delta {
   const DT* plain;    // [N, D] or null
@@ -16,12 +18,19 @@ struct Delta {
   const int* inv;     // [N * k]
   const DT* shared;   // [N, D] or null
   int k;
+  const DT* self;       // [N, D] or null (then no entry of inv is negative)
+  const float* self_w;  // [N, self_k]
+  int self_k;
   __device__ __forceinline__ bool any() const { return plain != nullptr || routed != nullptr; }
   __device__ __forceinline__ float at(size_t n, int d, int D) const {
     float v = 0.f;
     if (plain != nullptr) v = Num<DT>::load(plain + n * D + d);
     if (routed != nullptr) {
-      for (int j = 0; j < k; ++j) v += Num<DT>::load(routed + (size_t)inv[n * k + j] * D + d);
+      for (int j = 0; j < k; ++j) {
+        const int r = inv[n * k + j];
+        if (self == nullptr || r >= 0) v += Num<DT>::load(routed + (size_t)r * D + d);
+        else v = __builtin_fmaf(self_w[n * self_k + j], Num<DT>::load(self + n * D + d), v);
+      }
       if (shared != nullptr) v += Num<DT>::load(shared + n * D + d);
     }
     return v;
@@ -80,8 +89,17 @@ __device__ __forceinline__ f32x4_t delta_at4(const Delta<DT>& delta, size_t n, i
   if (delta.plain != nullptr) v = load4_as<STREAM, DT>(delta.plain + n * D + d);
   if (delta.routed != nullptr) {
 #pragma nounroll
-    for (int j = 0; j < delta.k; ++j)
-      v += load4_as<STREAM, DT>(delta.routed + (size_t)delta.inv[n * delta.k + j] * D + d);
+    for (int j = 0; j < delta.k; ++j) {
+      const int r = delta.inv[n * delta.k + j];
+      if (delta.self == nullptr || r >= 0) {
+        v += load4_as<STREAM, DT>(delta.routed + (size_t)r * D + d);
+      } else {
+        const float w = delta.self_w[n * delta.self_k + j];
+        const f32x4_t h = load4_as<STREAM, DT>(delta.self + n * D + d);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = __builtin_fmaf(w, h[i], v[i]);
+      }
+    }
     if (delta.shared != nullptr) v += load4_as<STREAM, DT>(delta.shared + n * D + d);
   }
   return v;
@@ -101,7 +119,7 @@ __device__ __forceinline__ DeltaRow<DT> delta_row(const Delta<DT>& delta, size_t
   DeltaRow<DT> r = {nullptr, nullptr, false, false};
   if (delta.plain != nullptr && delta.routed == nullptr) {
     r.a = delta.plain + n * D;
-  } else if (delta.plain == nullptr && delta.routed != nullptr && delta.k == 1) {
+  } else if (delta.plain == nullptr && delta.routed != nullptr && delta.k == 1 && delta.self == nullptr) {
     r.a = delta.routed + (size_t)delta.inv[n] * D;
     r.b = delta.shared != nullptr ? delta.shared + n * D : nullptr;
     r.from_zero = true;

@@ -28,11 +28,11 @@ _vp, _i, _f, _ll = ctypes.c_void_p, ctypes.c_int, ctypes.c_float, ctypes.c_longl
 
 _SIGNATURES = {
     "jle_embed": [_vp, _vp, _i, _vp, _i, _i, _vp],
-    "jle_add_rmsnorm": [_vp, _i, _vp, _vp, _vp, _i, _vp, _i, _vp, _f, _vp, _i, _vp, _i, _i, _vp],
+    "jle_add_rmsnorm": [_vp, _i, _vp, _vp, _vp, _i, _vp, _i, _vp, _f, _vp, _i, _vp, _i, _i, _vp, _vp, _i, _vp],
     "jle_add_residual": [_vp, _vp, _i, _ll, _vp],
     "jle_gather_rows": [_vp, _vp, _vp, _i, _i, _vp],
     "jle_silu_mul": [_vp, _vp, _i, _i, _i, _vp],
-    "jle_moe_combine": [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp],
+    "jle_moe_combine": [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp, _vp, _i, _vp],
     "jle_qk_prepare": [_vp, _vp, _vp, _vp, _vp, _vp, _f, _f, _f, _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i,
                        _vp],
     "jle_paged_attention_generic": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _i, _i, _vp,
@@ -42,8 +42,8 @@ _SIGNATURES = {
     "jle_attention_merge": [_vp, _vp, _vp, _i, _i, _i, _i, _vp],
     "jle_moe_route": [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp],
     "jle_norm_route": [_vp, _i, _vp, _vp, _vp, _i, _vp, _i, _vp, _f, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
-                       _vp, _vp, _i, _i, _i, _i, _i, _vp],
-    "jle_moe_align": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp],
+                       _vp, _vp, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _vp, _i, _i, _i, _i, _f, _f, _vp],
+    "jle_moe_align": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp],
     "jle_moe_route_align": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp],
     "jle_gemm_generic": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp],
     "jle_gemm_f32_skinny": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp],
@@ -74,9 +74,9 @@ _SIGNATURES = {
     "jle_embed_pair": [_vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _ll, _ll, _vp],
     "jle_act_mul": [_vp, _vp, _i, _i, _i, _i, _vp],
     "jle_softcap": [_vp, _ll, _f, _vp],
-    "jle_sigmoid_mul": [_vp, _vp, _i, _vp, _i, _i, _i, _vp],
+    "jle_sigmoid_mul": [_vp, _vp, _i, _vp, _i, _i, _i, _i, _vp],
     "jle_add_norm_pair": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _f, _vp, _vp, _i, _i, _i, _vp],
-    "jle_conv_rows": [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp],
+    "jle_conv_rows": [_vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp],
     "jle_conv_qk_prepare": [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _f, _f, _vp, _vp, _i, _i,
                             _i, _i, _i, _i, _i, _i, _i, _vp],
     "jle_gemm_stream": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp],
@@ -90,14 +90,19 @@ _SIGNATURES = {
     "jle_row_gate": [_vp, _i, _vp, _vp, _i, _i, _i, _vp],
     "jle_scaled_add_norm": [_vp, _vp, _i, _f, _vp, _i, _f, _vp, _vp, _f, _vp, _i, _vp, _i, _i, _vp, _i, _vp],
     "jle_moe_logits": [_vp, _vp, _vp, _i, _i, _i, _vp],
-    "jle_heads_prepare": [_vp, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i,
-                          _vp],
+    "jle_heads_prepare": [_vp, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i,
+                          _i, _vp],
     "jle_diff_combine": [_vp, _vp, _vp, _f, _f, _f, _i, _i, _i, _i, _i, _i, _vp],
     "jle_gated_delta": [_vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i,
                         _i, _i, _i, _i, _f, _f, _vp],
-    "jle_moe_choose": [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp],
+    "jle_moe_choose": [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _vp, _vp, _vp, _vp, _i, _i, _vp],
+    "jle_moe_choose_groups": [_i, _i, _i, _i],
+    "jle_mamba2": [_vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _f, _i,
+                   _vp],
+    "jle_mamba2_chunked_supported": [_i, _i],
+    "jle_latent_down_prepare": [_vp, _i, _i, _vp, _f, _vp, _i, _i, _vp, _vp, _i, _i, _f, _vp, _f, _vp, _vp, _vp, _i, _vp,
+                                _i, _i, _i, _vp],
     "jle_relu2": [_vp, _vp, _i, _ll, _vp],
-    "jle_conv_rows_act": [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp],
     "jle_attention_prefill_kept": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _f, _i, _i, _i, _i, _vp],
     "jle_paged_attention_kept": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _i, _i, _vp,
                                  _vp, _vp],
@@ -112,10 +117,11 @@ class KernelError(RuntimeError):
 
 class ExpertSum:
     """A feed-forward output that is not formed yet: ``sum_j routed[inv[n * k + j]] + shared[n]``.  The kernel
-    that adds it to the residual and norms the result reads the pieces directly."""
+    that adds it to the residual and norms the result reads the pieces directly.  ``own = (h, weights)``: a negative
+    ``inv[n * k + j]`` stands for ``weights[n, j] * h[n]`` (an identity expert)."""
 
-    def __init__(self, routed, inv, k: int, shared, n: int, d: int) -> None:
-        self.routed, self.inv, self.k, self.shared = routed, inv, k, shared
+    def __init__(self, routed, inv, k: int, shared, n: int, d: int, own=None) -> None:
+        self.routed, self.inv, self.k, self.shared, self.own = routed, inv, k, shared, own
         self.shape = torch.Size((n, d))
         self.dtype = routed.dtype
 
@@ -491,12 +497,7 @@ class HipOps:
         n, ld = rows.shape
         self._chk(rows, None, None, "projected rows")
         self._chk(positions, torch.int32, (n,), "positions")
-        pairing, rd, inv = 0, 0, None
-        magnitude = 1.0 if rotation is None else float(getattr(rotation, "magnitude", 1.0))
-        if rotation is not None:
-            rd = int(rotation.rotary_dim) or rope_dim
-            pairing = {"adjacent": 0, "half": 1}[rotation.pairing]
-            inv = self._chk(rotation.inv_freq, torch.float32, (rd // 2,), "rotary frequencies")
+        pairing, rd, inv, magnitude = self._rotation(rotation, rope_dim)
         if writes:
             np_, ps = latent_pages.shape[0], latent_pages.shape[1]
             self._chk(latent_pages, rows.dtype, (np_, ps, kv_rank), "latent pages")
@@ -511,6 +512,52 @@ class HipOps:
                    _p(latent_pages) if writes else None, _p(rope_pages) if writes else None,
                    _p(latent_t_pages) if writes else None, latent_pages.shape[1] if writes else 0,
                    _p(slot_mapping) if writes else None, int(bool(writes)), self._is_bf16(rows), n)
+
+    def latent_down_prepare(self, rows, query_rank: int, query_norm, query_eps: float, rope_dim: int, kv_rank: int,
+                            positions, rotation, latent_norm, eps: float, latent_pages, rope_pages, slot_mapping,
+                            writes: bool, latent_t_pages=None):
+        """The queries' latent at the rows' start normed (returned), the cached latent and the shared key part behind
+        it normed, turned and written; see :meth:`latent_prepare`."""
+        n, ld = rows.shape
+        self._chk(rows, None, None, "projected rows")
+        self._chk(positions, torch.int32, (n,), "positions")
+        self._chk(query_norm, torch.float32, (query_rank,), "query norm weight")
+        pairing, rd, inv, magnitude = self._rotation(rotation, rope_dim)
+        if writes:
+            np_, ps = latent_pages.shape[0], latent_pages.shape[1]
+            self._chk(latent_pages, rows.dtype, (np_, ps, kv_rank), "latent pages")
+            self._chk(rope_pages, rows.dtype, (np_, ps, rope_dim), "rotated key pages")
+            if latent_t_pages is not None:
+                self._chk(latent_t_pages, rows.dtype, (np_, ps, kv_rank), "transposed latent pages")
+            self._chk(slot_mapping, torch.int32, (n,), "slot mapping")
+            if latent_norm is not None:
+                self._chk(latent_norm, torch.float32, (kv_rank,), "latent norm weight")
+        cq = torch.empty(n, query_rank, dtype=rows.dtype, device=rows.device)
+        self._call("jle_latent_down_prepare", _p(rows), ld, query_rank, _p(query_norm), float(query_eps), _p(cq), rope_dim,
+                   kv_rank, _p(positions), _p(inv), pairing, rd, magnitude, _p(latent_norm) if writes else None,
+                   float(eps), _p(latent_pages) if writes else None, _p(rope_pages) if writes else None,
+                   _p(latent_t_pages) if writes else None, latent_pages.shape[1] if writes else 0,
+                   _p(slot_mapping) if writes else None, int(bool(writes)), self._is_bf16(rows), n)
+        return cq
+
+    def rotate_heads_(self, q, num_heads: int, nope_dim: int, rope_dim: int, positions, rotation) -> None:
+        """Turns the last ``rope_dim`` numbers of every head's query in place."""
+        if rotation is None:
+            return
+        n, ld = q.shape
+        self._chk(q, None, (n, num_heads * (nope_dim + rope_dim)), "queries")
+        self._chk(positions, torch.int32, (n,), "positions")
+        pairing, rd, inv, magnitude = self._rotation(rotation, rope_dim)
+        self._call("jle_latent_prepare", _p(q), ld, num_heads, nope_dim, rope_dim, 1, _p(positions), _p(inv), pairing, rd,
+                   magnitude, None, 0.0, None, None, None, 0, None, 0, self._is_bf16(q), n)
+
+    def _rotation(self, rotation, dim: int):
+        """``(pairing, turned elements, frequencies, magnitude)`` as the latent kernels take them."""
+        if rotation is None:
+            return 0, 0, None, 1.0
+        rd = int(rotation.rotary_dim) or dim
+        inv = self._chk(rotation.inv_freq, torch.float32, (rd // 2,), "rotary frequencies")
+        return {"adjacent": 0, "half": 1}[rotation.pairing], rd, inv, float(getattr(rotation, "magnitude", 1.0))
 
     LATENT_SPLIT_BELOW = 2048  # fewer (token, head) pairs than this: a query's key tiles are shared between wavefronts
 
@@ -647,7 +694,8 @@ class HipOps:
         self._chk(x, torch.float32, (n, d), "residual")
         terms = list(delta.terms)
         inv, inv_k = None, 0
-        if isinstance(terms[0][0], ExpertSum) and terms[0][0].shared is None:  # (its pieces are added up by the kernel)
+        if isinstance(terms[0][0], ExpertSum) and terms[0][0].shared is None and terms[0][0].own is None:
+            # (its pieces are added up by the kernel)
             pieces = terms[0][0]
             inv, inv_k = pieces.inv, pieces.k
             terms[0] = (pieces.routed, terms[0][1])
@@ -693,7 +741,7 @@ class HipOps:
         out = torch.empty(n, d, dtype=out_dtype, device=x.device)
         out32 = torch.empty(n, d, dtype=torch.float32, device=x.device) if want32 else None
         self._call("jle_add_rmsnorm", _p(x), kind, _p(plain), _p(routed), _p(inv), k, _p(shared), is_bf16, _p(weight),
-                   float(eps), _p(out), self._is_bf16(out), _p(out32), n, d)
+                   float(eps), _p(out), self._is_bf16(out), _p(out32), n, d, *self._own_rows(delta))
         return out, out32
 
     def defer_norm(self, x, delta, weight, eps: float, out_dtype) -> PendingNorm:
@@ -717,8 +765,14 @@ class HipOps:
         n, d = delta.shape
         out = torch.empty(n, d, dtype=torch.float32, device=delta.routed.device)
         self._call("jle_moe_combine", _p(delta.routed), _p(delta.inv), _p(delta.shared), _p(out),
-                   self._is_bf16(delta.routed), n, delta.k, d)
+                   self._is_bf16(delta.routed), n, delta.k, d, *self._own_rows(delta))
         return out
+
+    @staticmethod
+    def _own_rows(delta):
+        """``(rows, weights, weights a token)`` of an expert layer's identity experts, as the kernels take them."""
+        own = getattr(delta, "own", None)
+        return (None, None, 0) if own is None else (_p(own[0]), _p(own[1]), own[1].shape[1])
 
     def add_residual(self, x, delta) -> None:
         if hasattr(delta, "terms"):
@@ -783,13 +837,16 @@ class HipOps:
         return self.silu_mul(torch.matmul(h, w_gate_up.t()), activation)
 
     def sigmoid_mul(self, o, gate):
-        """``o * sigmoid(gate)``; ``gate`` may be a slice of wider rows (its last axis contiguous)."""
+        """``o * sigmoid(gate)``; ``gate`` may be a slice of wider rows (its last axis contiguous), and narrower than ``o``:
+        one gate for as many neighbouring elements as it is narrower."""
         n, c = o.shape
         self._chk(o, None, (n, c), "rows")
-        if gate.dtype != o.dtype or tuple(gate.shape) != (n, c) or gate.stride(1) != 1 or not gate.is_cuda:
-            raise KernelError("the gate must have the rows' shape and dtype, its last axis contiguous")
+        gc = gate.shape[1]
+        if gate.dtype != o.dtype or gate.shape[0] != n or c % gc or gate.stride(1) != 1 or not gate.is_cuda:
+            raise KernelError("the gate must have the rows' dtype and a divisor of their width, its last axis contiguous")
         out = torch.empty_like(o)
-        self._call("jle_sigmoid_mul", _p(o), _p(gate), gate.stride(0) if n > 1 else c, _p(out), self._is_bf16(o), n, c)
+        self._call("jle_sigmoid_mul", _p(o), _p(gate), gate.stride(0) if n > 1 else gc, _p(out), self._is_bf16(o), n, c,
+                   c // gc)
         return out
 
     def conv_attention(self, proj, bias, conv_w, taps: int, state, num_heads: int, num_kv_heads: int, head_dim: int,
@@ -823,13 +880,18 @@ class HipOps:
                                  page_dim, prep, ctx, kv_cache if writes else None, slot_mapping)
         return self.paged_attention(q, kv_cache, block_table, ctx.positions, ctx.token_segment, retention, scale, meta)
 
-    def conv_rows(self, proj, bias, conv_w, taps: int, state, ctx, activation=None):
+    def conv_rows(self, proj, bias, conv_w, taps: int, state, ctx, activation=None, conv_bias=None):
         """``y[t] = sum_j conv_w[j] * u[t - taps + 1 + j]`` (``conv_w``: ``[taps, channels]``) with ``u = proj + bias`` rounded to the run dtype, rows
         before a segment's start from the requests' two-halved state, whose other half gets the segment's last
-        ``taps - 1`` rows of ``u``; ``[N, C]`` in the run dtype.  See ``attention_conv.hip``."""
+        ``taps - 1`` rows of ``u``; ``[N, C]`` in the run dtype.  ``conv_bias``: what the sum over the taps starts from;
+        ``activation``: ``silu`` on the sum.  ``proj`` may be a view of wider rows.  See ``attention_conv.hip``."""
         n, channels = proj.shape
         dt = ctx.dtype
-        self._chk(proj, None, (n, channels), "projected rows")
+        if proj.stride(1) != 1 or not proj.is_cuda or (n > 1 and proj.stride(0) < channels):
+            raise KernelError("projected rows: neighbouring channels must lie side by side, on the kernels' device")
+        ld = proj.stride(0) if n > 1 else max(channels, proj.stride(0))
+        if conv_bias is not None:
+            self._chk(conv_bias, torch.float32, (channels,), "convolution bias")
         if proj.dtype not in (dt, torch.float32):
             raise KernelError(f"projected rows in {proj.dtype}, run dtype {dt}")
         if bias is not None:
@@ -844,18 +906,12 @@ class HipOps:
                                (ctx.state_phase, "state phases", (ctx.num_segments,))):
             self._chk(t, torch.int32, shape, what)
         y = torch.empty(n, channels, dtype=dt, device=proj.device)
-        if activation is not None:  # (on the convolution's result, float32, before the rounding)
-            if activation != "silu":
-                raise KernelError(f"the convolution kernel knows the activation silu, not {activation!r}")
-            self._call("jle_conv_rows_act", _p(proj), 1 if proj.dtype == torch.float32 else 0, _p(bias),
-                       _p(conv_w) if taps else None, int(taps), _p(state) if taps > 1 else None,
-                       _p(ctx.token_segment), _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(y),
-                       1 if dt == torch.bfloat16 else 0, n, ctx.num_segments, channels, 1)
-            return y
-        self._call("jle_conv_rows", _p(proj), 1 if proj.dtype == torch.float32 else 0, _p(bias),
-                   _p(conv_w) if taps else None, int(taps), _p(state) if taps > 1 else None, _p(ctx.token_segment),
-                   _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(y),
-                   1 if dt == torch.bfloat16 else 0, n, ctx.num_segments, channels)
+        if activation not in (None, "silu"):  # (on the convolution's result, float32, before the rounding)
+            raise KernelError(f"the convolution kernel knows the activation silu, not {activation!r}")
+        self._call("jle_conv_rows", _p(proj), 1 if proj.dtype == torch.float32 else 0, ld, _p(bias),
+                   _p(conv_w) if taps else None, _p(conv_bias), int(taps), _p(state) if taps > 1 else None,
+                   _p(ctx.token_segment), _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(y),
+                   1 if dt == torch.bfloat16 else 0, n, ctx.num_segments, channels, 0 if activation is None else 1)
         return y
 
     def heads_prepare(self, rows, q_heads: int, k_heads: int, v_heads: int, head_dim: int, value_dim: int,
@@ -875,9 +931,14 @@ class HipOps:
             rd = int(rot.rotary_dim) or dk
             inv_freq, magnitude = self._chk(rot.inv_freq, torch.float32, (rd // 2,), "inv_freq"), float(rot.magnitude)
             half = 1 if rot.pairing == "half" else 0
-        for w in (prep.norm_weight_q, prep.norm_weight_k):
-            if w is not None:
-                self._chk(w, torch.float32, (dk,), "q/k norm weight")
+        wq_stride = 0
+        if prep.norm_weight_q is not None and prep.norm_weight_q.dim() == 2:  # (weights of its own for every head)
+            self._chk(prep.norm_weight_q, torch.float32, (q_heads, dk), "q norm weights")
+            wq_stride = dk
+        elif prep.norm_weight_q is not None:
+            self._chk(prep.norm_weight_q, torch.float32, (dk,), "q norm weight")
+        if prep.norm_weight_k is not None:
+            self._chk(prep.norm_weight_k, torch.float32, (dk,), "k norm weight")
         self._chk(positions, torch.int32, (n,), "positions")
         ps = 1
         if kv_cache is not None:
@@ -887,8 +948,8 @@ class HipOps:
         q = torch.empty(n, q_heads, D, dtype=dt, device=rows.device)
         self._call("jle_heads_prepare", _p(rows), _p(positions), _p(slot_mapping) if kv_cache is not None else None,
                    _p(inv_freq), rd, half, magnitude, -1.0 if prep.norm_eps is None else float(prep.norm_eps),
-                   1 if prep.norm_first else 0, _p(prep.norm_weight_q), _p(prep.norm_weight_k), _p(q), _p(kv_cache),
-                   self._is_bf16(rows), n, q_heads, k_heads, v_heads, dk, dv, D, ps)
+                   1 if prep.norm_first else 0, _p(prep.norm_weight_q), wq_stride, _p(prep.norm_weight_k), _p(q),
+                   _p(kv_cache), self._is_bf16(rows), n, q_heads, k_heads, v_heads, dk, dv, D, ps)
         return q
 
     def diff_combine(self, o, lam: float, out_scale: float, eps: float, gate, num_heads: int, num_kv_heads: int,
@@ -934,6 +995,36 @@ class HipOps:
                    _p(out_gate), _p(state), _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(qn), _p(kn),
                    _p(beta), _p(decay), _p(kq), _p(o_raw), _p(out), n, ctx.num_segments, H, G, dk, dv, float(eps),
                    float(floor))
+        return out
+
+    MAMBA2_CHUNKS_FROM = 12  # a segment of so many tokens: the kernel that takes 64 at a time
+
+    def mamba2(self, proj, rows, dt_bias, a_log, skip, norm_weight, num_heads: int, value_dim: int, state_dim: int,
+               num_groups: int, norm_groups: int, eps: float, state, ctx):
+        """See ``mamba2.hip``: step sizes and decays of the step's tokens, the recurrence from and into the requests'
+        two-halved memory, gate and norm.  ``[N, H P]`` in the run dtype."""
+        n = rows.shape[0]
+        H, P, S, G = num_heads, value_dim, state_dim, num_groups
+        self._chk(rows, None, (n, H * P + 2 * G * S), "x | B | C rows")
+        self._chk(proj, rows.dtype, (n, 2 * H * P + 2 * G * S + H), "projected rows")
+        self._chk(state, torch.float32, (state.shape[0], 2, H, P, S), "memory")
+        for t, shape, what in ((dt_bias, (H,), "dt_bias"), (a_log, (H,), "a_log"), (skip, (H,), "skip"),
+                               (norm_weight, (H * P,), "norm weight")):
+            self._chk(t, torch.float32, shape, what)
+        for t, what, shape in ((ctx.cu_seqlens, "segment bounds", (ctx.num_segments + 1,)),
+                               (ctx.state_slots, "state slots", (ctx.num_segments,)),
+                               (ctx.state_phase, "state phases", (ctx.num_segments,))):
+            self._chk(t, torch.int32, shape, what)
+        if S > 512:
+            raise KernelError(f"the mamba2 kernels take states of up to 512 numbers a column, not {S}")
+        bf16 = self._is_bf16(rows)
+        chunked = (max(ctx.seg_lens, default=0) >= self.MAMBA2_CHUNKS_FROM
+                   and self._query("jle_mamba2_chunked_supported", S, bf16))
+        y = torch.empty(n, H * P, dtype=torch.float32, device=rows.device)
+        out = torch.empty(n, H * P, dtype=rows.dtype, device=rows.device)
+        self._call("jle_mamba2", _p(proj), proj.shape[1], _p(rows), bf16, _p(dt_bias), _p(a_log), _p(skip), _p(norm_weight),
+                   _p(state), _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(y), _p(out), n,
+                   ctx.num_segments, H, P, S, G, norm_groups, float(eps), int(bool(chunked)))
         return out
 
     def conv_qk_prepare(self, proj, bias, conv_w, taps: int, state, num_heads: int, num_kv_heads: int, head_dim: int,
@@ -1422,9 +1513,10 @@ class HipOps:
     F32_DECODE_ITEMS = 2048  # ... in a step of single tokens: about so many (token, kv head, key range) items
 
     def paged_attention(self, q, kv_cache, block_table, positions, token_segment, retention, scale: float, meta=None,
-                        bias=None, sink=None):
+                        bias=None, sink=None, penalty=None):
         """``bias``: float32 ``[Hq, L]``: a key ``n`` places back adds ``bias[h, min(n, L - 1)]`` to head ``h``'s scaled
-        score; ``sink``: float32 ``[Hq]``: ``exp(sink[h])`` is one more term of head ``h``'s denominator."""
+        score; ``sink``: float32 ``[Hq]``: ``exp(sink[h])`` is one more term of head ``h``'s denominator; ``penalty``:
+        float32 ``[Hq, 2]``: ``penalty[h, 0] * ln(1 + penalty[h, 1] * n)`` is taken off (without a ``bias``)."""
         n, hq, dh = q.shape
         hk, ps = kv_cache.shape[2], kv_cache.shape[3]
         self._chk(q, kv_cache.dtype, None, "q")
@@ -1435,12 +1527,17 @@ class HipOps:
         mode = _ret_mode(retention)
         param = int(retention[1]) if len(retention) > 1 else 0
         out = torch.empty(n, hq * dh, dtype=q.dtype, device=q.device)
+        if penalty is not None:
+            if bias is not None:
+                raise KernelError("the attention kernels take a distance table or a distance penalty, not both")
+            bias = self._chk(penalty, torch.float32, (hq, 2), "distance penalty")
         biased = bias is not None or sink is not None
         if retention[0] == "window_keep":
             return self._attention_kept(q, kv_cache, out, block_table, positions, token_segment, mode, param,
                                         int(retention[2]), scale, meta, biased)
         if bias is not None:
             self._chk(bias, torch.float32, (hq, bias.shape[1]), "distance bias")
+        bias_len = 0 if bias is None else -1 if penalty is not None else bias.shape[1]
         if sink is not None:
             self._chk(sink, torch.float32, (hq,), "sinks")
         if (q.dtype == torch.bfloat16 and hq // hk <= 32
@@ -1452,7 +1549,7 @@ class HipOps:
                 bias = self._zero_bias.get((hq, q.device))
                 if bias is None:
                     bias = self._zero_bias[(hq, q.device)] = torch.zeros(hq, 1, dtype=torch.float32, device=q.device)
-            bias_len = bias.shape[1] if biased else 0
+                bias_len = 1
             tile = self.BIASED_TILE if biased and grouped == 1 else self.PREFILL_TILE
             key = f"attn_plan_{grouped}_{tile}"
             plan = meta.meta.get(key) if meta is not None else None
@@ -1543,7 +1640,7 @@ class HipOps:
             self._call("jle_paged_attention_biased", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                        _p(block_table), block_table.shape[1], mode, param, float(scale), self._is_bf16(q), n, hq, hk,
                        dh, ps, splits, tiles_per_split, _p(ws_ml), _p(ws_o), _p(bias),
-                       0 if bias is None else bias.shape[1], _p(sink))
+                       bias_len, _p(sink))
             return out
         self._call("jle_paged_attention_generic", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                    _p(block_table), block_table.shape[1], mode, param, float(scale), self._is_bf16(q), n, hq, hk, dh,
@@ -1605,12 +1702,30 @@ class HipOps:
         return out
 
     # ------------------------------------------------------------------ routed experts
-    def moe_choose(self, h32, router, correction, top_k: int, groups=None, keep_groups=None, group_terms: int = 2):
+    def moe_choose(self, h32, router, correction, top_k: int, groups=None, keep_groups=None, group_terms: int = 2,
+                   scores: str = "sigmoid", normalize=None, weight_scale: float = 1.0, num_experts=None,
+                   extra_group: bool = False):
         """Router logits in float32 (the router kernel), then the choice by scores with a correction and groups
-        (``moe_choose.hip``) and the grouping of the choices by expert.  Returns ``(ids, weights, grouping)``."""
-        h32 = self._rows(h32, want32=True)
+        (``route.h``) and the grouping of the choices by expert, of the first ``num_experts`` of the router's rows
+        (``extra_group``: with the rows of a shared expert behind them, noted as one more row of every token); in steps
+        of few tokens one launch with the norm, or one launch for choice and grouping.  Returns ``(ids, weights,
+        grouping)``."""
         n, d = h32.shape
         e = router.shape[0]
+        experts = e if num_experts is None else int(num_experts)
+        # (the shared expert's rows ride in the routed experts' launches in steps of few tokens only)
+        extra_group = extra_group and n <= self.SHARED_RIDES_ROWS and n * top_k <= 2 * self.SKINNY_MAX_ROWS
+        if scores not in ("sigmoid", "softmax"):
+            raise KernelError(f"unknown scores {scores!r}")
+        how = (0 if groups is None else int(groups), 0 if groups is None else int(keep_groups), int(group_terms),
+               1 if scores == "softmax" else 0, -1.0 if normalize is None else float(normalize), float(weight_scale))
+        if isinstance(h32, PendingNorm):
+            fused = None if h32.done or hasattr(h32.delta, "terms") or n > self.NORM_CHOOSE_ROWS else \
+                self._norm_route(h32, router, top_k, scored=(experts, correction, how, extra_group))
+            if fused is not None:
+                ids, weights, _, grouping = fused
+                return ids, weights, grouping
+            h32 = h32.rows(want32=True)
         self._chk(h32, torch.float32, None, "router input")
         self._chk(router, torch.float32, (e, d), "router matrix")
         if correction is not None:
@@ -1620,9 +1735,25 @@ class HipOps:
         self._call("jle_moe_logits", _p(h32), _p(router), _p(logits), n, d, e)
         ids = torch.empty(n, top_k, dtype=torch.int32, device=dev)
         weights = torch.empty(n, top_k, dtype=torch.float32, device=dev)
-        self._call("jle_moe_choose", _p(logits), _p(correction), _p(ids), _p(weights), n, e, top_k,
-                   0 if groups is None else int(groups), 0 if groups is None else int(keep_groups), int(group_terms))
-        return ids, weights, self.moe_align(ids, weights, e)
+        if self._query("jle_moe_choose_groups", n, e, top_k, experts):
+            grouping = self._grouping_arrays(n, top_k, experts, extra_group, dev)
+            self._call("jle_moe_choose", _p(logits), _p(correction), _p(ids), _p(weights), n, e, top_k, *how, experts,
+                       *(_p(t) for t in grouping), int(extra_group), top_k + int(extra_group))
+            return ids, weights, grouping
+        self._call("jle_moe_choose", _p(logits), _p(correction), _p(ids), _p(weights), n, e, top_k, *how, 0, None, None, None,
+                   None, 0, top_k)
+        return ids, weights, self.moe_align(ids, weights, experts, extra_group=extra_group, note_extra=extra_group)
+
+    NORM_CHOOSE_ROWS = 64  # up to here the choice by scores is made in the launch that norms the rows
+
+    @staticmethod
+    def _grouping_arrays(n: int, k: int, experts: int, extra: bool, dev):
+        """Offsets, sorted tokens and weights, and where each pair went (see ``route.h``)."""
+        x = int(extra)
+        return (torch.empty(experts + 1 + x, dtype=torch.int32, device=dev),
+                torch.empty(n * (k + x), dtype=torch.int32, device=dev),
+                torch.empty(n * (k + x), dtype=torch.float32, device=dev),
+                torch.empty(n * (k + x), dtype=torch.int32, device=dev))
 
     def relu2(self, x):
         """``relu(x)^2`` element by element."""
@@ -1632,41 +1763,69 @@ class HipOps:
         return y
 
     def moe_experts_scored(self, h, expert_ids, weights, w_up, w_down, activation: str = "relu2", tiled: bool = False,
-                           grouping=None):
+                           grouping=None, shared_weights=None, identity: bool = False):
         """``sum_j weights[j] * W_down[e_j] relu(W_up[e_j] h)^2``: the choices grouped by expert, the first product
         plain, the activation a kernel of its own, the weights the second product's row scale (applied to its float32
-        sums); the sum over a token's choices stays in pieces (:class:`ExpertSum`)."""
-        if activation != "relu2":
+        sums); the sum over a token's choices stays in pieces (:class:`ExpertSum`).  ``activation = "swiglu"``: ``w_up`` holds
+        gate and up rows, the activation is part of the first product.  ``identity``: choices beyond the experts are identity
+        experts (they have no row; the sum adds the token's own).  ``shared_weights``: a SwiGLU expert of every token,
+        unweighted; in steps of few tokens one more group of the two products."""
+        if activation not in ("relu2", "swiglu"):
             raise KernelError(f"unknown activation {activation!r}")
         h = self._rows(h)
         n, d = h.shape
-        e, f, _ = w_up.shape
+        e, f = w_up.shape[0], w_down.shape[2]
+        swiglu = activation == "swiglu"
         k = expert_ids.shape[1]
         m = n * k
-        if grouping is None:
-            grouping = self.moe_align(expert_ids.contiguous(), weights.contiguous(), e)
-        offsets, sorted_token, sorted_weight, inv = grouping
         mfma = h.dtype == torch.bfloat16 and d % 8 == 0 and f % 8 == 0
+        ride = (shared_weights is not None and swiglu and mfma and n <= self.SHARED_RIDES_ROWS
+                and m <= 2 * self.SKINNY_MAX_ROWS and tuple(shared_weights[0].shape) == (2 * f, d)
+                and (grouping is None or grouping[0].numel() == e + 2))
+        if grouping is None:
+            extra = ride
+            grouping = self.moe_align(expert_ids.contiguous(), weights.contiguous(), e, extra_group=extra, note_extra=extra)
+        offsets, sorted_token, sorted_weight, inv = grouping
+        own = (h, weights.contiguous()) if identity else None
+        if ride:  # (a token's row of the shared expert is noted in ``inv`` behind its choices')
+            act = self.gemm_skinny(h, w_up, offsets=offsets, a_rows=sorted_token, swiglu=True, tiled=tiled,
+                                   b_last=shared_weights[0], rows=m + n)
+            routed = self.gemm_skinny(act, w_down, offsets=offsets, scale=sorted_weight, tiled=tiled,
+                                      b_last=shared_weights[1])
+            return ExpertSum(routed, inv, k + 1, None, n, d, own)
+        shared = None
+        if offsets.numel() == e + 2:  # (grouped with the shared expert's rows: they are the sum's last piece all the same)
+            offsets = offsets[: e + 1]
+            inv = inv.view(n, k + 1)[:, :k].contiguous().view(-1)
+            sorted_token, sorted_weight = sorted_token[:m], sorted_weight[:m]
+        if shared_weights is not None:
+            shared = self.linear(self.swiglu_linear(h, shared_weights[0]), shared_weights[1])
 
-        def product(x, w, nout, kdim, **kw):
+        def product(x, w, nout, kdim, fused=False, **kw):
+            kw.update(offsets=offsets)
             if mfma and m <= 2 * self.SKINNY_MAX_ROWS:
-                return self.gemm_skinny(x, w, offsets=offsets, tiled=tiled, **kw)
-            if mfma and tiled and self.stream_supported(nout, kdim, False):
-                return self.gemm_stream(x, w, offsets=offsets, **kw)
+                return self.gemm_skinny(x, w, swiglu=fused, tiled=tiled, **kw)
+            if mfma and tiled and self.stream_supported(nout, kdim, fused):
+                return self.gemm_stream(x, w, swiglu=fused, **kw)
             if mfma:
-                return self.gemm_grouped(x, w, offsets=offsets, tiled=tiled, **kw)
+                return self.gemm_grouped(x, w, swiglu=fused, tiled=tiled, **kw)
             if tiled:
                 raise KernelError("weights in the streaming layout need the MFMA product kernels")
-            if (x.dtype == torch.float32 and kdim % 4 == 0 and nout % 4 == 0 and m <= self.F32_SKINNY_ROWS):
-                return self.gemm_f32_skinny(x, w, offsets=offsets, **kw)
-            if (x.dtype == torch.float32 and self.f32_stream_supported(nout, kdim, False) and x.numel() < 2 ** 32
+            if (x.dtype == torch.float32 and kdim % 4 == 0 and (nout // 2 if fused else nout) % 4 == 0
+                    and m <= self.F32_SKINNY_ROWS):
+                return self.gemm_f32_skinny(x, w, swiglu=fused, **kw)
+            if (x.dtype == torch.float32 and self.f32_stream_supported(nout, kdim, fused) and x.numel() < 2 ** 32
                     and m * nout < 2 ** 32 and not (x.data_ptr() | w.data_ptr()) % 16):
-                return self.gemm_f32_stream(x, w, offsets=offsets, **kw)
-            return self.gemm(x, w, offsets=offsets, **kw)
+                return self.gemm_f32_stream(x, w, swiglu=fused, **kw)
+            y = self.gemm(x, w, **kw)
+            return self.silu_mul(y) if fused else y
 
-        up = product(h, w_up, f, d, a_rows=sorted_token)
-        routed = product(self.relu2(up), w_down, d, f, scale=sorted_weight)
-        return ExpertSum(routed, inv, k, None, n, d)
+        if swiglu:
+            act = product(h, w_up, 2 * f, d, fused=True, a_rows=sorted_token)
+        else:
+            act = self.relu2(product(h, w_up, f, d, a_rows=sorted_token))
+        routed = product(act, w_down, d, f, scale=sorted_weight)
+        return ExpertSum(routed, inv, k, shared, n, d, own)
 
     def moe_route(self, h32, router, top_k: int, want_logits: bool = False, group: bool = False):
         """``group``: also return the grouping of the choices by expert (what ``moe_align`` gives), made in
@@ -1703,14 +1862,15 @@ class HipOps:
 
     NORM_ROUTE_ROWS = 256
 
-    def _norm_route(self, pending: PendingNorm, router, top_k: int):
-        """The pending addition and norm, the router's logits, the choice and the grouping (with the extra group
+    def _norm_route(self, pending: PendingNorm, router, top_k: int, scored=None):
+        """``scored = (experts, correction, how, extra_group)``: the choice by scores (see :meth:`moe_choose`).  The pending addition and norm, the router's logits, the choice and the grouping (with the extra group
         of a shared expert's rows) in one launch, for a step of few tokens; ``None`` if the sizes do not fit."""
         x, delta = pending.x, pending.delta
         n, d = x.shape
         e = router.shape[0]
-        words = 2 * e + 1 + 2 * n * top_k
-        if (n > self.NORM_ROUTE_ROWS or d % 8 or not 1024 < d <= 8192 or not 1 <= top_k <= min(8, e) or e > 4096
+        words = 2 * e + 1 + 2 * n * top_k + (0 if scored is None else 8 * e)
+        most = 8 if scored is None else 64
+        if (n > self.NORM_ROUTE_ROWS or d % 8 or not 1024 < d <= 8192 or not 1 <= top_k <= min(most, e) or e > 4096
                 or 4 * max(words, d) > 48 * 1024 or x.dtype != torch.float32 or router.dtype != torch.float32):
             return None
         kind, plain, routed, inv_in, k_in, shared, is_bf16 = 0, None, None, None, 0, None, 0
@@ -1720,7 +1880,9 @@ class HipOps:
         elif delta is not None:
             self._chk(delta, None, (n, d), "branch output")
             kind, plain, is_bf16 = 1, delta, self._is_bf16(delta)
-        tensors = [t for t in (x, plain, routed, shared, pending.weight, router) if t is not None]
+        own = self._own_rows(delta)
+        rows_own = None if own[0] is None else delta.own[0]
+        tensors = [t for t in (x, plain, routed, shared, rows_own, pending.weight, router) if t is not None]
         if any(t.data_ptr() % 16 or not t.is_contiguous() for t in tensors):
             return None
         self._chk(router, torch.float32, (e, d), "router matrix")
@@ -1729,25 +1891,26 @@ class HipOps:
         dev = x.device
         x_out = torch.empty_like(x)
         h = torch.empty(n, d, dtype=pending.dtype, device=dev)
-        m = n * top_k
         ids = torch.empty(n, top_k, dtype=torch.int32, device=dev)
         gates = torch.empty(n, top_k, dtype=torch.float32, device=dev)
         logits = torch.empty(n, e, dtype=torch.float32, device=dev)
-        offsets = torch.empty(e + 2, dtype=torch.int32, device=dev)
-        sorted_token = torch.empty(m + n, dtype=torch.int32, device=dev)
-        sorted_gate = torch.empty(m + n, dtype=torch.float32, device=dev)
-        inv = torch.empty(m, dtype=torch.int32, device=dev)
+        m = n * top_k
+        experts, correction, how, extra = (0, None, (0, 0, 1, 0, -1.0, 1.0), True) if scored is None else scored
+        if correction is not None:
+            self._chk(correction, torch.float32, (e,), "correction")
+        offsets, sorted_token, sorted_gate, inv = self._grouping_arrays(n, top_k, experts or e, extra, dev)
         self._call("jle_norm_route", _p(x), kind, _p(plain), _p(routed), _p(inv_in), k_in, _p(shared), is_bf16,
                    _p(pending.weight), pending.eps, _p(x_out), _p(h), self._is_bf16(h), _p(router), _p(logits),
                    _p(ids), _p(gates), _p(offsets), _p(sorted_token), _p(sorted_gate), _p(inv),
-                   self._tickets[-1:].data_ptr(), n, d, e, top_k, 1)
+                   self._tickets[-1:].data_ptr(), n, d, e, top_k, int(extra), *own, experts, _p(correction), *how)
         pending.x_out, pending.h = x_out, h
-        return ids, gates, logits, (offsets, sorted_token, sorted_gate, inv)
+        return ids, gates, logits, (offsets, sorted_token, sorted_gate, inv if scored is not None else inv[:m])
 
-    def moe_align(self, expert_ids, gates, num_experts: int, extra_group: bool = False):
+    def moe_align(self, expert_ids, gates, num_experts: int, extra_group: bool = False, note_extra: bool = False):
         """Stable grouping of the (token, choice) pairs by expert: offsets ``[E + 1]``, the token and the gate of
         every sorted row, and where each pair went.  ``extra_group``: one more group behind the experts' that
-        holds every token once, in order, with gate 1 (the rows of a shared expert)."""
+        holds every token once, in order, with gate 1 (the rows of a shared expert); ``note_extra``: ``inv`` has that
+        row of every token behind its choices'.  A choice of ``num_experts`` or beyond has no row (``inv`` -1)."""
         n, k = expert_ids.shape
         m = n * k
         x = n if extra_group else 0
@@ -1757,9 +1920,10 @@ class HipOps:
         offsets = torch.empty(num_experts + (2 if extra_group else 1), dtype=torch.int32, device=dev)
         sorted_token = torch.empty(m + x, dtype=torch.int32, device=dev)
         sorted_gate = torch.empty(m + x, dtype=torch.float32, device=dev)
-        inv = torch.empty(m, dtype=torch.int32, device=dev)
+        ld = k + int(note_extra and extra_group)
+        inv = torch.empty(n * ld, dtype=torch.int32, device=dev)
         self._call("jle_moe_align", _p(expert_ids), _p(gates), _p(offsets), _p(sorted_token), _p(sorted_gate), _p(inv),
-                   m, num_experts, k, int(extra_group))
+                   m, num_experts, k, int(extra_group), ld)
         return offsets, sorted_token, sorted_gate, inv
 
     def row_gate_(self, rows, h32, w):

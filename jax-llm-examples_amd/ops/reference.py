@@ -383,7 +383,7 @@ class ReferenceOps:
         """``proj``: ``[N, 2 H P + 2 G S + H]`` = gate z | (values x | write keys B | read keys C before their convolution) |
         step sizes, run dtype; ``rows``: ``[N, H P + 2 G S]`` = x | B | C behind convolution and activation, run dtype.
         Per head, with the B and C of its group, token by token from the request's memory (``state[slot, phase]``:
-        ``[H, S, P]``; the new one goes to ``state[slot, 1 - phase]``)::
+        ``[H, P, S]``, a value column's numbers side by side; the new one goes to ``state[slot, 1 - phase]``)::
 
             d = softplus(dt + dt_bias);  M <- exp(-exp(a_log) d) M + d B x^T;  y = M^T C + skip x
 
@@ -404,8 +404,8 @@ class ReferenceOps:
         for s in range(len(cu) - 1):
             M = state[slots[s], phase[s]].float().clone()
             for t in range(cu[s], cu[s + 1]):
-                M = decay[t][:, None, None] * M + (d[t][:, None] * B[t])[:, :, None] * x[t][:, None, :]
-                y[t] = torch.einsum("hsp,hs->hp", M, C[t]) + skip.float()[:, None] * x[t]
+                M = decay[t][:, None, None] * M + x[t][:, :, None] * (d[t][:, None] * B[t])[:, None, :]
+                y[t] = torch.einsum("hps,hs->hp", M, C[t]) + skip.float()[:, None] * x[t]
             state[slots[s], 1 - phase[s]] = M.to(state.dtype)
         y = y.reshape(n, inner) * torch.nn.functional.silu(proj[:, :inner].float())
         y = y.reshape(n, norm_groups, inner // norm_groups)
@@ -765,7 +765,7 @@ class ReferenceOps:
         return ids.to(torch.int32), w * weight_scale, None
 
     def moe_experts_scored(self, h, expert_ids, weights, w_up, w_down, activation: str = "relu2", tiled: bool = False,
-                           grouping=None, shared_weights=None):
+                           grouping=None, shared_weights=None, identity: bool = False):
         """``sum_j weights[j] * W_down[e_j] act(W_up[e_j] h)`` per token, float32 result; ``w_up`` ``[E, F, D]``,
         ``w_down`` ``[E, D, F]``; ``act = relu2``: the square of relu.  ``swiglu``: ``w_up`` is ``[E, 2F, D]`` (gate
         rows, then up rows) and ``act`` gives ``silu(gate) * up``.  A choice ``e_j >= E`` is an identity expert: its

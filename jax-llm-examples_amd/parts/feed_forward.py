@@ -227,7 +227,7 @@ class MoEScored(FeedForward):
                 grouping = None
         return ops.moe_experts_scored(h, expert_ids, weights, self.params[self.up_name], self.params["w_down"],
                                       activation=self.activation, tiled=self.tiled, grouping=grouping,
-                                      shared_weights=shared)
+                                      shared_weights=shared, identity=self.identity > 0)
 
 
 @register_feed_forward("dense_polynorm")

@@ -69,7 +69,7 @@ class Mamba2(Mixer):
         self.conv_by_tap = self.params["conv"].t().contiguous()
 
     def cache_need(self) -> CacheNeed:
-        states = [("memory", (2, self.num_heads, self.state_dim, self.value_dim), torch.float32)]
+        states = [("memory", (2, self.num_heads, self.value_dim, self.state_dim), torch.float32)]  # (S transposed)
         if self.conv_taps > 1:
             states.append(("conv", (2, self.conv_taps - 1, self.channels), self.state_dtype))
         return CacheNeed(states=tuple(states))
