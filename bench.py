@@ -104,8 +104,24 @@ def design_configs(size: dict, layers: int):
                 "layers": [{"type": "attention", "mixer": s_diff, "mlp": s_moe} if i % 3 == 2 else
                            {"type": "parallel", "mixer": {"left": s_left, "right": s_right, "left_scale": 1.0,
                                                           "right_scale": 0.7}, "mlp": s_moe} for i in range(layers)]}
+    # Folivik: two Mamba-2 layers (twice the width inside) to one of window attention with distance penalties and one
+    # over a latent with the queries through a latent of their own; eight experts and two identity experts in five
+    # groups, two a token, beside a shared one.  Its closest models here: Mazotar (recurrent memory, attention with a
+    # distance bias, shared expert) and, for the latent layer, Rovidra
+    f_mem = {"heads": size["width"] // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    f_attn = {"heads": size["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+              "mask": {"size": size["span"]}}
+    f_latent = {"heads": size["heads"], "dim": size["dim"], "rot_dim": size["rot"], "vdim": size["vdim"],
+                "kv_rank": size["rank"], "q_rank": 3 * size["rank"], "scale": (size["dim"] + size["rot"]) ** -0.5,
+                "rot": {"base": 500000.0, "dims": size["rot"]}}
+    f_moe = {"kind": "moe", "router": {"experts": 8, "top": 2, "identity": 2, "scale": 2.0,
+                                       "groups": {"count": 5, "keep": 3}},
+             "expert": {"ff": size["ff"] // 2}, "shared": {"ff": size["ff"] // 2}}
+    f_kinds = [("mamba2", f_mem), ("attention", f_attn), ("mamba2", f_mem), ("latent_attention", f_latent)]
+    folivik = {"architecture": "Folivik", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5},
+               "layers": [{"type": f_kinds[i % 4][0], "mixer": f_kinds[i % 4][1], "mlp": f_moe} for i in range(layers)]}
     return {"rovidra": rovidra, "tiradra": tiradra, "llama4-dense": llama, "mazotar": mazotar, "llama4-moe": llama_moe,
-            "sudilorn": sudilorn}
+            "sudilorn": sudilorn, "folivik": folivik}
 
 
 def bench_designs(args) -> int:
@@ -214,10 +230,10 @@ def main() -> int:
     ap.add_argument("--no-prefill", action="store_true")
     ap.add_argument("--design-points", default="1@2048,8@2048,64@2048", help="decode steps of --designs: batch@context")
     ap.add_argument("--designs", default="", help="instead of the default workload: prefill and decode of the Rovidra, "
-                    "Tiradra, Mazotar and Sudilorn designs beside the Llama 4 layers of equal sizes, at the named sizes "
+                    "Tiradra, Mazotar, Sudilorn and Folivik designs beside the Llama 4 layers of equal sizes, at the named sizes "
                     "(comma-separated, of " + ", ".join(DESIGN_SIZES) + "; 'all')")
     ap.add_argument("--design-names", default="", help="with --designs: only these of rovidra, tiradra, llama4-dense, "
-                    "mazotar, llama4-moe, sudilorn")
+                    "mazotar, llama4-moe, sudilorn, folivik")
     args = ap.parse_args()
     if args.designs:
         return bench_designs(args)

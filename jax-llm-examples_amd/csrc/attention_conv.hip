@@ -243,8 +243,9 @@ constexpr int kTapsInRegisters = 8;
 // A block takes rows_per_block consecutive tokens of the step for its channels (one in a step of few tokens, where
 // the blocks are few as it is): the taps' weights and the bias are read once per block (up to kTapsInRegisters taps;
 // more are read again for every token), and the rows that neighbouring tokens share come from the first-level
-// cache.  A token's sums are the same whatever the number.
-template <typename PT, typename T>
+// cache.  KT > 0 (the number of taps, in steps of many tokens): a block whose tokens are of one segment asks for all
+// its rows at once and keeps them in registers, every row read once.  A token's sums are the same whatever the number.
+template <typename PT, typename T, int KT>
 __global__ __launch_bounds__(256) void conv_rows_vec_kernel(ConvArgs<PT, T> a, T* __restrict__ y_out, int N,
                                                             int token_blocks, int rows_per_block) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
@@ -280,6 +281,36 @@ __global__ __launch_bounds__(256) void conv_rows_vec_kernel(ConvArgs<PT, T> a, T
   for (int j = 0; j < kTapsInRegisters; ++j)
     if (j < K) Row8<float>::load(a.w + (size_t)j * a.C + c, wreg[j]);
   const int n_end = min(N, ((int)blockIdx.x + 1) * rows_per_block);
+  if (KT > 0) {
+    const int n0 = blockIdx.x * kRowsPerBlock;
+    const int seg = a.token_segment[n0];
+    if (n_end - n0 == kRowsPerBlock && a.token_segment[n_end - 1] == seg) {
+      const int t0 = n0 - a.cu_seqlens[seg];
+      const T* old = nullptr;
+      if (KT > 1) old = a.state + ((size_t)a.state_slots[seg] * 2 + a.state_phase[seg]) * (KT - 1) * a.C;
+      constexpr int B = KT > 0 ? KT - 1 : 0;  // rows in front of the block's first
+      float run[B + kRowsPerBlock][8];
+#pragma unroll
+      for (int i = 0; i < B + kRowsPerBlock; ++i) {
+        if (t0 + i - B >= 0) projected8(a, (size_t)(n0 + i - B), c, bias8, run[i]);
+        else Row8<T>::load(old + (size_t)(t0 + i) * a.C + c, run[i]);
+      }
+#pragma unroll
+      for (int r = 0; r < kRowsPerBlock; ++r) {
+        float y[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) y[i] = start8[i];
+#pragma unroll
+        for (int j = 0; j < KT; ++j)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) y[i] = __builtin_fmaf(wreg[j][i], run[r + j][i], y[i]);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) y[i] = Num<T>::round(conv_act(y[i], a.act));
+        Row8<T>::store(y_out + (size_t)(n0 + r) * a.C + c, y);
+      }
+      return;
+    }
+  }
   for (int n = blockIdx.x * rows_per_block; n < n_end; ++n) {
     float y[8];
     if (K == 0) {
@@ -329,8 +360,14 @@ int launch_conv_rows(const ConvArgs<PT, T>& a, void* y_out, int N, int R, hipStr
   {
     const int per = N >= 512 ? kRowsPerBlock : 1;
     const int token_blocks = (N + per - 1) / per;
-    hipLaunchKernelGGL((conv_rows_vec_kernel<PT, T>), dim3(token_blocks + (a.taps > 1 ? R : 0), (a.C / 8 + 255) / 256),
-                       dim3(256), 0, s, a, (T*)y_out, N, token_blocks, per);
+    const dim3 grid(token_blocks + (a.taps > 1 ? R : 0), (a.C / 8 + 255) / 256);
+#define JLE_ROWS(KT) \
+  hipLaunchKernelGGL((conv_rows_vec_kernel<PT, T, KT>), grid, dim3(256), 0, s, a, (T*)y_out, N, token_blocks, per)
+    if (per == kRowsPerBlock && a.taps == 4) JLE_ROWS(4);
+    else if (per == kRowsPerBlock && a.taps == 3) JLE_ROWS(3);
+    else if (per == kRowsPerBlock && a.taps == 2) JLE_ROWS(2);
+    else JLE_ROWS(0);
+#undef JLE_ROWS
   }
   else
     hipLaunchKernelGGL((conv_rows_kernel<PT, T>), dim3(N + (a.taps > 1 ? R : 0), (a.C + 255) / 256), dim3(256), 0, s, a,

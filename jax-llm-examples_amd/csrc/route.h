@@ -41,17 +41,68 @@ __device__ __forceinline__ void wave_sees_own_writes() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
+// Over all lanes without a trip through shared memory: within rows of 16 lanes by lane permutations that ride on an
+// operand (neighbour, neighbour's neighbour, mirrored half row, mirrored row), then rows and halves swapped.
+template <int CTRL>
+__device__ __forceinline__ uint32_t permuted(uint32_t v) {
+  return (uint32_t)__builtin_amdgcn_mov_dpp((int)v, CTRL, 0xf, 0xf, true);
+}
+template <typename F>
+__device__ __forceinline__ float lanes_reduce(float x, F f) {
+  uint32_t u = __float_as_uint(x);
+  u = __float_as_uint(f(__uint_as_float(u), __uint_as_float(permuted<0xB1>(u))));
+  u = __float_as_uint(f(__uint_as_float(u), __uint_as_float(permuted<0x4E>(u))));
+  u = __float_as_uint(f(__uint_as_float(u), __uint_as_float(permuted<0x141>(u))));
+  u = __float_as_uint(f(__uint_as_float(u), __uint_as_float(permuted<0x140>(u))));
+  auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+  u = __float_as_uint(f(__uint_as_float(r[0]), __uint_as_float(r[1])));
+  r = __builtin_amdgcn_permlane32_swap(u, u, false, false);
+  return f(__uint_as_float(r[0]), __uint_as_float(r[1]));
+}
+__device__ __forceinline__ float lanes_sum(float x) {
+  return lanes_reduce(x, [](float a, float b) { return a + b; });
+}
+__device__ __forceinline__ float lanes_max(float x) {
+  return lanes_reduce(x, [](float a, float b) { return fmaxf(a, b); });
+}
+
 // the larger of two (value, index) pairs in all lanes, the lower index among equals; INT_MAX: none
 __device__ __forceinline__ void wave_best(float& v, int& at) {
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1) {
-    const float ov = __shfl_xor(v, o, 64);
-    const int oa = __shfl_xor(at, o, 64);
+  auto better = [&](float ov, int oa) {
     if (oa != INT_MAX && (at == INT_MAX || ov > v || (ov == v && oa < at))) {
       v = ov;
       at = oa;
     }
+  };
+  better(__uint_as_float(permuted<0xB1>(__float_as_uint(v))), (int)permuted<0xB1>((uint32_t)at));
+  better(__uint_as_float(permuted<0x4E>(__float_as_uint(v))), (int)permuted<0x4E>((uint32_t)at));
+  better(__uint_as_float(permuted<0x141>(__float_as_uint(v))), (int)permuted<0x141>((uint32_t)at));
+  better(__uint_as_float(permuted<0x140>(__float_as_uint(v))), (int)permuted<0x140>((uint32_t)at));
+  {
+    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    const auto b = __builtin_amdgcn_permlane16_swap((uint32_t)at, (uint32_t)at, false, false);
+    v = __uint_as_float(a[0]);
+    at = (int)b[0];
+    better(__uint_as_float(a[1]), (int)b[1]);
   }
+  const auto a = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  const auto b = __builtin_amdgcn_permlane32_swap((uint32_t)at, (uint32_t)at, false, false);
+  v = __uint_as_float(a[0]);
+  at = (int)b[0];
+  better(__uint_as_float(a[1]), (int)b[1]);
+}
+
+// how many of the lanes 0 .. n - 1 whose bit is set in `open` come before this lane when they are ordered by their
+// values, largest first, the lower lane first among equals
+__device__ __forceinline__ int lanes_rank(float v, int n, unsigned long long open) {
+  const int lane = threadIdx.x & 63;
+  int rank = 0;
+  for (int i = 0; i < n; ++i) {
+    if (!((open >> i) & 1ull)) continue;
+    const float o = __uint_as_float((uint32_t)__builtin_amdgcn_readlane((int)__float_as_uint(v), i));
+    rank += (o > v || (o == v && i < lane)) ? 1 : 0;
+  }
+  return rank;
 }
 
 // A wavefront chooses for one token.  z: the token's logits; scores, choices: E floats of shared memory each, the
@@ -71,14 +122,14 @@ __device__ __forceinline__ void choose_by_wave(const float* z, const Choice& a, 
   }
   float inv = 1.0f;
   if (a.softmax) {
-    top = wave_max(top);
+    top = lanes_max(top);
     float sum = 0.f;
     for (int e = lane; e < E; e += 64) {
       const float p = expf(scores[e] - top);
       scores[e] = p;
       sum += p;
     }
-    inv = wave_sum(sum);
+    inv = lanes_sum(sum);
   }
   for (int e = lane; e < E; e += 64) {
     const float s = a.softmax ? scores[e] / inv : 1.0f / (1.0f + expf(-scores[e]));
@@ -109,20 +160,29 @@ __device__ __forceinline__ void choose_by_wave(const float* z, const Choice& a, 
       for (int i = 0; i < kChoiceMaxTerms; ++i)
         if (i < a.terms && i < per) mine += best[i];
     }
-    kept = 0ull;
-    for (int r = 0; r < a.keep; ++r) {
-      float v = mine;
-      int at = lane < a.groups && !((kept >> lane) & 1ull) ? lane : INT_MAX;
-      wave_best(v, at);
-      kept |= 1ull << at;
-    }
+    kept = __ballot(lane < a.groups && lanes_rank(mine, a.groups, ~0ull) < a.keep);
   }
   unsigned long long open = 0ull;  // bit j: this lane's expert lane + 64 j can still be chosen
   for (int j = 0, e = lane; e < E; ++j, e += 64)
     if (a.groups == 0 || ((kept >> (e / per)) & 1ull)) open |= 1ull << j;
-  id = 0;
+  id = lane < E ? lane : 0;
   weight = 0.f;
-  for (int r = 0; r < a.top_k; ++r) {
+  if (E <= 64) {  // an expert a lane: every lane counts those ahead of it, and leaves its number at its place
+    const bool mine = (open & 1ull) != 0ull;
+    const float c = lane < E ? choices[lane] : 0.f;
+    const float s = lane < E ? scores[lane] : 0.f;
+    const int rank = lanes_rank(c, E, __ballot(mine));
+    wave_sees_own_writes();  // (the lanes have read their scores)
+    int* place = reinterpret_cast<int*>(choices);
+    if (lane < a.top_k) place[lane] = lane;  // (what stays there if no order can be told: a number all the same)
+    wave_sees_own_writes();
+    if (mine && rank < a.top_k) place[rank] = lane;
+    wave_sees_own_writes();
+    if (lane < a.top_k) id = place[lane];
+    weight = __shfl(s, id, 64);
+    if (lane >= a.top_k) weight = 0.f;
+  }
+  for (int r = 0; E > 64 && r < a.top_k; ++r) {
     float v = 0.f;
     int at = INT_MAX;
     for (int j = 0, e = lane; e < E; ++j, e += 64) {
@@ -141,7 +201,7 @@ __device__ __forceinline__ void choose_by_wave(const float* z, const Choice& a, 
     }
   }
   if (a.floor_ >= 0.f) {
-    const float total = wave_sum(lane < a.top_k ? weight : 0.f) + a.floor_;
+    const float total = lanes_sum(lane < a.top_k ? weight : 0.f) + a.floor_;
     weight = weight / total;
   }
   weight *= a.scale;

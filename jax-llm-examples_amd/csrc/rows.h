@@ -106,23 +106,39 @@ __device__ __forceinline__ f32x4_t delta_at4(const Delta<DT>& delta, size_t n, i
 }
 
 // What a row's delta is made of, looked up once per row: for a plain tensor and for tokens with one expert the
-// row(s) to read; tokens with several experts keep the general sum (delta_at4), piece by piece.
+// row(s) to read, for tokens with up to kDeltaPieces of them the rows and their factors; tokens with more keep the
+// general sum (delta_at4), piece by piece.  The sums and their order are delta_at4's.
+constexpr int kDeltaPieces = 4;
 template <typename DT>
 struct DeltaRow {
   const DT* a;      // the plain row, or the row of the token's one expert
   const DT* b;      // the shared expert's row, or null
   bool from_zero;   // a is an expert's row: the sum starts from zero, as delta_at4's does
   bool general;
+  // a few experts' rows (or the token's own, weighted): looked up once, so that no piece waits for the look-up
+  int count;
+  const DT* piece[kDeltaPieces];
+  float factor[kDeltaPieces];
 };
 template <typename DT>
 __device__ __forceinline__ DeltaRow<DT> delta_row(const Delta<DT>& delta, size_t n, int D) {
-  DeltaRow<DT> r = {nullptr, nullptr, false, false};
+  DeltaRow<DT> r = {nullptr, nullptr, false, false, 0, {}, {}};
   if (delta.plain != nullptr && delta.routed == nullptr) {
     r.a = delta.plain + n * D;
   } else if (delta.plain == nullptr && delta.routed != nullptr && delta.k == 1 && delta.self == nullptr) {
     r.a = delta.routed + (size_t)delta.inv[n] * D;
     r.b = delta.shared != nullptr ? delta.shared + n * D : nullptr;
     r.from_zero = true;
+  } else if (delta.plain == nullptr && delta.routed != nullptr && delta.k <= kDeltaPieces) {
+    r.count = delta.k;
+    r.b = delta.shared != nullptr ? delta.shared + n * D : nullptr;
+#pragma unroll
+    for (int j = 0; j < kDeltaPieces; ++j) {
+      const int at = j < delta.k ? delta.inv[n * delta.k + j] : 0;
+      const bool own = delta.self != nullptr && at < 0;
+      r.piece[j] = own ? delta.self + n * D : delta.routed + (size_t)at * D;
+      r.factor[j] = own ? delta.self_w[n * delta.self_k + j] : 1.0f;
+    }
   } else {
     r.general = true;
   }
@@ -132,6 +148,19 @@ template <bool STREAM, typename DT>
 __device__ __forceinline__ f32x4_t delta_row_at4(const Delta<DT>& delta, const DeltaRow<DT>& row, size_t n, int d,
                                                  int D) {
   if (row.general) return delta_at4<STREAM, DT>(delta, n, d, D);
+  if (row.count > 0) {
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < kDeltaPieces; ++j) {
+      if (j < row.count) {
+        const f32x4_t h = load4_as<STREAM, DT>(row.piece[j] + d);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = __builtin_fmaf(row.factor[j], h[i], v[i]);
+      }
+    }
+    if (row.b != nullptr) v += load4_as<STREAM, DT>(row.b + d);
+    return v;
+  }
   f32x4_t v = load4_as<STREAM, DT>(row.a + d);
   if (row.from_zero) v = f32x4_t{0.f, 0.f, 0.f, 0.f} + v;
   if (row.b != nullptr) v += load4_as<STREAM, DT>(row.b + d);
