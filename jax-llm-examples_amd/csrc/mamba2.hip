@@ -11,8 +11,9 @@
 //  scan: token after token.  A wavefront takes 16 value columns of one (segment, head): lane (pg, l), pg = lane / 16, l =
 //    lane % 16, holds the columns pg, pg + 4, .. and of each the numbers 4 l .. 4 l + 3 of every 64; the products with C
 //    are summed over l by lane exchanges.  Both dtypes; steps of single tokens and of short segments.
-//  chunks (bfloat16 rows): a block takes 64 value columns of one (segment, head) and goes through the segment 64 tokens at
-//    a time, the memory in registers.  With L_t the running sum of a in the chunk and S0 the memory in front of it:
+//  chunks (bfloat16 rows): a block of eight wavefronts takes 64 value columns of one (segment, head) and goes through the
+//    segment 64 tokens at a time, the memory in registers (two wavefronts share 16 columns, each holds half of a
+//    column's numbers).  With L_t the running sum of a in the chunk and S0 the memory in front of it:
 //      y_t = exp(L_t) S0^T C_t + sum_{s <= t} exp(L_t - L_s) d_s (C_t . B_s) x_s + skip x_t
 //      S   = exp(L_end) S0 + sum_s exp(L_end - L_s) d_s B_s x_s^T
 //    as products on the bfloat16 matrix instructions.  B, C and x enter exactly (they are bfloat16 numbers); what is not -
@@ -182,6 +183,7 @@ __global__ __launch_bounds__(64) void mamba2_scan_kernel(const T* __restrict__ p
 constexpr int kChunk = 64;          // tokens of a chunk, and value columns of a block
 constexpr int kTS = kChunk + 8;     // from one row of a transposed array (or of the scores) to the next
 constexpr int kPadS = 8;            // numbers behind a row of B or C
+constexpr int kChunkThreads = 512;
 
 __device__ __forceinline__ f32x4 mma(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
@@ -257,19 +259,23 @@ __device__ __forceinline__ void store_turned(const Piece& q, bf16_t* dst) {
 template <int NT>
 constexpr size_t chunk_lds() {  // bytes
   constexpr int NP = 32 * NT, SB = NP + kPadS;
-  return sizeof(bf16_t) * (2 * kChunk * SB + NP * kTS + 3 * kChunk * kTS) + sizeof(double) * kChunk + 3 * sizeof(float) * kChunk;
+  return sizeof(bf16_t) * (2 * kChunk * SB + NP * kTS + 3 * kChunk * kTS) + sizeof(double) * kChunk +
+         3 * sizeof(float) * kChunk + 16 * 64 * sizeof(f32x4);
 }
 
 // NT: S, filled up to a multiple of 32, over 32.  VEC: S, P and the rows' width are multiples of 8, rows aligned.
 template <int NT, bool VEC>
-__global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restrict__ proj,
+__global__ __launch_bounds__(kChunkThreads) void mamba2_chunk_kernel(const bf16_t* __restrict__ proj,
                                                            const bf16_t* __restrict__ rows,
                                                            const float* __restrict__ dt_bias,
                                                            const float* __restrict__ a_log,
                                                            const float* __restrict__ skip, Memory mem,
                                                            float* __restrict__ y, Sizes z) {
   constexpr int NP = 32 * NT, SB = NP + kPadS;
-  constexpr int BP = (NT * 64 + 255) / 256;  // pieces of B a thread takes
+  constexpr int TH = kChunkThreads;
+  constexpr int BP = (NT * 64 + TH - 1) / TH;   // pieces of B a thread takes
+  constexpr int CP = (NT * 256 + TH - 1) / TH;  // eights of C
+  constexpr int KH = (NT + 1) / 2;              // 32s of a column's numbers that a wavefront holds
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
   double* s_L = reinterpret_cast<double*>(lds);               // [64] running sums of a
   float* s_d = reinterpret_cast<float*>(s_L + kChunk);        // [64] step sizes
@@ -281,6 +287,7 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
   bf16_t* xT = bT + NP * kTS;                                 // [64][kTS] this block's value columns, turned round
   bf16_t* Ph = xT + kChunk * kTS;                             // [64][kTS] weighted scores [query][key], leading term
   bf16_t* Pl = Ph + kChunk * kTS;                             // and the next
+  f32x4* sF = reinterpret_cast<f32x4*>(Pl + kChunk * kTS);    // [16][64] what two wavefronts hand each other
   const int seg = blockIdx.x, h = blockIdx.y, p0 = blockIdx.z * kChunk;
   const int tid = threadIdx.x, lane = tid & 63, w = wave_index(), c16 = lane & 15, g = lane >> 4;
   const int t_begin = mem.cu[seg], t_end = mem.cu[seg + 1];
@@ -290,43 +297,45 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
   const int grp = h / (z.H / z.G), W = z.width(), inner = z.inner();
   const float neg_rate = -expf(a_log[h]), bias = dt_bias[h], sk = skip[h];
 
-  // this wavefront's value columns: p0 + 16 w + c16; element r of M[kk][u]: number 32 kk + 8 g + 4 u + r of the column
-  const int p = p0 + 16 * w + c16;
-  const bool wave_live = p0 + 16 * w < z.P;
-  f32x4 M[NT][2];
+  // this wavefront's value columns: p0 + 16 pt + c16; element r of M[k][u]: number 32 (k0 + k) + 8 g + 4 u + r of the
+  // column; the queries whose outputs it forms: 32 hf .. 32 hf + 31 of a chunk
+  const int pt = w & 3, hf = w >> 2, k0 = hf * KH;
+  const int p = p0 + 16 * pt + c16;
+  const bool wave_live = p0 + 16 * pt < z.P;
+  f32x4 M[KH][2];
 #pragma unroll
-  for (int kk = 0; kk < NT; ++kk)
+  for (int k = 0; k < KH; ++k)
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      const int s = 32 * kk + 8 * g + 4 * u;
-      M[kk][u] = p < z.P ? load_up_to4<float, VEC>(st_in + (size_t)p * z.S + s, z.S - s) : f32x4{0.f, 0.f, 0.f, 0.f};
+      const int s = 32 * (k0 + k) + 8 * g + 4 * u;
+      M[k][u] = p < z.P ? load_up_to4<float, VEC>(st_in + (size_t)p * z.S + s, z.S - s) : f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
   // the next chunk's rows, asked for while this chunk is worked on
   Piece nB[BP], nX;
-  uint4 nC[NT];
+  uint4 nC[CP];
   float nd = 0.f;
   auto fetch = [&](int t0) {
     const int n = min(kChunk, t_end - t0);
     const bf16_t* base = rows + (size_t)t0 * W;
 #pragma unroll
     for (int i = 0; i < BP; ++i) {
-      const int idx = tid + 256 * i;
+      const int idx = tid + TH * i;
       const int s4 = (idx & 15) * 4, c8 = (idx >> 4) * 8;
       if (idx < NT * 64) nB[i] = load_piece<VEC>(base + (size_t)s4 * W + inner + grp * z.S + c8, W, n - s4, z.S - c8);
     }
     {
-      const int s4 = (tid & 15) * 4, c8 = (tid >> 4) * 8;
-      if (tid < 128) nX = load_piece<VEC>(base + (size_t)s4 * W + h * z.P + p0 + c8, W, n - s4, z.P - p0 - c8);
+      const int s4 = (tid & 15) * 4, c8 = ((tid >> 4) & 7) * 8;
+      if (w >= 4 && w < 6) nX = load_piece<VEC>(base + (size_t)s4 * W + h * z.P + p0 + c8, W, n - s4, z.P - p0 - c8);
     }
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int idx = tid + 256 * i;
+    for (int i = 0; i < CP; ++i) {
+      const int idx = tid + TH * i;
       const int s = idx / (4 * NT), c8 = (idx - s * (4 * NT)) * 8;
       nC[i] = uint4{0u, 0u, 0u, 0u};
       if (s < n) nC[i] = load8<VEC>(base + (size_t)s * W + inner + (z.G + grp) * z.S + c8, z.S - c8);
     }
-    if (tid < 64 && tid < n) nd = Num<bf16_t>::load(proj + (size_t)(t0 + tid) * z.ld + z.dt_off + h);
+    if (w == 7 && lane < n) nd = Num<bf16_t>::load(proj + (size_t)(t0 + lane) * z.ld + z.dt_off + h);
   };
   if (t_begin < t_end) fetch(t_begin);
   for (int t0 = t_begin; t0 < t_end; t0 += kChunk) {
@@ -334,7 +343,7 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
     // the chunk into shared memory
 #pragma unroll
     for (int i = 0; i < BP; ++i) {
-      const int idx = tid + 256 * i;
+      const int idx = tid + TH * i;
       const int s4 = (idx & 15) * 4, c8 = (idx >> 4) * 8;
       if (idx < NT * 64) {
 #pragma unroll
@@ -342,14 +351,14 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
         store_turned(nB[i], bT + c8 * kTS + s4);
       }
     }
-    if (tid < 128) store_turned(nX, xT + (tid >> 4) * 8 * kTS + (tid & 15) * 4);
+    if (w >= 4 && w < 6) store_turned(nX, xT + ((tid >> 4) & 7) * 8 * kTS + (tid & 15) * 4);
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int idx = tid + 256 * i;
+    for (int i = 0; i < CP; ++i) {
+      const int idx = tid + TH * i;
       const int s = idx / (4 * NT), c8 = (idx - s * (4 * NT)) * 8;
-      *reinterpret_cast<uint4*>(sC + s * SB + c8) = nC[i];
+      if (s < kChunk) *reinterpret_cast<uint4*>(sC + s * SB + c8) = nC[i];
     }
-    if (w == 0) {
+    if (w == 7) {
       const bool ok = lane < n;
       const float d = ok ? softplus_(nd + bias) : 0.f;
       double L = (double)(neg_rate * d);
@@ -366,17 +375,17 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
     }
     __syncthreads();
     if (t0 + kChunk < t_end) fetch(t0 + kChunk);
-    // the weighted scores of this wavefront's 16 queries, key block by key block up to the diagonal (and zeros up to
-    // the end of the 32 keys that a product takes at a time)
-    if (16 * w < n) {
-      const int t = 16 * w + c16;
+    // the weighted scores of 16 queries (two wavefronts share them, every other key block each), key block by key block
+    // up to the diagonal, and zeros up to the end of the 32 keys that a product takes at a time
+    if (16 * pt < n) {
+      const int t = 16 * pt + c16;
       const double Lt = s_L[t];
       bf16x8 cq[NT];
 #pragma unroll
       for (int kk = 0; kk < NT; ++kk) cq[kk] = piece(sC + t * SB + 32 * kk + 8 * g);
-      for (int sb = 0; sb <= (w | 1); ++sb) {
+      for (int sb = hf; sb <= (pt | 1); sb += 2) {
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        if (sb <= w) {
+        if (sb <= pt) {
 #pragma unroll
           for (int kk = 0; kk < NT; ++kk) acc = mma(piece(sB + (16 * sb + c16) * SB + 32 * kk + 8 * g), cq[kk], acc);
         }
@@ -396,17 +405,21 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
       }
     }
     __syncthreads();
+    // values of this wavefront's columns, a column a lane row: tokens 32 ks + 8 g .. + 7
+    bf16x8 xa[2];
+    f32x4 inside[2];  // the chunk's own part of this wavefront's two query tiles
+    f32x4 mine[2];    // this wavefront's half of the memory's part of them
     if (wave_live) {
-      // values of this wavefront's columns, a column a lane row: tokens 32 ks + 8 g .. + 7
-      bf16x8 xa[2];
 #pragma unroll
-      for (int ks = 0; ks < 2; ++ks) xa[ks] = piece(xT + (16 * w + c16) * kTS + 32 * ks + 8 * g);
+      for (int ks = 0; ks < 2; ++ks) xa[ks] = piece(xT + (16 * pt + c16) * kTS + 32 * ks + 8 * g);
       f32x4 front[4];  // S0^T C_t of the four query tiles (rows: value columns)
 #pragma unroll
       for (int tt = 0; tt < 4; ++tt) front[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int kk = 0; kk < NT; ++kk) {
-        float v[8] = {M[kk][0][0], M[kk][0][1], M[kk][0][2], M[kk][0][3], M[kk][1][0], M[kk][1][1], M[kk][1][2], M[kk][1][3]};
+      for (int k = 0; k < KH; ++k) {
+        const int kk = k0 + k;
+        if (kk >= NT) break;
+        float v[8] = {M[k][0][0], M[k][0][1], M[k][0][2], M[k][0][3], M[k][1][0], M[k][1][1], M[k][1][2], M[k][1][3]};
         const bf16x8 m_hi = take_term(v), m_lo = pack8(v);
 #pragma unroll
         for (int tt = 0; tt < 4; ++tt) {
@@ -415,25 +428,40 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
           front[tt] = mma(m_hi, c, front[tt]);
         }
       }
+      // the other wavefront's queries' part goes to it, its comes back behind the barrier
 #pragma unroll
-      for (int tt = 0; tt < 4; ++tt) {
-        if (16 * tt >= n) break;
-        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        const int t = 16 * tt + c16;
+      for (int i = 0; i < 2; ++i) {
+        mine[i] = hf == 0 ? front[i] : front[2 + i];
+        sF[(w * 2 + i) * 64 + lane] = hf == 0 ? front[2 + i] : front[i];
+      }
 #pragma unroll
-        for (int ks = 0; ks <= tt / 2; ++ks) {
-          acc = mma(xa[ks], piece(Pl + t * kTS + 32 * ks + 8 * g), acc);
-          acc = mma(xa[ks], piece(Ph + t * kTS + 32 * ks + 8 * g), acc);
+      for (int i = 0; i < 2; ++i) {
+        inside[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        const int t = 32 * hf + 16 * i + c16;
+        if (32 * hf + 16 * i >= n) continue;
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks) {
+          if (ks > hf) break;
+          inside[i] = mma(xa[ks], piece(Pl + t * kTS + 32 * ks + 8 * g), inside[i]);
+          inside[i] = mma(xa[ks], piece(Ph + t * kTS + 32 * ks + 8 * g), inside[i]);
         }
+      }
+    }
+    __syncthreads();
+    if (wave_live) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int t = 32 * hf + 16 * i + c16;
         if (t < n) {
           const float e = s_e[t];
+          const f32x4 other = sF[((w ^ 4) * 2 + i) * 64 + lane];
           f32x4 o;
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const float x = bf16_to_float(xT[(16 * w + 4 * g + r) * kTS + t]);
-            o[r] = fmaf(e, front[tt][r], acc[r]) + sk * x;
+            const float x = bf16_to_float(xT[(16 * pt + 4 * g + r) * kTS + t]);
+            o[r] = fmaf(e, mine[i][r] + other[r], inside[i][r]) + sk * x;
           }
-          const int pc = p0 + 16 * w + 4 * g;
+          const int pc = p0 + 16 * pt + 4 * g;
           float* dst = y + (size_t)(t0 + t) * inner + h * z.P + pc;
           if (VEC) {
             if (pc < z.P) *reinterpret_cast<f32x4*>(dst) = o;
@@ -447,9 +475,9 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
       // the memory behind the chunk
       const float fade = s_e[kChunk - 1];
 #pragma unroll
-      for (int kk = 0; kk < NT; ++kk)
+      for (int k = 0; k < KH; ++k)
 #pragma unroll
-        for (int u = 0; u < 2; ++u) M[kk][u] *= fade;
+        for (int u = 0; u < 2; ++u) M[k][u] *= fade;
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         if (32 * ks >= n) break;
@@ -461,14 +489,15 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
           v[j] = __uint_as_float((j & 1) ? (xw[j >> 1] & 0xffff0000u) : (xw[j >> 1] << 16)) * s_w[32 * ks + 8 * g + j];
         const bf16x8 v1 = take_term(v), v2 = take_term(v), v3 = pack8(v);
 #pragma unroll
-        for (int kk = 0; kk < NT; ++kk)
+        for (int k = 0; k < KH; ++k)
 #pragma unroll
           for (int u = 0; u < 2; ++u) {
-            const int s = 32 * kk + 8 * (c16 >> 2) + 4 * u + (c16 & 3);
+            if (k0 + k >= NT) break;
+            const int s = 32 * (k0 + k) + 8 * (c16 >> 2) + 4 * u + (c16 & 3);
             const bf16x8 b = piece(bT + s * kTS + 32 * ks + 8 * g);
-            M[kk][u] = mma(b, v3, M[kk][u]);
-            M[kk][u] = mma(b, v2, M[kk][u]);
-            M[kk][u] = mma(b, v1, M[kk][u]);
+            M[k][u] = mma(b, v3, M[k][u]);
+            M[k][u] = mma(b, v2, M[k][u]);
+            M[k][u] = mma(b, v1, M[k][u]);
           }
       }
     }
@@ -476,17 +505,17 @@ __global__ __launch_bounds__(256) void mamba2_chunk_kernel(const bf16_t* __restr
   }
   if (p < z.P) {
 #pragma unroll
-    for (int kk = 0; kk < NT; ++kk)
+    for (int k = 0; k < KH; ++k)
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        const int s = 32 * kk + 8 * g + 4 * u;
+        const int s = 32 * (k0 + k) + 8 * g + 4 * u;
         float* dst = st_out + (size_t)p * z.S + s;
         if (VEC) {
-          if (s < z.S) *reinterpret_cast<f32x4*>(dst) = M[kk][u];
+          if (s < z.S) *reinterpret_cast<f32x4*>(dst) = M[k][u];
         } else {
 #pragma unroll
           for (int e = 0; e < 4; ++e)
-            if (s + e < z.S) dst[e] = M[kk][u][e];
+            if (s + e < z.S) dst[e] = M[k][u][e];
         }
       }
   }
@@ -594,7 +623,7 @@ int launch_chunks(const bf16_t* proj, const bf16_t* rows, const float* dt_bias, 
     if (e != hipSuccess) return (int)e;
     allowed = true;
   }
-  hipLaunchKernelGGL((mamba2_chunk_kernel<NT, VEC>), dim3(R, z.H, (z.P + kChunk - 1) / kChunk), dim3(256), smem, s, proj,
+  hipLaunchKernelGGL((mamba2_chunk_kernel<NT, VEC>), dim3(R, z.H, (z.P + kChunk - 1) / kChunk), dim3(kChunkThreads), smem, s, proj,
                      rows, dt_bias, a_log, skip, mem, y, z);
   JLE_LAUNCH_CHECK();
   return 0;
