@@ -208,34 +208,34 @@ __device__ __forceinline__ bf16x8 take_term(float* v) {
   return t;
 }
 
-// Four rows of eight neighbouring numbers (a piece of B or x, to be stored both ways round), or fewer where the
-// chunk or the row ends (zeros then).
+// Eight neighbouring numbers.  VEC: what lies past the end is read from the end instead (one load, no branch, so that
+// nothing waits for it before it is used) and made zero by `there` when it has come; else only what is there is read.
+template <bool VEC>
+__device__ __forceinline__ uint4 load8(const bf16_t* row, int col, int cols) {
+  if (VEC) return *reinterpret_cast<const uint4*>(row + min(col, cols - 8));
+  uint32_t w[4] = {0u, 0u, 0u, 0u};
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+    if (col + i < cols) w[i >> 1] |= (uint32_t)row[col + i] << (16 * (i & 1));
+  return uint4{w[0], w[1], w[2], w[3]};
+}
+__device__ __forceinline__ uint4 there(uint4 v, bool ok) {
+  return uint4{ok ? v.x : 0u, ok ? v.y : 0u, ok ? v.z : 0u, ok ? v.w : 0u};
+}
+// Four rows of them (a piece of B or x, to be stored both ways round)
 struct Piece {
   uint4 r[4];
 };
 template <bool VEC>
-__device__ __forceinline__ uint4 load8(const bf16_t* p, int count) {
-  uint4 v = {0u, 0u, 0u, 0u};
-  if (VEC) {
-    if (count > 0) v = *reinterpret_cast<const uint4*>(p);
-  } else {
-    uint32_t w[4] = {0u, 0u, 0u, 0u};
-#pragma unroll
-    for (int i = 0; i < 8; ++i)
-      if (i < count) w[i >> 1] |= (uint32_t)p[i] << (16 * (i & 1));
-    v = uint4{w[0], w[1], w[2], w[3]};
-  }
-  return v;
-}
-template <bool VEC>
-__device__ __forceinline__ Piece load_piece(const bf16_t* first, size_t width, int rows_left, int count) {
+__device__ __forceinline__ Piece load_piece(const bf16_t* rows, size_t width, int row, int n, int col, int cols) {
   Piece q;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    q.r[i] = uint4{0u, 0u, 0u, 0u};
-    if (i < rows_left) q.r[i] = load8<VEC>(first + i * width, count);
-  }
+  for (int i = 0; i < 4; ++i) q.r[i] = load8<VEC>(rows + (size_t)min(row + i, n - 1) * width, col, cols);
   return q;
+}
+__device__ __forceinline__ void piece_there(Piece& q, int row, int n, bool cols_there) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) q.r[i] = there(q.r[i], cols_there && row + i < n);
 }
 // dst[column][row .. row + 3]: the piece turned round, eight stores of four numbers
 __device__ __forceinline__ void store_turned(const Piece& q, bf16_t* dst) {
@@ -256,6 +256,31 @@ __device__ __forceinline__ void store_turned(const Piece& q, bf16_t* dst) {
   }
 }
 
+// the sum over the lanes up to and including this one, by lane permutations that ride on an operand (rows of 16 lanes,
+// then the rows' and the halves' last lanes handed on)
+template <int CTRL, int ROWS>
+__device__ __forceinline__ double moved_up(double v) {
+  const unsigned long long u = __double_as_longlong(v);
+  const uint32_t lo = (uint32_t)__builtin_amdgcn_update_dpp(0, (int)(uint32_t)u, CTRL, ROWS, 0xf, false);
+  const uint32_t hi = (uint32_t)__builtin_amdgcn_update_dpp(0, (int)(uint32_t)(u >> 32), CTRL, ROWS, 0xf, false);
+  return __longlong_as_double((long long)(((unsigned long long)hi << 32) | lo));
+}
+__device__ __forceinline__ double sum_up_to_lane(double v) {
+  v += moved_up<0x111, 0xf>(v);
+  v += moved_up<0x112, 0xf>(v);
+  v += moved_up<0x114, 0xf>(v);
+  v += moved_up<0x118, 0xf>(v);
+  v += moved_up<0x142, 0xa>(v);
+  v += moved_up<0x143, 0xc>(v);
+  return v;
+}
+__device__ __forceinline__ double last_lane(double v) {
+  const unsigned long long u = __double_as_longlong(v);
+  const uint32_t lo = (uint32_t)__builtin_amdgcn_readlane((int)(uint32_t)u, 63);
+  const uint32_t hi = (uint32_t)__builtin_amdgcn_readlane((int)(uint32_t)(u >> 32), 63);
+  return __longlong_as_double((long long)(((unsigned long long)hi << 32) | lo));
+}
+
 template <int NT>
 constexpr size_t chunk_lds() {  // bytes
   constexpr int NP = 32 * NT, SB = NP + kPadS;
@@ -273,11 +298,11 @@ __global__ __launch_bounds__(kChunkThreads) void mamba2_chunk_kernel(const bf16_
                                                            float* __restrict__ y, Sizes z) {
   constexpr int NP = 32 * NT, SB = NP + kPadS;
   constexpr int TH = kChunkThreads;
-  constexpr int BP = (NT * 64 + TH - 1) / TH;   // pieces of B a thread takes
-  constexpr int CP = (NT * 256 + TH - 1) / TH;  // eights of C
-  constexpr int KH = (NT + 1) / 2;              // 32s of a column's numbers that a wavefront holds
+  constexpr int PP = (NT * 64 + 128 + TH - 1) / TH;  // pieces of B and x a thread takes
+  constexpr int CP = (NT * 256 + TH - 1) / TH;       // eights of C
+  constexpr int KH = (NT + 1) / 2;                   // 32s of a column's numbers that a wavefront holds
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
-  double* s_L = reinterpret_cast<double*>(lds);               // [64] running sums of a
+  double* s_L = reinterpret_cast<double*>(lds);               // [64] running sums of a, in units of ln 2
   float* s_d = reinterpret_cast<float*>(s_L + kChunk);        // [64] step sizes
   float* s_w = s_d + kChunk;                                  // [64] exp(L_end - L_s) d_s
   float* s_e = s_w + kChunk;                                  // [64] exp(L_t)
@@ -311,67 +336,67 @@ __global__ __launch_bounds__(kChunkThreads) void mamba2_chunk_kernel(const bf16_
       M[k][u] = p < z.P ? load_up_to4<float, VEC>(st_in + (size_t)p * z.S + s, z.S - s) : f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
-  // the next chunk's rows, asked for while this chunk is worked on
-  Piece nB[BP], nX;
+  // the next chunk's rows, asked for while this chunk is worked on.  A thread takes PP pieces of the write keys and the
+  // values (which of them: by the thread's number, without a branch, so that no load is waited for before its use)
+  Piece nP[PP];
   uint4 nC[CP];
-  float nd = 0.f;
+  bf16_t nd = 0;
   auto fetch = [&](int t0) {
     const int n = min(kChunk, t_end - t0);
     const bf16_t* base = rows + (size_t)t0 * W;
 #pragma unroll
-    for (int i = 0; i < BP; ++i) {
-      const int idx = tid + TH * i;
-      const int s4 = (idx & 15) * 4, c8 = (idx >> 4) * 8;
-      if (idx < NT * 64) nB[i] = load_piece<VEC>(base + (size_t)s4 * W + inner + grp * z.S + c8, W, n - s4, z.S - c8);
+    for (int i = 0; i < PP; ++i) {
+      const int idx = min(tid + TH * i, NT * 64 + 127);
+      const bool keys = idx < NT * 64;
+      const int at = keys ? idx : idx - NT * 64;
+      nP[i] = load_piece<VEC>(base + (keys ? inner + grp * z.S : h * z.P + p0), W, (at & 15) * 4, n, (at >> 4) * 8,
+                              keys ? z.S : z.P - p0);
     }
-    {
-      const int s4 = (tid & 15) * 4, c8 = ((tid >> 4) & 7) * 8;
-      if (w >= 4 && w < 6) nX = load_piece<VEC>(base + (size_t)s4 * W + h * z.P + p0 + c8, W, n - s4, z.P - p0 - c8);
-    }
+    nd = proj[(size_t)(t0 + min(lane, n - 1)) * z.ld + z.dt_off + h];
 #pragma unroll
     for (int i = 0; i < CP; ++i) {
       const int idx = tid + TH * i;
       const int s = idx / (4 * NT), c8 = (idx - s * (4 * NT)) * 8;
-      nC[i] = uint4{0u, 0u, 0u, 0u};
-      if (s < n) nC[i] = load8<VEC>(base + (size_t)s * W + inner + (z.G + grp) * z.S + c8, z.S - c8);
+      nC[i] = load8<VEC>(base + (size_t)min(s, n - 1) * W + inner + (z.G + grp) * z.S, c8, z.S);
     }
-    if (w == 7 && lane < n) nd = Num<bf16_t>::load(proj + (size_t)(t0 + lane) * z.ld + z.dt_off + h);
   };
+  // vmcnt(0): the memory has come (left pending, it would be waited for inside the loop, and the next chunk's rows with it)
+  __builtin_amdgcn_s_waitcnt(0x0F70);
+  asm volatile("" ::: "memory");
   if (t_begin < t_end) fetch(t_begin);
   for (int t0 = t_begin; t0 < t_end; t0 += kChunk) {
     const int n = min(kChunk, t_end - t0);
     // the chunk into shared memory
 #pragma unroll
-    for (int i = 0; i < BP; ++i) {
+    for (int i = 0; i < PP; ++i) {
       const int idx = tid + TH * i;
-      const int s4 = (idx & 15) * 4, c8 = (idx >> 4) * 8;
-      if (idx < NT * 64) {
+      const bool keys = idx < NT * 64;
+      const int at = keys ? idx : idx - NT * 64;
+      const int s4 = (at & 15) * 4, c8 = (at >> 4) * 8;
+      if (idx < NT * 64 + 128) {
+        piece_there(nP[i], s4, n, c8 < (keys ? z.S : z.P - p0));
+        store_turned(nP[i], (keys ? bT : xT) + c8 * kTS + s4);
+        if (keys) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) *reinterpret_cast<uint4*>(sB + (s4 + r) * SB + c8) = nB[i].r[r];
-        store_turned(nB[i], bT + c8 * kTS + s4);
+          for (int r = 0; r < 4; ++r) *reinterpret_cast<uint4*>(sB + (s4 + r) * SB + c8) = nP[i].r[r];
+        }
       }
     }
-    if (w >= 4 && w < 6) store_turned(nX, xT + ((tid >> 4) & 7) * 8 * kTS + (tid & 15) * 4);
 #pragma unroll
     for (int i = 0; i < CP; ++i) {
       const int idx = tid + TH * i;
       const int s = idx / (4 * NT), c8 = (idx - s * (4 * NT)) * 8;
-      if (s < kChunk) *reinterpret_cast<uint4*>(sC + s * SB + c8) = nC[i];
+      if (s < kChunk) *reinterpret_cast<uint4*>(sC + s * SB + c8) = there(nC[i], s < n && c8 < z.S);
     }
     if (w == 7) {
       const bool ok = lane < n;
-      const float d = ok ? softplus_(nd + bias) : 0.f;
-      double L = (double)(neg_rate * d);
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const double u = __shfl_up(L, o, 64);
-        if (lane >= o) L += u;
-      }
-      const double end = __shfl(L, 63, 64);  // (tokens behind the chunk's last add nothing)
+      const float d = ok ? softplus_(bf16_to_float(nd) + bias) : 0.f;
+      const double L = sum_up_to_lane((double)(neg_rate * d) * 1.4426950408889634);
+      const double end = last_lane(L);  // (tokens behind the chunk's last add nothing)
       s_L[lane] = L;
       s_d[lane] = d;
-      s_w[lane] = expf((float)(end - L)) * d;
-      s_e[lane] = expf((float)L);
+      s_w[lane] = __builtin_amdgcn_exp2f((float)(end - L)) * d;
+      s_e[lane] = __builtin_amdgcn_exp2f((float)L);
     }
     __syncthreads();
     if (t0 + kChunk < t_end) fetch(t0 + kChunk);
@@ -383,17 +408,24 @@ __global__ __launch_bounds__(kChunkThreads) void mamba2_chunk_kernel(const bf16_
       bf16x8 cq[NT];
 #pragma unroll
       for (int kk = 0; kk < NT; ++kk) cq[kk] = piece(sC + t * SB + 32 * kk + 8 * g);
-      for (int sb = hf; sb <= (pt | 1); sb += 2) {
-        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        if (sb <= pt) {
+      f32x4 acc[2];  // (both key blocks' products side by side)
 #pragma unroll
-          for (int kk = 0; kk < NT; ++kk) acc = mma(piece(sB + (16 * sb + c16) * SB + 32 * kk + 8 * g), cq[kk], acc);
-        }
+      for (int i = 0; i < 2; ++i) {
+        acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (hf + 2 * i > pt) continue;
+#pragma unroll
+        for (int kk = 0; kk < NT; ++kk)
+          acc[i] = mma(piece(sB + (16 * (hf + 2 * i) + c16) * SB + 32 * kk + 8 * g), cq[kk], acc[i]);
+      }
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int sb = hf + 2 * i;
+        if (sb > (pt | 1)) continue;
         float v[4], lo[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int s = 16 * sb + 4 * g + r;
-          v[r] = s <= t ? acc[r] * (expf((float)(Lt - s_L[s])) * s_d[s]) : 0.f;
+          v[r] = s <= t ? acc[i][r] * (__builtin_amdgcn_exp2f((float)(Lt - s_L[s])) * s_d[s]) : 0.f;
         }
         const uint2 hi = {pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3])};
         lo[0] = v[0] - __uint_as_float(hi.x << 16);
