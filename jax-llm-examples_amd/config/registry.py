@@ -94,3 +94,4 @@ def _ensure_builtin() -> None:
     from ..parts import mazotar as _mazotar  # noqa: F401
     from ..parts import sudilorn as _sudilorn  # noqa: F401
     from ..parts import folivik as _folivik  # noqa: F401
+    from ..parts import lifesun as _lifesun  # noqa: F401

@@ -135,6 +135,25 @@ class LoopConfig:
     stop: int
     times: int
 
+    @classmethod
+    def from_dict(cls, m: Mapping[str, Any], num_layers: int) -> "LoopConfig":
+        _only(m, ("start", "stop", "times"), "loop")
+        c = cls(*(int(_need(m, k, "loop")) for k in ("start", "stop", "times")))
+        if not 0 <= c.start <= c.stop <= num_layers or c.times < 1:
+            raise ConfigError(f"config.json: loop {dict(m)} does not fit {num_layers} layers")
+        return c
+
+
+def looped_order(num_layers: int, loop: Optional[LoopConfig]) -> list:
+    """``(layer, number of the pass this run starts or None)`` in the order the layers run: the looped stretch
+    ``times`` times in a row."""
+    if loop is None:
+        return [(i, None) for i in range(num_layers)]
+    order = [(i, None) for i in range(loop.start)]
+    for t in range(loop.times):
+        order += [(i, t if i == loop.start else None) for i in range(loop.start, loop.stop)]
+    return order + [(i, None) for i in range(loop.stop, num_layers)]
+
 
 _MIXERS = {"attention": ConvAttentionConfig, "latent_attention": SinkLatentAttentionConfig}
 
@@ -179,10 +198,7 @@ class TiradraConfig:
         loop = None
         lp = top.get("loop")
         if lp is not None:
-            _only(lp, ("start", "stop", "times"), "loop")
-            loop = LoopConfig(*(int(_need(lp, k, "loop")) for k in ("start", "stop", "times")))
-            if not 0 <= loop.start <= loop.stop <= len(layers) or loop.times < 1:
-                raise ConfigError(f"config.json: loop {lp} does not fit {len(layers)} layers")
+            loop = LoopConfig.from_dict(lp, len(layers))
         cap = top.get("logit_softcap")
         if cap is not None and float(cap) <= 0:
             raise ConfigError("config.json: logit_softcap must be positive")
@@ -206,14 +222,7 @@ class TiradraConfig:
     def run_order(self) -> list:
         """``(layer, number of the pass this run starts or None)`` in the order the layers run: the looped stretch
         ``times`` times in a row."""
-        n = len(self.layers)
-        if self.loop is None:
-            return [(i, None) for i in range(n)]
-        lo, hi, times = self.loop.start, self.loop.stop, self.loop.times
-        order = [(i, None) for i in range(lo)]
-        for t in range(times):
-            order += [(i, t if i == lo else None) for i in range(lo, hi)]
-        return order + [(i, None) for i in range(hi, n)]
+        return looped_order(len(self.layers), self.loop)
 
     def plan(self) -> ModelPlan:
         D, eps = self.width, self.norm_eps

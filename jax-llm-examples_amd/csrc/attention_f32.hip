@@ -11,6 +11,8 @@
 // Which steps a query visits, and the order of every sum, depend on the query's own position and the retention
 // rule only (steps are absolute multiples of 16; a step in which a query sees no key changes nothing of its
 // state), so a token's result does not depend on how the request was cut or on what else is in the step.
+// cap > 0: a scaled score s becomes cap tanh(s / cap).  sink: [Hq] or null, exp(sink[h]) is one more term of head h's
+// denominator.
 // Page layout per kv head: keys [page_size][head_dim], values [head_dim][page_size].
 #include "common.h"
 
@@ -46,7 +48,8 @@ __global__ __launch_bounds__(256) void attention_f32_tiles_kernel(
     const float* __restrict__ q, const float* __restrict__ kv, float* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
     int table_width, const int* __restrict__ tiles, int num_tiles, int ret_mode, int ret_param, float scale, int Hq,
-    int Hkv, int dh, int ps, int splits, int keys_per_split, float* __restrict__ ws_ml, float* __restrict__ ws_o) {
+    int Hkv, int dh, int ps, int splits, int keys_per_split, float* __restrict__ ws_ml, float* __restrict__ ws_o,
+    float cap, const float* __restrict__ sink) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + wave_index();
   const int c16 = lane & 15, g = lane >> 4;
@@ -140,6 +143,10 @@ __global__ __launch_bounds__(256) void attention_f32_tiles_kernel(
         s = __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, qreg[c].w, s, 0, 0, 0);
       }
     }
+    if (cap > 0.f) {  // (the same for the whole launch)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) s[v] = cap * tanhf(s[v] / cap);
+    }
     // s[v]: key key0 + 4 g + v, query c16.  A key a query may read whose page is not there is an error.
     float p[4];
     float mx = -INFINITY;
@@ -223,6 +230,7 @@ __global__ __launch_bounds__(256) void attention_f32_tiles_kernel(
       if (t < dt) *reinterpret_cast<float4*>(ws_o + slot * dh + 16 * t + 4 * g) = float4{acc[t][0], acc[t][1], acc[t][2], acc[t][3]};
     return;
   }
+  if (sink != nullptr) l += expf(sink[HEADS ? h + c16 : h] - m);  // one more term of the denominator, without a value
   const float inv = bad ? __builtin_nanf("") : 1.0f / l;
   float* o = out + col0 + (size_t)c16 * col_stride + 4 * g;
 #pragma unroll
@@ -239,8 +247,9 @@ __global__ __launch_bounds__(256) void attention_f32_tiles_kernel(
 JLE_API int jle_attention_f32_tiles(const float* q, const float* kv, float* out, const int* positions,
                                     const int* token_segment, const int* block_table, int table_width,
                                     const int* tiles, int num_tiles, int ret_mode, int ret_param, float scale, int Hq,
-                                    int Hkv, int dh, int ps, hipStream_t s) {
+                                    int Hkv, int dh, int ps, float cap, const float* sink, hipStream_t s) {
   if (num_tiles <= 0) return 0;
+  if (cap < 0.f) return JLE_BAD_ARG;
   if (dh % 16 || dh > 256 || dh <= 0 || ps % 16 || ps <= 0 || Hkv <= 0 || Hq % Hkv) return JLE_BAD_ARG;
   if ((ret_mode == 1 || ret_mode == 2) && ret_param <= 0) return JLE_BAD_ARG;
   if (ret_mode < 0 || ret_mode > 2 || tiles == nullptr) return JLE_BAD_ARG;
@@ -251,7 +260,7 @@ JLE_API int jle_attention_f32_tiles(const float* q, const float* kv, float* out,
 #define LAUNCH_A(DT)                                                                                            \
   hipLaunchKernelGGL((attention_f32_tiles_kernel<DT, false>), g, b, 0, s, q, kv, out, positions, token_segment, \
                      block_table, table_width, tiles, num_tiles, ret_mode, ret_param, scale, Hq, Hkv, dh, ps, 1, 0, \
-                     nullptr, nullptr)
+                     nullptr, nullptr, cap, sink)
   if (dh <= 64) LAUNCH_A(4);
   else if (dh <= 128) LAUNCH_A(8);
   else LAUNCH_A(16);
@@ -263,12 +272,14 @@ JLE_API int jle_attention_f32_tiles(const float* q, const float* kv, float* out,
 // The same for a step of N single tokens: a wavefront takes the query heads of one kv head (at most 16) and
 // keys_per_split keys (a multiple of 16; splits of them cover the longest range of keys any token reads).  With
 // splits > 1 the results go to ws_ml [N * Hq * splits * 2] and ws_o [N * Hq * splits * dh], in the layout of
-// jle_paged_attention_generic's, for the caller to merge (jle_attention_merge).
+// jle_paged_attention_generic's, for the caller to merge (jle_attention_merge, which then adds the sinks' terms).
 JLE_API int jle_attention_f32_heads(const float* q, const float* kv, float* out, const int* positions,
                                     const int* token_segment, const int* block_table, int table_width, int N,
                                     int ret_mode, int ret_param, float scale, int Hq, int Hkv, int dh, int ps,
-                                    int splits, int keys_per_split, float* ws_ml, float* ws_o, hipStream_t s) {
+                                    int splits, int keys_per_split, float* ws_ml, float* ws_o, float cap,
+                                    const float* sink, hipStream_t s) {
   if (N <= 0) return 0;
+  if (cap < 0.f) return JLE_BAD_ARG;
   if (dh % 16 || dh > 256 || dh <= 0 || ps % 16 || ps <= 0 || Hkv <= 0 || Hq % Hkv || Hq / Hkv > 16) return JLE_BAD_ARG;
   if ((ret_mode == 1 || ret_mode == 2) && ret_param <= 0) return JLE_BAD_ARG;
   if (ret_mode < 0 || ret_mode > 2) return JLE_BAD_ARG;
@@ -281,7 +292,7 @@ JLE_API int jle_attention_f32_heads(const float* q, const float* kv, float* out,
 #define LAUNCH_H(DT)                                                                                           \
   hipLaunchKernelGGL((attention_f32_tiles_kernel<DT, true>), g, b, 0, s, q, kv, out, positions, token_segment, \
                      block_table, table_width, nullptr, N, ret_mode, ret_param, scale, Hq, Hkv, dh, ps, splits, \
-                     keys_per_split, ws_ml, ws_o)
+                     keys_per_split, ws_ml, ws_o, cap, sink)
   if (dh <= 64) LAUNCH_H(4);
   else if (dh <= 128) LAUNCH_H(8);
   else LAUNCH_H(16);

@@ -45,7 +45,7 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
     const int* __restrict__ token_segment, const int* __restrict__ block_table, int table_width, int ret_mode,
     int ret_param, float scale, int N, int Hq, int Hkv, int dh, int ps, int splits, int tiles_per_split,
     float* __restrict__ ws_ml, float* __restrict__ ws_o, const float* __restrict__ bias, int bias_len,
-    const float* __restrict__ sink, int keep) {
+    const float* __restrict__ sink, int keep, float cap) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + wave_index();
   if (item >= N * Hq * splits) return;  // whole wavefront leaves; no block-wide barrier below
@@ -100,6 +100,7 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
           for (int i = 0; i < Vec16<T>::kN; ++i) dot += qv.get(i) * kvv.get(i);
         }
         s = dot * scale;
+        if (cap > 0.f) s = cap * tanhf(s / cap);
         // a learned number per head and distance; every key further back than the table is long takes its last entry
         // (a negative length: a penalty that grows with the distance, two numbers per head)
         if (bias_len < 0) s -= bias[2 * h] * log1pf(bias[2 * h + 1] * (float)(pos - key));
@@ -252,13 +253,14 @@ __global__ __launch_bounds__(256) void paged_attention_generic_merge_kernel(cons
 // splits > 1 (few tokens with many keys: decode): every (token, head) is shared between `splits` wavefronts,
 // tiles_per_split tiles of 64 keys each, and merged by a second kernel; ws_ml: [N * Hq * splits * 2] float32,
 // ws_o: [N * Hq * splits * dh] float32.  splits * tiles_per_split must cover the longest range of keys.
+// cap > 0: a scaled score s becomes cap tanh(s / cap).
 // bias: float32 [Hq][bias_len] or null: a key n places back adds bias[h][min(n, bias_len - 1)] to head h's scaled
 // score (bias_len < 0: bias is [Hq][2], and bias[h][0] * ln(1 + bias[h][1] * n) is taken off it); sink: float32 [Hq] or null: exp(sink[h]) is one more term of head h's denominator.
 static int launch_generic(const void* q, const void* kv, void* out, const int* positions, const int* token_segment,
                           const int* block_table, int table_width, int ret_mode, int ret_param, float scale,
                           int is_bf16, int N, int Hq, int Hkv, int dh, int ps, int splits, int tiles_per_split,
                           float* ws_ml, float* ws_o, const float* bias, int bias_len, const float* sink,
-                          hipStream_t s, int keep = 0) {
+                          hipStream_t s, int keep = 0, float cap = 0.f) {
   if (N <= 0) return 0;
   if (keep < 0) return JLE_BAD_ARG;
   if ((bias == nullptr) != (bias_len == 0)) return JLE_BAD_ARG;
@@ -272,7 +274,8 @@ static int launch_generic(const void* q, const void* kv, void* out, const int* p
   if (is_bf16) {
     hipLaunchKernelGGL(paged_attention_generic_kernel<bf16_t>, g, b, 0, s, (const bf16_t*)q, (const bf16_t*)kv,
                        (bf16_t*)out, positions, token_segment, block_table, table_width, ret_mode, ret_param, scale,
-                       N, Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, keep);
+                       N, Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, keep,
+                       cap);
     JLE_LAUNCH_CHECK();
     if (splits > 1)
       hipLaunchKernelGGL(paged_attention_generic_merge_kernel<bf16_t>, gm, b, 0, s, ws_ml, ws_o, (bf16_t*)out, N * Hq,
@@ -280,7 +283,8 @@ static int launch_generic(const void* q, const void* kv, void* out, const int* p
   } else {
     hipLaunchKernelGGL(paged_attention_generic_kernel<float>, g, b, 0, s, (const float*)q, (const float*)kv,
                        (float*)out, positions, token_segment, block_table, table_width, ret_mode, ret_param, scale, N,
-                       Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, keep);
+                       Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, keep,
+                       cap);
     JLE_LAUNCH_CHECK();
     if (splits > 1)
       hipLaunchKernelGGL(paged_attention_generic_merge_kernel<float>, gm, b, 0, s, ws_ml, ws_o, (float*)out, N * Hq, dh,
@@ -303,9 +307,10 @@ JLE_API int jle_paged_attention_biased(const void* q, const void* kv, void* out,
                                        const int* token_segment, const int* block_table, int table_width,
                                        int ret_mode, int ret_param, float scale, int is_bf16, int N, int Hq, int Hkv,
                                        int dh, int ps, int splits, int tiles_per_split, float* ws_ml, float* ws_o,
-                                       const float* bias, int bias_len, const float* sink, hipStream_t s) {
+                                       const float* bias, int bias_len, const float* sink, float cap, hipStream_t s) {
+  if (cap < 0.f) return JLE_BAD_ARG;
   return launch_generic(q, kv, out, positions, token_segment, block_table, table_width, ret_mode, ret_param, scale,
-                        is_bf16, N, Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, s);
+                        is_bf16, N, Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, bias, bias_len, sink, s, 0, cap);
 }
 
 // The same under a rule that also keeps the sequence's first `keep` keys visible (a window with kept first tokens).
@@ -317,18 +322,19 @@ JLE_API int jle_paged_attention_kept(const void* q, const void* kv, void* out, c
                         is_bf16, N, Hq, Hkv, dh, ps, splits, tiles_per_split, ws_ml, ws_o, nullptr, 0, nullptr, s, keep);
 }
 
-// The merge alone, for kernels that leave their key ranges' results in the same layout (attention_f32.hip).
+// The merge alone, for kernels that leave their key ranges' results in the same layout (attention_f32.hip).  sink:
+// [Hq] or null (NH: tokens times Hq).
 JLE_API int jle_attention_merge(const float* ws_ml, const float* ws_o, void* out, int is_bf16, int NH, int dh,
-                                int splits, hipStream_t s) {
+                                int splits, const float* sink, int Hq, hipStream_t s) {
   if (NH <= 0) return 0;
-  if (splits < 1 || dh <= 0 || dh > 256 || ws_ml == nullptr || ws_o == nullptr) return JLE_BAD_ARG;
+  if (splits < 1 || dh <= 0 || dh > 256 || Hq < 1 || ws_ml == nullptr || ws_o == nullptr) return JLE_BAD_ARG;
   dim3 gm((unsigned)(((long long)NH + 3) / 4)), b(256);
   if (is_bf16)
     hipLaunchKernelGGL(paged_attention_generic_merge_kernel<bf16_t>, gm, b, 0, s, ws_ml, ws_o, (bf16_t*)out, NH, dh, splits,
-                       nullptr, 1);
+                       sink, Hq);
   else
     hipLaunchKernelGGL(paged_attention_generic_merge_kernel<float>, gm, b, 0, s, ws_ml, ws_o, (float*)out, NH, dh, splits,
-                       nullptr, 1);
+                       sink, Hq);
   JLE_LAUNCH_CHECK();
   return 0;
 }

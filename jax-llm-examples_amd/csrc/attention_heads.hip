@@ -4,7 +4,7 @@
 // once for each of the `share` key heads that use it: two score maps over the same values), an RMS norm of q and k
 // with or without weights before or behind the rotation, the rotation over adjacent or half-split pairs of the
 // leading elements with a magnitude on sines and cosines.
-//     rows [N, Hq dk + Hk dk + Hv dv]  ->  q_out [N, Hq, D],  pages [.., 2, Hk, ps, D] (values [D][ps])
+//     rows [N, Hq dk + Hk dk + Hv dv] (or the leading part of wider rows)  ->  q_out [N, Hq, D],  pages [.., 2, Hk, ps, D] (values [D][ps])
 // and the combination of two score maps' outputs into one head's:
 //     d = a1 - lam a2;  d / sqrt(mean(d^2) + eps) * scale * sigmoid(gate)
 // One wavefront per (token, head); a lane holds elements lane, lane + 64, ...  Everything in float32; the order of
@@ -29,6 +29,7 @@ struct HeadsArgs {
   T* kv_cache;  // or null
   float magnitude, norm_eps;  // norm_eps < 0: no norm
   int rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps;
+  int ld;         // from one row to the next (at least their width)
   int wq_stride;  // from one query head's norm weights to the next's (0: one for all)
 };
 
@@ -38,10 +39,9 @@ __global__ __launch_bounds__(64) void heads_prepare_kernel(HeadsArgs<T> a) {
   const int n = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const bool is_q = h < a.Hq, is_v = h >= a.Hq + a.Hk;
   if (!is_q && a.kv_cache == nullptr) return;
-  const int C = (a.Hq + a.Hk) * a.dk + a.Hv * a.dv;
   const int dim = is_v ? a.dv : a.dk;
   const int c0 = is_v ? (a.Hq + a.Hk) * a.dk + (h - a.Hq - a.Hk) * a.dv : h * a.dk;
-  const T* src = a.rows + (size_t)n * C + c0;
+  const T* src = a.rows + (size_t)n * a.ld + c0;
   float x[kMaxPerLane];
 #pragma unroll
   for (int i = 0; i < kMaxPerLane; ++i) {
@@ -159,7 +159,7 @@ __global__ __launch_bounds__(64) void diff_combine_kernel(const T* __restrict__ 
 
 }  // namespace
 
-JLE_API int jle_heads_prepare(const void* rows, const int* positions, const int* slot_mapping, const float* inv_freq,
+JLE_API int jle_heads_prepare(const void* rows, int ld, const int* positions, const int* slot_mapping, const float* inv_freq,
                               int rotary_dim, int half_pairs, float magnitude, float norm_eps, int norm_first,
                               const float* wq, int wq_stride, const float* wk, void* q_out, void* kv_cache, int is_bf16, int N, int Hq,
                               int Hk, int Hv, int dk, int dv, int D, int ps, hipStream_t s) {
@@ -171,14 +171,15 @@ JLE_API int jle_heads_prepare(const void* rows, const int* positions, const int*
     return JLE_BAD_ARG;
   if (kv_cache != nullptr && slot_mapping == nullptr) return JLE_BAD_ARG;
   if (wq_stride != 0 && wq_stride != dk) return JLE_BAD_ARG;
+  if (ld < (Hq + Hk) * dk + Hv * dv) return JLE_BAD_ARG;
   const dim3 grid(N, Hq + Hk + Hv);
   if (is_bf16) {
     HeadsArgs<bf16_t> a{(const bf16_t*)rows, positions, slot_mapping, inv_freq, wq, wk, (bf16_t*)q_out, (bf16_t*)kv_cache,
-                        magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, wq_stride};
+                        magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, ld, wq_stride};
     hipLaunchKernelGGL(heads_prepare_kernel<bf16_t>, grid, dim3(64), 0, s, a);
   } else {
     HeadsArgs<float> a{(const float*)rows, positions, slot_mapping, inv_freq, wq, wk, (float*)q_out, (float*)kv_cache,
-                       magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, wq_stride};
+                       magnitude, norm_eps, rotary_dim, half_pairs, norm_first, Hq, Hk, Hv, dk, dv, D, ps, ld, wq_stride};
     hipLaunchKernelGGL(heads_prepare_kernel<float>, grid, dim3(64), 0, s, a);
   }
   JLE_LAUNCH_CHECK();

@@ -53,11 +53,20 @@ struct Columns {  // per lane, for each of its column tiles
 
 // A learned number per (query head, distance) added to the scaled score: table[h][min(pos - key, L - 1)], float32.
 // Or (L < 0) a penalty that grows with the distance: table[h] = (r1, r2), r1 ln(1 + r2 (pos - key)) taken off.
+// Or a cap: a scaled score s becomes cap tanh(s / cap); cap_in = 2 log2(e) scale / cap, cap_out = cap log2(e).
 struct Biasing {
   const float* table;
   int L;
+  float cap_in, cap_out;
 };
-constexpr int kNoBias = 0, kBiasTable = 1, kBiasPenalty = 2;  // what a kernel is compiled for
+constexpr int kNoBias = 0, kBiasTable = 1, kBiasPenalty = 2, kCapped = 3;  // what a kernel is compiled for
+constexpr bool light(int biased) { return biased == kNoBias || biased == kCapped; }  // (few registers beyond the plain kernel's)
+
+// cap tanh(s / cap) in the exponent's base-2 units from an unscaled score: tanh z = 1 - 2 / (exp(2 z) + 1)
+__device__ __forceinline__ float capped_log2(float v, const Biasing& b) {
+  const float e = __builtin_amdgcn_exp2f(v * b.cap_in);
+  return fmaf(-2.0f * b.cap_out, __builtin_amdgcn_rcpf(e + 1.0f), b.cap_out);
+}
 
 // the penalty in the exponent's base-2 units: r1 ln(x) log2(e) = r1 log2(x)
 __device__ __forceinline__ float penalty_log2(float r1, float r2, float back) {
@@ -101,7 +110,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
                                                    const V4 (&vraw)[DH / 16], int kb, const Columns (&col)[CT],
                                                    int k_lo, int k_hi, float scale_log2, float (&m)[CT],
                                                    float (&l)[CT], f32x4 (&acc)[CT][DH / 16],
-                                                   Biasing bias = Biasing{nullptr, 0}, bool far = false,
+                                                   Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}, bool far = false,
                                                    const float* far_b = nullptr) {
   constexpr int DT = DH / 16;
   const int g = (threadIdx.x & 63) >> 4;
@@ -119,6 +128,7 @@ __device__ __forceinline__ void softmax_and_values(const f32x4 (&st)[CT][2], boo
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         float v = st[ct][tt][i];
+        if (BIASED == kCapped) v = capped_log2(v, bias);
         if (BIASED == kBiasPenalty)
           v = fmaf(v, scale_log2, -penalty_log2(far_b[ct], far_b[CT + ct], (float)(col[ct].pos - kb - 4 * g) - (float)(16 * tt + i)));
         if (BIASED == kBiasTable) {
@@ -267,7 +277,7 @@ __device__ __forceinline__ void attend_with(const bf16x8 (&qb)[CT][DH / 32], con
                                             const int* __restrict__ table, const Columns (&col)[CT], int k_lo,
                                             int k_hi, int hk, int Hkv, int ps, float scale_log2, float (&m)[CT],
                                             float (&l)[CT], f32x4 (&acc)[CT][DH / 16], bool& bad,
-                                            Biasing bias = Biasing{nullptr, 0}, bool fresh = true, bool close = true) {
+                                            Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}, bool fresh = true, bool close = true) {
   const int lane = threadIdx.x & 63;
   const int c16 = lane & 15, g = lane >> 4;
   constexpr int KC = DH / 32;  // k-steps of the first product
@@ -425,7 +435,7 @@ __device__ __forceinline__ void attend(const bf16_t* __restrict__ q, const bf16_
                                        const int* __restrict__ table, const Columns (&col)[CT], int k_lo, int k_hi,
                                        int hk, int Hq, int Hkv, int ps, float scale_log2, float (&m)[CT],
                                        float (&l)[CT], f32x4 (&acc)[CT][DH / 16], bool& bad,
-                                       Biasing bias = Biasing{nullptr, 0}, bool fresh = true, bool close = true) {
+                                       Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}, bool fresh = true, bool close = true) {
   bf16x8 qb[CT][DH / 32];
   load_queries<DH, CT>(q, col, Hq, qb);
   attend_with<DH, CT, ONCE, BIASED>(qb, kv, table, col, k_lo, k_hi, hk, Hkv, ps, scale_log2, m, l, acc, bad, bias,
@@ -439,11 +449,11 @@ __device__ __forceinline__ void attend(const bf16_t* __restrict__ q, const bf16_
 // BIASED: a distance bias (see Biasing) on every score and, with `sink`, one more term exp(sink[h]) in head h's
 // denominator.
 template <int DH, int CT, int BIASED = kNoBias>
-__global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && !BIASED) ? 2 : 1) void attention_prefill_kernel(
+__global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && light(BIASED)) ? 2 : 1) void attention_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, bf16_t* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
     int table_width, const int* __restrict__ tiles, int num_tiles, int ret_mode, int ret_param, float scale_log2,
-    int Hq, int Hkv, int ps, Biasing bias = Biasing{nullptr, 0}, const float* __restrict__ sink = nullptr) {
+    int Hq, int Hkv, int ps, Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}, const float* __restrict__ sink = nullptr) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + wave_index();
   if (item >= num_tiles * Hq) return;
@@ -476,7 +486,7 @@ __global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && !BIASED) ? 2 : 1) voi
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
     if (ct * 16 + c16 >= nt) continue;
-    if (BIASED && sink != nullptr) l[ct] += exp2f(sink[h] * kLog2e - m[ct]);
+    if (sink != nullptr) l[ct] += exp2f(sink[h] * kLog2e - m[ct]);
     const float inv = bad ? __builtin_nanf("") : (l[ct] > 0.f ? 1.0f / l[ct] : 0.f);
     bf16_t* o = out + ((size_t)col[ct].token * Hq + h) * DH + 4 * g;
 #pragma unroll
@@ -527,9 +537,9 @@ __global__ __launch_bounds__(256, (CT == 1 && DH <= 128) ? 2 : 1) void attention
   const int* table = block_table + (size_t)token_segment[n0] * table_width;
   if (kept_hi >= 0) {
     attend<DH, CT, false, false>(q, kv, table, kept, 0, kept_hi, hk, Hq, Hkv, ps, scale_log2, m, l, acc, bad,
-                                 Biasing{nullptr, 0}, true, false);
+                                 Biasing{nullptr, 0, 0.f, 0.f}, true, false);
     attend<DH, CT, false, false>(q, kv, table, col, k_lo, k_hi, hk, Hq, Hkv, ps, scale_log2, m, l, acc, bad,
-                                 Biasing{nullptr, 0}, false, true);
+                                 Biasing{nullptr, 0, 0.f, 0.f}, false, true);
   } else {
     attend<DH, CT, false, false>(q, kv, table, col, k_lo, k_hi, hk, Hq, Hkv, ps, scale_log2, m, l, acc, bad);
   }
@@ -559,12 +569,14 @@ __global__ __launch_bounds__(256, (CT == 1 && DH <= 128) ? 2 : 1) void attention
 // outside its own tile's range.
 //   groups: [num_groups][4] = (first tile, first head within the kv head's group of that tile, items, 0),
 //   longest first; grid = num_groups * Hkv.
-template <int DH, int WAVES>
+// BIASED: none or a cap on the scores; with `sink`, one more term exp(sink[h]) in head h's denominator.
+template <int DH, int WAVES, int BIASED>
 __global__ __launch_bounds__(WAVES * 64, DH <= 128 ? 2 : 1) void attention_prefill_shared_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, bf16_t* __restrict__ out,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
     int table_width, const int* __restrict__ tiles, const int* __restrict__ groups, int ret_mode, int ret_param,
-    float scale_log2, int Hq, int Hkv, int ps) {
+    float scale_log2, int Hq, int Hkv, int ps, Biasing bias, const float* __restrict__ sink) {
+  static_assert(light(BIASED), "the kernels that share keys through registers take a cap, no bias");
   constexpr int CT = 2, KC = DH / 32, DT = DH / 16;
   constexpr int KP = DH + 8;
   constexpr int THREADS = WAVES * 64;
@@ -766,10 +778,12 @@ __global__ __launch_bounds__(WAVES * 64, DH <= 128 ? 2 : 1) void attention_prefi
           vraw[dt] = uint4{t0.x, t0.y, t1.x, t1.y};
         }
         if (kb >= all_lo && kb + 31 <= all_hi) {  // the same for the whole wavefront
-          softmax_and_values<DH, CT, false>(st, true, true, vraw, kb, col, k_lo, k_hi, scale_log2, m, l, acc);
+          softmax_and_values<DH, CT, false, uint4, BIASED>(st, true, true, vraw, kb, col, k_lo, k_hi, scale_log2, m, l, acc,
+                                                           bias);
         } else {
           const bool act0 = kb <= k_hi && kb + 15 >= k_lo, act1 = kb + 16 <= k_hi && kb + 31 >= k_lo;
-          softmax_and_values<DH, CT, true>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l, acc);
+          softmax_and_values<DH, CT, true, uint4, BIASED>(st, act0, act1, vraw, kb, col, k_lo, k_hi, scale_log2, m, l, acc,
+                                                          bias);
         }
       }
       buf ^= 1;
@@ -779,7 +793,8 @@ __global__ __launch_bounds__(WAVES * 64, DH <= 128 ? 2 : 1) void attention_prefi
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
     if (ct * 16 + c16 >= nt) continue;
-    const float sum = column_sum(l[ct]);
+    float sum = column_sum(l[ct]);
+    if (sink != nullptr) sum += exp2f(sink[h] * kLog2e - m[ct]);
     const float inv = bad ? __builtin_nanf("") : (sum > 0.f ? 1.0f / sum : 0.f);
     bf16_t* o = out + ((size_t)col[ct].token * Hq + h) * DH + 4 * g;
 #pragma unroll
@@ -830,7 +845,7 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
                                                      const unsigned char* sv, uint32_t v_rd, int tile_bytes, int kb,
                                                      const Columns (&col)[CT], int k_lo, int k_hi, float scale_log2,
                                                      float (&m)[CT], float (&l)[CT], f32x4 (&acc)[CT][DH / 16],
-                                                     Biasing bias = Biasing{nullptr, 0}, bool far = false,
+                                                     Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}, bool far = false,
                                                      const float* far_b = nullptr) {
   constexpr int DT = DH / 16;
   const int g = (threadIdx.x & 63) >> 4;
@@ -847,6 +862,10 @@ __device__ __forceinline__ void softmax64_and_values(f32x4 (&st)[CT][4], int hal
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         float v = st[ct][tt][i];
+        if (BIASED == kCapped) {
+          v = capped_log2(v, bias);
+          st[ct][tt][i] = v;
+        }
         if (BIASED == kBiasPenalty) {
           v = fmaf(v, scale_log2, -penalty_log2(far_b[ct], far_b[CT + ct], (float)(col[ct].pos - kb - 8 * g) -
                                                                                (float)(32 * (tt >> 1) + 4 * (tt & 1) + i)));
@@ -1154,7 +1173,7 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
   for (int ct = 0; ct < CT; ++ct) {
     if (ct * 16 + c16 >= nt) continue;
     float sum = column_sum(l[ct]);
-    if (BIASED && sink != nullptr) sum += exp2f(sink[h] * kLog2e - m[ct]);
+    if (sink != nullptr) sum += exp2f(sink[h] * kLog2e - m[ct]);
     const float inv = bad ? __builtin_nanf("") : (sum > 0.f ? 1.0f / sum : 0.f);
     bf16_t* o = out + ((size_t)col[ct].token * Hq + h) * DH + 4 * g;
 #pragma unroll
@@ -1171,11 +1190,11 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_lds_kernel(
 // (decode token, kv head, key range); ws_ml: [item][16 * CT][2], ws_o: [item][16 * CT][DH],
 // item = (d * Hkv + hk) * max_splits + split.
 template <int DH, int CT, int BIASED = kNoBias>
-__global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && !BIASED) ? 2 : 1) void attention_decode_kernel(
+__global__ __launch_bounds__(256, (CT == 1 && DH <= 128 && light(BIASED)) ? 2 : 1) void attention_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, float* __restrict__ ws_ml, float* __restrict__ ws_o,
     const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_table,
     int table_width, const int* __restrict__ dec_tokens, int num_dec, int max_splits, int kSplit, int ret_mode,
-    int ret_param, float scale_log2, int Hq, int Hkv, int ps, Biasing bias = Biasing{nullptr, 0}) {
+    int ret_param, float scale_log2, int Hq, int Hkv, int ps, Biasing bias = Biasing{nullptr, 0, 0.f, 0.f}) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + wave_index();
   if (item >= num_dec * Hkv * max_splits) return;
@@ -1584,13 +1603,14 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
                                   const int* token_segment, const int* block_table, int table_width, const int* tiles,
                                   int num_tiles, int tile_tokens, const int* groups, int num_groups, int ret_mode,
                                   int ret_param, float scale, int Hq, int Hkv, int dh, int ps, const float* bias,
-                                  int bias_len, const float* sink, hipStream_t s) {
+                                  int bias_len, const float* sink, float cap, hipStream_t s) {
   if (num_tiles <= 0) return 0;
   if (!jle_attention_mfma_supported(dh, Hq, Hkv, ps)) return JLE_BAD_ARG;
-  // bias: [Hq][bias_len] (with a sink and no bias: a table of zeros), or bias_len < 0: a penalty's [Hq][2]; the kernels that share keys take neither
-  if ((bias == nullptr) != (bias_len == 0) || (sink != nullptr && bias == nullptr)) return JLE_BAD_ARG;
+  // bias: [Hq][bias_len], or bias_len < 0: a penalty's [Hq][2] (the kernels that share keys take neither, but at heads of
+  // 128); cap > 0: a cap on the scaled scores (then no bias); sink: [Hq] or null
+  if ((bias == nullptr) != (bias_len == 0) || cap < 0.f || (cap > 0.f && bias != nullptr)) return JLE_BAD_ARG;
   if (bias != nullptr && groups != nullptr && dh != 128) return JLE_BAD_ARG;  // (of those, the kernel for 128 alone)
-  const Biasing bs = {bias, bias_len};
+  const Biasing bs = {bias, bias_len, cap > 0.f ? 2.0f * kLog2e * scale / cap : 0.f, cap * kLog2e};
   if ((ret_mode == 1 || ret_mode == 2) && ret_param <= 0) return JLE_BAD_ARG;
   const long long items = (long long)num_tiles * Hq;
   dim3 g((unsigned)((items + 3) / 4)), b(256);
@@ -1599,11 +1619,15 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
   if (groups != nullptr) {
     if (tile_tokens != 32 || num_groups <= 0) return JLE_BAD_ARG;
     dim3 gs((unsigned)((long long)num_groups * Hkv));
-#define LAUNCH_S(DH, WV)                                                                                          \
-  hipLaunchKernelGGL((attention_prefill_shared_kernel<DH, WV>), gs, dim3(WV * 64), 0, s, (const bf16_t*)q,        \
+#define LAUNCH_S(DH, WV, BIASED)                                                                                  \
+  hipLaunchKernelGGL((attention_prefill_shared_kernel<DH, WV, BIASED>), gs, dim3(WV * 64), 0, s, (const bf16_t*)q, \
                      (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,  \
-                     groups, ret_mode, ret_param, sl, Hq, Hkv, ps)
-#define PICK_S(DH) LAUNCH_S(DH, kGroupWaves)
+                     groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink)
+#define PICK_S(DH)                                        \
+  do {                                                    \
+    if (cap > 0.f) LAUNCH_S(DH, kGroupWaves, kCapped);    \
+    else LAUNCH_S(DH, kGroupWaves, kNoBias);              \
+  } while (0)
     switch (dh) {
       case 32: PICK_S(32); break;
       case 64: PICK_S(64); break;
@@ -1611,6 +1635,10 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
       case 128:  // (the kernel whose loads go straight into shared memory)
         if (bias_len < 0)
           hipLaunchKernelGGL(attention_prefill_lds_kernel<kBiasPenalty>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
+                             (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,
+                             groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink);
+        else if (cap > 0.f)
+          hipLaunchKernelGGL(attention_prefill_lds_kernel<kCapped>, gs, dim3(kGroupWaves * 64), 0, s, (const bf16_t*)q,
                              (const bf16_t*)kv, (bf16_t*)out, positions, token_segment, block_table, table_width, tiles,
                              groups, ret_mode, ret_param, sl, Hq, Hkv, ps, bs, sink);
         else if (bias != nullptr)
@@ -1637,10 +1665,12 @@ JLE_API int jle_attention_prefill(const void* q, const void* kv, void* out, cons
   do {                                                                                                               \
     if (tile_tokens == 32) {                                                                                         \
       if (bias_len < 0) LAUNCH_B(DH, 2, kBiasPenalty);                                                               \
+      else if (cap > 0.f) LAUNCH_B(DH, 2, kCapped);                                                                  \
       else if (bias != nullptr) LAUNCH_B(DH, 2, kBiasTable);                                                         \
       else LAUNCH_B(DH, 2, kNoBias);                                                                                 \
     } else {                                                                                                         \
       if (bias_len < 0) LAUNCH_B(DH, 1, kBiasPenalty);                                                               \
+      else if (cap > 0.f) LAUNCH_B(DH, 1, kCapped);                                                                  \
       else if (bias != nullptr) LAUNCH_B(DH, 1, kBiasTable);                                                         \
       else LAUNCH_B(DH, 1, kNoBias);                                                                                 \
     }                                                                                                                \
@@ -1697,11 +1727,11 @@ JLE_API int jle_attention_decode(const void* q, const void* kv, void* out, float
                                  const int* positions, const int* token_segment, const int* block_table,
                                  int table_width, const int* dec_tokens, int num_dec, int max_splits, int split,
                                  int ret_mode, int ret_param, float scale, int Hq, int Hkv, int dh, int ps,
-                                 const float* bias, int bias_len, const float* sink, hipStream_t s) {
+                                 const float* bias, int bias_len, const float* sink, float cap, hipStream_t s) {
   if (num_dec <= 0) return 0;
   if (!jle_attention_mfma_supported(dh, Hq, Hkv, ps) || max_splits < 1 || split < 32 || split % 32) return JLE_BAD_ARG;
-  if ((bias == nullptr) != (bias_len == 0) || (sink != nullptr && bias == nullptr)) return JLE_BAD_ARG;
-  const Biasing bs = {bias, bias_len};
+  if ((bias == nullptr) != (bias_len == 0) || cap < 0.f || (cap > 0.f && bias != nullptr)) return JLE_BAD_ARG;
+  const Biasing bs = {bias, bias_len, cap > 0.f ? 2.0f * kLog2e * scale / cap : 0.f, cap * kLog2e};
   if ((ret_mode == 1 || ret_mode == 2) && ret_param <= 0) return JLE_BAD_ARG;
   const int G = Hq / Hkv;
   if (G > 32) return JLE_BAD_ARG;
@@ -1718,6 +1748,9 @@ JLE_API int jle_attention_decode(const void* q, const void* kv, void* out, float
     if (bias_len < 0) {                      \
       if (ct == 1) LAUNCH(DH, 1, kBiasPenalty); \
       else LAUNCH(DH, 2, kBiasPenalty);      \
+    } else if (cap > 0.f) {                  \
+      if (ct == 1) LAUNCH(DH, 1, kCapped);   \
+      else LAUNCH(DH, 2, kCapped);           \
     } else if (bias != nullptr) {            \
       if (ct == 1) LAUNCH(DH, 1, kBiasTable); \
       else LAUNCH(DH, 2, kBiasTable);        \

@@ -1,7 +1,8 @@
 // Queries and keys normed over the whole projection, then queries to their rows and keys and values to their pages.
 //
 // rows: [N][Hq dk] (queries only) or [N][Hq dk + Hk dk + Hk dv].  One RMS norm over all Hq dk queries of a token
-// (weights wq of that size) and one over all its Hk dk keys (wk); the queries times 1 + attn_scale * ln(1 +
+// (weights wq of that size) and one over all its Hk dk keys (wk); then (rd > 0) the leading rd elements of every q and
+// k head turned by pos * inv_freq[j], element j paired with j + rd / 2 (angles float32); the queries times 1 + attn_scale * ln(1 +
 // floor((pos + 1) / floor_scale)) (floor_scale <= 0: no factor).  Heads are stored PD elements wide (PD >= dk, dv),
 // zeros behind the real ones: q_out [N][Hq][PD]; pages [page][2][Hk][..]: keys [ps][PD], values [PD][ps].
 // One block per token; statistics, weights and the factor in float32; sums of squares in an order that depends on the
@@ -16,12 +17,30 @@ __global__ __launch_bounds__(256) void span_prepare_kernel(const T* __restrict__
                                                            const int* __restrict__ slot_mapping,
                                                            const float* __restrict__ wq, const float* __restrict__ wk,
                                                            float eps, float floor_scale, float attn_scale, int Hq,
-                                                           int Hk, int dk, int dv, int PD, int ps, int own_kv) {
+                                                           int Hk, int dk, int dv, int PD, int ps, int own_kv,
+                                                           const float* __restrict__ inv_freq, int rd) {
   __shared__ float red[4];
+  extern __shared__ float turn[];  // [rd / 2][2]: the token's cosines and sines
+  const int hr = rd / 2;
   const size_t n = blockIdx.x;
   const int nq = Hq * dk, nk = Hk * dk, nv = Hk * dv;
   const int width = own_kv ? nq + nk + nv : nq;
   const T* r = rows + n * width;
+  for (int j = threadIdx.x; j < hr; j += 256) {  // (visible to all behind block_sum's barriers)
+    float sn, cs;
+    sincosf((float)positions[n] * inv_freq[j], &sn, &cs);
+    turn[2 * j] = cs;
+    turn[2 * j + 1] = sn;
+  }
+  // element d of a head whose weighted (not yet divided) elements lie at x * w
+  auto turned = [&](const T* x, const float* w, int d) {
+    const float v = Num<T>::load(x + d) * w[d];
+    if (d >= rd) return v;
+    const bool first = d < hr;
+    const int j = first ? d : d - hr, p = first ? d + hr : d - hr;
+    const float o = Num<T>::load(x + p) * w[p], cs = turn[2 * j], sn = turn[2 * j + 1];
+    return first ? v * cs - o * sn : v * cs + o * sn;
+  };
   float ssq = 0.f, ssk = 0.f;
   for (int c = threadIdx.x; c < nq; c += 256) {
     const float v = Num<T>::load(r + c);
@@ -41,7 +60,7 @@ __global__ __launch_bounds__(256) void span_prepare_kernel(const T* __restrict__
   for (int c = threadIdx.x; c < Hq * PD; c += 256) {
     const int h = c / PD, d = c - h * PD;
     float v = 0.f;
-    if (d < dk) v = Num<T>::load(r + h * dk + d) * wq[h * dk + d] * inv_q;
+    if (d < dk) v = turned(r + h * dk, wq + h * dk, d) * inv_q;
     Num<T>::store(qo + c, v);
   }
   if (!write) return;
@@ -55,7 +74,7 @@ __global__ __launch_bounds__(256) void span_prepare_kernel(const T* __restrict__
   for (int c = threadIdx.x; c < Hk * PD; c += 256) {
     const int h = c / PD, d = c - h * PD;
     float kx = 0.f, vx = 0.f;
-    if (d < dk) kx = Num<T>::load(r + nq + h * dk + d) * wk[h * dk + d] * inv_k;
+    if (d < dk) kx = turned(r + nq + h * dk, wk + h * dk, d) * inv_k;
     if (d < dv) vx = Num<T>::load(r + nq + nk + h * dv + d);
     Num<T>::store(kpage + h * plane + (size_t)off * PD + d, kx);
     Num<T>::store(vpage + h * plane + (size_t)d * ps + off, vx);
@@ -65,18 +84,19 @@ __global__ __launch_bounds__(256) void span_prepare_kernel(const T* __restrict__
 JLE_API int jle_span_prepare(const void* rows, void* q_out, void* kv, const int* positions, const int* slot_mapping,
                              const float* wq, const float* wk, float eps, float floor_scale, float attn_scale,
                              int is_bf16, int N, int Hq, int Hk, int dk, int dv, int PD, int ps, int own_kv,
-                             hipStream_t s) {
+                             const float* inv_freq, int rd, hipStream_t s) {
   if (N <= 0) return 0;
   if (Hq < 1 || Hk < 1 || dk < 1 || dv < 1 || PD < dk || PD < dv || ps < 1 || wq == nullptr) return JLE_BAD_ARG;
+  if (rd < 0 || rd % 2 || rd > dk || rd > 4096 || (rd > 0 && (inv_freq == nullptr || positions == nullptr))) return JLE_BAD_ARG;
   if (kv != nullptr && (!own_kv || wk == nullptr || slot_mapping == nullptr)) return JLE_BAD_ARG;
   if (is_bf16)
-    hipLaunchKernelGGL(span_prepare_kernel<bf16_t>, dim3(N), dim3(256), 0, s, (const bf16_t*)rows, (bf16_t*)q_out,
+    hipLaunchKernelGGL(span_prepare_kernel<bf16_t>, dim3(N), dim3(256), rd * sizeof(float), s, (const bf16_t*)rows, (bf16_t*)q_out,
                        (bf16_t*)kv, positions, slot_mapping, wq, wk, eps, floor_scale, attn_scale, Hq, Hk, dk, dv, PD,
-                       ps, own_kv);
+                       ps, own_kv, inv_freq, rd);
   else
-    hipLaunchKernelGGL(span_prepare_kernel<float>, dim3(N), dim3(256), 0, s, (const float*)rows, (float*)q_out,
+    hipLaunchKernelGGL(span_prepare_kernel<float>, dim3(N), dim3(256), rd * sizeof(float), s, (const float*)rows, (float*)q_out,
                        (float*)kv, positions, slot_mapping, wq, wk, eps, floor_scale, attn_scale, Hq, Hk, dk, dv, PD, ps,
-                       own_kv);
+                       own_kv, inv_freq, rd);
   JLE_LAUNCH_CHECK();
   return 0;
 }

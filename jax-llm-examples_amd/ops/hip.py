@@ -37,9 +37,10 @@ _SIGNATURES = {
                        _vp],
     "jle_paged_attention_generic": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _i, _i, _vp,
                                     _vp, _vp],
-    "jle_attention_f32_tiles": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _vp],
-    "jle_attention_f32_heads": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp],
-    "jle_attention_merge": [_vp, _vp, _vp, _i, _i, _i, _i, _vp],
+    "jle_attention_f32_tiles": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _f, _vp, _vp],
+    "jle_attention_f32_heads": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _vp, _vp, _f, _vp,
+                                _vp],
+    "jle_attention_merge": [_vp, _vp, _vp, _i, _i, _i, _i, _vp, _i, _vp],
     "jle_moe_route": [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp],
     "jle_norm_route": [_vp, _i, _vp, _vp, _vp, _i, _vp, _i, _vp, _f, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
                        _vp, _vp, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _vp, _i, _i, _i, _i, _f, _f, _vp],
@@ -51,9 +52,9 @@ _SIGNATURES = {
     "jle_sample": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp],
     "jle_attention_mfma_supported": [_i, _i, _i, _i],
     "jle_attention_prefill": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _vp,
-                              _i, _vp, _vp],
+                              _i, _vp, _f, _vp],
     "jle_attention_decode": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i,
-                             _vp, _i, _vp, _vp],
+                             _vp, _i, _vp, _f, _vp],
     "jle_attention_decode_fused": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _i, _i,
                                    _i, _i, _vp, _f, _f, _f, _vp, _i, _vp],
     "jle_gemm_grouped": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp],
@@ -86,11 +87,17 @@ _SIGNATURES = {
     "jle_mlstm": [_vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _f, _f, _f, _vp],
     "jle_mlstm_chunked": [_vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i,
                           _i, _i, _f, _f, _f, _vp],
-    "jle_span_prepare": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _f, _f, _f, _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp],
+    "jle_span_prepare": [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _f, _f, _f, _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp],
+    "jle_terms": [_vp, _vp, _f, _vp, _f, _vp, _f, _i, _vp, _vp, _vp, _f, _i, _vp, _i, _vp, _vp, _i, _i, _vp],
+    "jle_gated_unit": [_vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _f, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp, _i, _vp,
+                       _vp, _vp],
+    "jle_retention_angles": [_vp, _vp, _i, _f, _vp, _i, _vp],
+    "jle_retention": [_vp, _i, _vp, _vp, _i, _i, _f, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _vp, _vp, _i,
+                      _vp, _vp, _vp],
     "jle_row_gate": [_vp, _i, _vp, _vp, _i, _i, _i, _vp],
     "jle_scaled_add_norm": [_vp, _vp, _i, _f, _vp, _i, _f, _vp, _vp, _f, _vp, _i, _vp, _i, _i, _vp, _i, _vp],
     "jle_moe_logits": [_vp, _vp, _vp, _i, _i, _i, _vp],
-    "jle_heads_prepare": [_vp, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i,
+    "jle_heads_prepare": [_vp, _i, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i,
                           _i, _vp],
     "jle_diff_combine": [_vp, _vp, _vp, _f, _f, _f, _i, _i, _i, _i, _i, _i, _vp],
     "jle_gated_delta": [_vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i,
@@ -107,7 +114,7 @@ _SIGNATURES = {
     "jle_paged_attention_kept": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _i, _i, _vp,
                                  _vp, _vp],
     "jle_paged_attention_biased": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _i, _i, _vp,
-                                   _vp, _vp, _i, _vp, _vp],
+                                   _vp, _vp, _i, _vp, _f, _vp],
 }
 
 
@@ -171,7 +178,9 @@ def _bind(path: str):
                        ("jle_gemm_stream_supported", [_i, _i, _i]), ("jle_gemm_f32_stream_supported", [_i, _i, _i]),
                        ("jle_latent_attention_mfma_supported", [_i, _i, _i, _i, _i]), ("jle_attention_group_waves", []),
                        ("jle_mlstm_chunked_supported", [_i, _i]), ("jle_mlstm_chunk_tokens", []),
-                       ("jle_gated_delta_padded", [_i])):
+                       ("jle_gated_delta_padded", [_i]), ("jle_gated_unit_chunk_tokens", []),
+                       ("jle_retention_chunk_tokens", []), ("jle_retention_chunked_supported", [_i, _i]),
+                       ("jle_retention_workspace_kib", [_i, _i, _i, _i, _i])):
         fn = getattr(lib, name, None)
         if fn is not None:
             fn.argtypes = args
@@ -210,7 +219,6 @@ class HipOps:
         # counters of the kernels in which the last wavefront (or block) to finish does the closing work: zero
         # between launches (whoever closes puts its counter back), so they are cleared here once
         self._tickets = torch.zeros(self.TICKETS, dtype=torch.int32, device=self.device)
-        self._zero_bias = {}  # (heads, device) -> a distance table of zeros, for sinks without a bias
         self._slice_tickets = torch.zeros(self.SLICE_TICKETS, dtype=torch.int32, device=self.device)
         self._compute_units = torch.cuda.get_device_properties(self.device).multi_processor_count
         torch.backends.cuda.matmul.allow_tf32 = False
@@ -335,6 +343,24 @@ class HipOps:
                    self._is_bf16(out) if out is not None else 0, _p(out32), n, s_, d, int(bool(norm)))
         return out, out32
 
+    # ------------------------------------------------------------------ a step's segments in chunks
+    @staticmethod
+    def _chunk_table(ctx, per: int, device):
+        """The step's segments cut into chunks of ``per`` tokens: int32 ``[chunks, 3]`` (segment, first token, tokens), the
+        segments' first chunks ``[segments + 1]``, the number of chunks (made once per step)."""
+        key = f"chunks_of_{per}"
+        table = ctx.scratch.get(key)
+        if table is None:
+            flat, firsts, o = [], [0], 0
+            for i, ln in enumerate(ctx.seg_lens):
+                for t in range(0, ln, per):
+                    flat += [i, o + t, min(per, ln - t)]
+                firsts.append(len(flat) // 3)
+                o += ln
+            both = torch.tensor(flat + firsts, dtype=torch.int32).to(device)
+            table = ctx.scratch[key] = (both[: len(flat)], both[len(flat):], len(flat) // 3)
+        return table
+
     # ------------------------------------------------------------------ a matrix memory per head
     MLSTM_CHUNKS_FROM = 8  # a step with a segment of this many tokens takes the matrix memory in chunks
 
@@ -363,18 +389,7 @@ class HipOps:
         if (max(ctx.seg_lens, default=0) >= self.MLSTM_CHUNKS_FROM
                 and self._query("jle_mlstm_chunked_supported", dk, dv)):
             # a segment of many tokens: all segments in chunks that are worked on side by side
-            table = ctx.scratch.get("mlstm_chunks")
-            if table is None:
-                per = int(self._query("jle_mlstm_chunk_tokens"))
-                flat, firsts, o = [], [0], 0
-                for i, ln in enumerate(ctx.seg_lens):
-                    for t in range(0, ln, per):
-                        flat += [i, o + t, min(per, ln - t)]
-                    firsts.append(len(flat) // 3)
-                    o += ln
-                both = torch.tensor(flat + firsts, dtype=torch.int32).to(rows.device)
-                table = ctx.scratch["mlstm_chunks"] = (both[: len(flat)], both[len(flat):], len(flat) // 3)
-            chunks, seg_chunk0, nc = table
+            chunks, seg_chunk0, nc = self._chunk_table(ctx, int(self._query("jle_mlstm_chunk_tokens")), rows.device)
             ws = torch.empty(nc * H * (dk * dv + dk + 3), dtype=torch.float32, device=rows.device)
             ws_c, ws_n = ws[: nc * H * dk * dv], ws[nc * H * dk * dv: nc * H * (dk * dv + dk)]
             ws_m, ws_m0 = ws[nc * H * (dk * dv + dk): nc * H * (dk * dv + dk + 2)], ws[nc * H * (dk * dv + dk + 2):]
@@ -717,7 +732,67 @@ class HipOps:
                    1 if out_dtype == torch.bfloat16 else 0, _p(h32), n, d, _p(inv), inv_k)
         return h, h32
 
+    def _terms(self, x, delta):
+        """``(tensors, factors, whether they are bfloat16, vector)`` of what is added to ``x``: up to three of one type."""
+        n, d = x.shape
+        self._chk(x, torch.float32, (n, d), "residual")
+        vector = None
+        if delta is None:
+            terms = []
+        elif hasattr(delta, "terms"):
+            terms, vector = [(self.materialize(t), f) for t, f in delta.terms], delta.vector
+        elif hasattr(delta, "a"):
+            terms = [(t, 1.0) for t in (delta.a, delta.b) if t is not None]
+        elif hasattr(delta, "gate"):
+            raise KernelError("the kernel that adds up terms takes no gated branch")
+        else:
+            terms = [(self.materialize(delta), 1.0)]
+        if len({t.dtype for t, _ in terms}) > 1:
+            terms = [(t.float(), f) for t, f in terms]
+        for t, _ in terms:
+            self._chk(t, None, (n, d), "branch output")
+        if vector is not None:
+            self._chk(vector, torch.float32, (d,), "channel scale")
+        bf16 = self._is_bf16(terms[0][0]) if terms else 0
+        terms = terms + [(None, 0.0)] * (3 - len(terms))
+        return terms, bf16, vector
+
+    def _terms_call(self, x, delta, weight, bias, eps: float, mode: int, out, out32, rows=None):
+        terms, bf16, vector = self._terms(x, delta)
+        n, d = x.shape
+        for w, what in ((weight, "norm weight"), (bias, "norm bias")):
+            if w is not None:
+                self._chk(w, torch.float32, (d,), what)
+        flat = [v for t, f in terms for v in (_p(t), float(f))]
+        self._call("jle_terms", _p(x), *flat, bf16, _p(vector), _p(weight), _p(bias), float(eps), mode, _p(out),
+                   0 if out is None else self._is_bf16(out), _p(out32), _p(rows), n, d)
+
+    def terms_norm(self, x, delta, weight, bias, eps: float, out_dtype, want32: bool = False, center: bool = False,
+                   norm: bool = True):
+        """``x += delta`` in place (a sum of up to three weighted terms), then (``norm``) the rows' layer norm (``center``)
+        or root-mean-square norm; one launch.  See ``terms.hip``."""
+        n, d = x.shape
+        h = torch.empty(n, d, dtype=out_dtype, device=x.device) if norm else None
+        h32 = torch.empty(n, d, dtype=torch.float32, device=x.device) if norm and want32 else None
+        self._terms_call(x, delta, weight, bias, eps, int(bool(center)), h, h32)
+        return h, h32
+
+    def add_layernorm(self, x, delta, weight, bias, eps: float, out_dtype, want32: bool = False):
+        """``x += delta`` in place, then the layer norm's rows; one launch."""
+        return self.terms_norm(x, delta, weight, bias, eps, out_dtype, want32, center=True)
+
+    def joined_rows(self, x, delta, rows, out_dtype):
+        """``x + delta`` (not kept) and ``rows`` side by side: float32 ``[N, 2 D]``, or in bfloat16 ``[N, 3 D]``: the
+        leading term of ``x + delta``, ``rows``, and the remainder of ``x + delta``; one launch."""
+        n, d = x.shape
+        self._chk(rows, torch.float32, (n, d), "rows to join")
+        out = torch.empty(n, d * (3 if out_dtype == torch.bfloat16 else 2), dtype=out_dtype, device=x.device)
+        self._terms_call(x, delta, None, None, 0.0, 2, out, None, rows)
+        return out
+
     def add_rmsnorm(self, x, delta, weight, eps: float, out_dtype, want32: bool = False):
+        if hasattr(delta, "terms") and len(delta.terms) > 2:
+            return self.terms_norm(x, delta, weight, None, eps, out_dtype, want32)
         if hasattr(delta, "terms"):  # a sum with factors: the kernel that knows it
             return self.scaled_add_norm(x, delta, weight, eps, out_dtype, want32)
         if hasattr(delta, "a"):  # the sum of two parallel branches: the kernel that knows it
@@ -758,6 +833,9 @@ class HipOps:
         if hasattr(delta, "terms"):
             first = delta.terms[0][0]
             total = torch.zeros(first.shape[0], first.shape[1], dtype=torch.float32, device=self.device)
+            if len(delta.terms) > 2:
+                self.terms_norm(total, delta, None, None, 0.0, torch.float32, norm=False)
+                return total
             self.scaled_add_norm(total, delta, None, 0.0, torch.float32, norm=False)
             return total
         if not isinstance(delta, ExpertSum):
@@ -775,6 +853,9 @@ class HipOps:
         return (None, None, 0) if own is None else (_p(own[0]), _p(own[1]), own[1].shape[1])
 
     def add_residual(self, x, delta) -> None:
+        if hasattr(delta, "terms") and len(delta.terms) > 2:
+            self.terms_norm(x, delta, None, None, 0.0, torch.float32, norm=False)
+            return
         if hasattr(delta, "terms"):
             self.scaled_add_norm(x, delta, None, 0.0, torch.float32, norm=False)
             return
@@ -810,6 +891,10 @@ class HipOps:
             return out if out_dtype is None or out_dtype == out.dtype else out.to(out_dtype)
         out = torch.matmul(h, w.t())
         return out if out_dtype is None or out_dtype == out.dtype else out.to(out_dtype)
+
+    def linear_float32(self, h, w, tiled: bool = False):
+        """``h @ w.T`` with the float32 sums as they are; ``tiled``: ``w`` is in the streaming layout."""
+        return self.lm_head(h, w, tiled)
 
     def linear_bias(self, h, w, bias, bias_run=None):
         """``h @ w.T + bias``.  Returns ``(rows, bias still to be added or None)``: the library's product adds the
@@ -921,7 +1006,10 @@ class HipOps:
         it).  Returns q ``[N, q_heads, page_dim]``."""
         n = rows.shape[0]
         dk, dv, D = head_dim, value_dim, page_dim
-        self._chk(rows, None, (n, (q_heads + k_heads) * dk + v_heads * dv), "projected rows")
+        width = (q_heads + k_heads) * dk + v_heads * dv
+        if not rows.is_cuda or rows.shape[1] != width or rows.stride(1) != 1 or (n > 1 and rows.stride(0) < width):
+            raise KernelError(f"projected rows must be {width} wide, neighbouring elements side by side, on the GPU")
+        ld = rows.stride(0) if n > 1 else max(width, rows.stride(0))
         dt = rows.dtype
         if prep.query_scale is not None or prep.norm_span != "head":
             raise KernelError("this preparation kernel has no query scale and norms a head at a time")
@@ -946,7 +1034,7 @@ class HipOps:
             self._chk(kv_cache, dt, (kv_cache.shape[0], 2, k_heads, ps, D), "kv pages")
             self._chk(slot_mapping, torch.int32, (n,), "slot mapping")
         q = torch.empty(n, q_heads, D, dtype=dt, device=rows.device)
-        self._call("jle_heads_prepare", _p(rows), _p(positions), _p(slot_mapping) if kv_cache is not None else None,
+        self._call("jle_heads_prepare", _p(rows), ld, _p(positions), _p(slot_mapping) if kv_cache is not None else None,
                    _p(inv_freq), rd, half, magnitude, -1.0 if prep.norm_eps is None else float(prep.norm_eps),
                    1 if prep.norm_first else 0, _p(prep.norm_weight_q), wq_stride, _p(prep.norm_weight_k), _p(q),
                    _p(kv_cache), self._is_bf16(rows), n, q_heads, k_heads, v_heads, dk, dv, D, ps)
@@ -995,6 +1083,80 @@ class HipOps:
                    _p(out_gate), _p(state), _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(qn), _p(kn),
                    _p(beta), _p(decay), _p(kq), _p(o_raw), _p(out), n, ctx.num_segments, H, G, dk, dv, float(eps),
                    float(floor))
+        return out
+
+    def gated_unit(self, u, y, y_bias, w_ra, b_ra, w_ri, b_ri, lam, rate: float, state, ctx):
+        """See ``gated_unit.hip``: gates, decays and the recurrence from and into the requests' two-halved memory, times
+        ``gelu(y + y_bias)``; ``y`` may be a view of wider rows.  ``[N, W]`` in the run dtype."""
+        n, W = u.shape
+        blocks, size = w_ra.shape[0], w_ra.shape[1]
+        self._chk(u, None, (n, W), "convolved rows")
+        if y.shape != u.shape or y.dtype != u.dtype or not y.is_cuda or y.stride(1) != 1:
+            raise KernelError("the other branch must have the rows' shape and dtype, neighbouring channels side by side")
+        for t, what in ((w_ra, "decay gates' matrices"), (w_ri, "input gates' matrices")):
+            self._chk(t, u.dtype, (blocks, size, size), what)
+        if blocks * size != W:
+            raise KernelError("the gates' blocks do not fill the rows")
+        for t, what in ((b_ra, "decay gates' biases"), (b_ri, "input gates' biases")):
+            self._chk(t, torch.float32, (blocks, size), what)
+        for t, what in ((y_bias, "branch bias"), (lam, "lam")):
+            self._chk(t, torch.float32, (W,), what)
+        self._chk(state, torch.float32, (state.shape[0], 2, W), "memory")
+        r = ctx.num_segments
+        for t, what in ((ctx.state_slots, "state slots"), (ctx.state_phase, "state phases")):
+            self._chk(t, torch.int32, (r,), what)
+        out = torch.empty(n, W, dtype=u.dtype, device=u.device)
+        chunks = firsts = ws = None
+        nc = 0
+        if n != r:  # (some segment has more than one token)
+            chunks, firsts, nc = self._chunk_table(ctx, int(self._query("jle_gated_unit_chunk_tokens")), u.device)
+            ws = torch.empty((2 * n + 2 * nc) * W, dtype=torch.float32, device=u.device)
+        self._call("jle_gated_unit", _p(u), _p(y), y.stride(0) if n > 1 else max(W, y.stride(0)), _p(y_bias), _p(w_ra),
+                   _p(b_ra), _p(w_ri), _p(b_ri), _p(lam), float(rate), _p(state), _p(ctx.state_slots),
+                   _p(ctx.state_phase), _p(out), self._is_bf16(u), n, r, W, blocks, _p(chunks), nc, _p(firsts), _p(ws))
+        return out
+
+    RETENTION_CHUNKS_FROM = 16  # a segment of so many tokens (bfloat16): the kernels that take chunks side by side
+
+    def retention(self, rows, num_heads: int, head_dim: int, value_dim: int, rotation, decays, eps: float, state, ctx):
+        """See ``retention.hip``: queries and keys turned, the recurrence from and into the requests' two-halved memory,
+        head norm and output gate.  ``[N, H dv]`` in the run dtype."""
+        n = rows.shape[0]
+        H, dk, dv = num_heads, head_dim, value_dim
+        self._chk(rows, None, (n, 2 * H * (dk + dv)), "q | k | v | gate rows")
+        self._chk(state, torch.float32, (state.shape[0], 2, H, dv, dk), "memory")
+        self._chk(decays, torch.float32, (2, H), "decays")
+        self._chk(ctx.positions, torch.int32, (n,), "positions")
+        r = ctx.num_segments
+        for t, what, shape in ((ctx.cu_seqlens, "segment bounds", (r + 1,)), (ctx.state_slots, "state slots", (r,)),
+                               (ctx.state_phase, "state phases", (r,))):
+            self._chk(t, torch.int32, shape, what)
+        if dk > 512 or dv > 8192:
+            raise KernelError(f"the retention kernels take keys of up to 512 elements and values of up to 8192, not {dk}, {dv}")
+        pairing, rd, inv, magnitude = self._rotation(rotation, dk)
+        bf16 = self._is_bf16(rows)
+        out = torch.empty(n, H * dv, dtype=rows.dtype, device=rows.device)
+        how, angles, chunks, firsts, ws, nc = 0, None, None, None, None, 0
+        if n != r:
+            chunked = (bf16 and max(ctx.seg_lens) >= self.RETENTION_CHUNKS_FROM
+                       and self._query("jle_retention_chunked_supported", dk, dv))
+            how = 2 if chunked else 1
+            if rd:
+                # (a step with portions of prompts is never recorded: its angles can be kept for its other layers)
+                angles, _ = ctx.scratch.setdefault(("retention_angles", id(inv), rd, magnitude), (None, None))
+                if angles is None:
+                    angles = torch.empty(n, rd // 2, 2, dtype=torch.float32, device=rows.device)
+                    self._call("jle_retention_angles", _p(ctx.positions), _p(inv), rd, magnitude, _p(angles), n)
+                    ctx.scratch[("retention_angles", id(inv), rd, magnitude)] = (angles, inv)
+            if chunked:
+                chunks, firsts, nc = self._chunk_table(ctx, int(self._query("jle_retention_chunk_tokens")), rows.device)
+                kib = self._query("jle_retention_workspace_kib", n, nc, H, dk, dv)
+                ws = torch.empty(kib * 1024, dtype=torch.uint8, device=rows.device)
+            else:
+                ws = torch.empty(n * H * (2 * dk + dv), dtype=torch.float32, device=rows.device)
+        self._call("jle_retention", _p(rows), bf16, _p(ctx.positions), _p(inv), rd, pairing, magnitude, _p(decays), _p(state),
+                   _p(ctx.cu_seqlens), _p(ctx.state_slots), _p(ctx.state_phase), _p(out), n, r, H, dk, dv, float(eps), how,
+                   _p(angles), _p(chunks), nc, _p(firsts), _p(ws))
         return out
 
     MAMBA2_CHUNKS_FROM = 12  # a segment of so many tokens: the kernel that takes 64 at a time
@@ -1326,7 +1488,7 @@ class HipOps:
     def qkv_span_prepare(self, rows, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, page_dim: int,
                          own_kv: bool, prep, positions, kv_cache, slot_mapping):
         """One RMS norm over all of a token's queries and one over all its keys (weights of those sizes), the queries
-        times ``prep.query_scale``'s factor, keys and values into their pages with heads of ``page_dim`` elements
+        turned by ``prep.rotation`` (if there is one) and times ``prep.query_scale``'s factor, keys and values into their pages with heads of ``page_dim`` elements
         (zeros behind the real ones).  Returns q ``[N, Hq, page_dim]``."""
         n = rows.shape[0]
         hq, hk, dk, dv, pd = num_heads, num_kv_heads, head_dim, value_dim, page_dim
@@ -1336,6 +1498,13 @@ class HipOps:
         self._chk(prep.norm_weight_q, torch.float32, (hq * dk,), "q norm weight")
         if prep.norm_eps is None:
             raise KernelError("the norm over the projection needs its eps")
+        rot = prep.rotation
+        inv_freq, rd = None, 0
+        if rot is not None:
+            if rot.pairing != "half" or float(rot.magnitude) != 1.0:
+                raise KernelError("this preparation kernel turns half-split pairs, sines and cosines as they are")
+            rd = int(rot.rotary_dim) or dk
+            inv_freq = self._chk(rot.inv_freq, torch.float32, (rd // 2,), "inv_freq")
         ps = 1
         if kv_cache is not None:
             if not own_kv:
@@ -1349,7 +1518,7 @@ class HipOps:
         self._call("jle_span_prepare", _p(rows), _p(q), _p(kv_cache), _p(positions),
                    _p(slot_mapping) if kv_cache is not None else None, _p(prep.norm_weight_q),
                    _p(prep.norm_weight_k) if kv_cache is not None else None, float(prep.norm_eps), float(fs), float(sc),
-                   self._is_bf16(rows), n, hq, hk, dk, dv, pd, ps, int(bool(own_kv)))
+                   self._is_bf16(rows), n, hq, hk, dk, dv, pd, ps, int(bool(own_kv)), _p(inv_freq), rd)
         return q
 
     TICKETS = 1 << 16
@@ -1513,10 +1682,11 @@ class HipOps:
     F32_DECODE_ITEMS = 2048  # ... in a step of single tokens: about so many (token, kv head, key range) items
 
     def paged_attention(self, q, kv_cache, block_table, positions, token_segment, retention, scale: float, meta=None,
-                        bias=None, sink=None, penalty=None):
+                        bias=None, sink=None, penalty=None, cap=None):
         """``bias``: float32 ``[Hq, L]``: a key ``n`` places back adds ``bias[h, min(n, L - 1)]`` to head ``h``'s scaled
         score; ``sink``: float32 ``[Hq]``: ``exp(sink[h])`` is one more term of head ``h``'s denominator; ``penalty``:
-        float32 ``[Hq, 2]``: ``penalty[h, 0] * ln(1 + penalty[h, 1] * n)`` is taken off (without a ``bias``)."""
+        float32 ``[Hq, 2]``: ``penalty[h, 0] * ln(1 + penalty[h, 1] * n)`` is taken off (without a ``bias``); ``cap``: a scaled
+        score ``s`` becomes ``cap tanh(s / cap)`` (without either)."""
         n, hq, dh = q.shape
         hk, ps = kv_cache.shape[2], kv_cache.shape[3]
         self._chk(q, kv_cache.dtype, None, "q")
@@ -1531,10 +1701,13 @@ class HipOps:
             if bias is not None:
                 raise KernelError("the attention kernels take a distance table or a distance penalty, not both")
             bias = self._chk(penalty, torch.float32, (hq, 2), "distance penalty")
-        biased = bias is not None or sink is not None
+        biased = bias is not None
+        cap = 0.0 if cap is None else float(cap)
+        if cap < 0 or (cap and biased):
+            raise KernelError("a score cap is positive and comes without a distance table and a penalty")
         if retention[0] == "window_keep":
             return self._attention_kept(q, kv_cache, out, block_table, positions, token_segment, mode, param,
-                                        int(retention[2]), scale, meta, biased)
+                                        int(retention[2]), scale, meta, biased or sink is not None or cap > 0)
         if bias is not None:
             self._chk(bias, torch.float32, (hq, bias.shape[1]), "distance bias")
         bias_len = 0 if bias is None else -1 if penalty is not None else bias.shape[1]
@@ -1542,14 +1715,9 @@ class HipOps:
             self._chk(sink, torch.float32, (hq,), "sinks")
         if (q.dtype == torch.bfloat16 and hq // hk <= 32
                 and self._query("jle_attention_mfma_supported", dh, hq, hk, ps)):
-            # (with a bias or sinks the kernel for heads of 128 alone shares keys between wavefronts; at other sizes
+            # (with a bias the kernel for heads of 128 alone shares keys between wavefronts; at other sizes
             # every (tile, head) is a wavefront of its own, in tiles of 16 tokens)
             grouped = hq // hk if (not biased or dh == 128) else 1
-            if biased and bias is None:
-                bias = self._zero_bias.get((hq, q.device))
-                if bias is None:
-                    bias = self._zero_bias[(hq, q.device)] = torch.zeros(hq, 1, dtype=torch.float32, device=q.device)
-                bias_len = 1
             tile = self.BIASED_TILE if biased and grouped == 1 else self.PREFILL_TILE
             key = f"attn_plan_{grouped}_{tile}"
             plan = meta.meta.get(key) if meta is not None else None
@@ -1563,7 +1731,7 @@ class HipOps:
                 self._call("jle_attention_prefill", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                            _p(block_table), block_table.shape[1], _p(plan["tiles"]), plan["num_tiles"],
                            tile, _p(plan["groups"]), plan["num_groups"], mode, param, float(scale), hq,
-                           hk, dh, ps, _p(bias), bias_len, _p(sink))
+                           hk, dh, ps, _p(bias), bias_len, _p(sink), cap)
             if plan["num_dec"]:
                 cols = 16 if hq // hk <= 16 else 32
                 items = plan["num_dec"] * hk * plan["max_splits"]
@@ -1572,7 +1740,7 @@ class HipOps:
                 self._call("jle_attention_decode", _p(q), _p(kv_cache), _p(out), _p(ws_ml), _p(ws_o), _p(positions),
                            _p(token_segment), _p(block_table), block_table.shape[1], _p(plan["dec"]), plan["num_dec"],
                            plan["max_splits"], plan["split"], mode, param, float(scale), hq, hk, dh, ps, _p(bias),
-                           bias_len, _p(sink))
+                           bias_len, _p(sink), cap)
             return out
         if dh % 8 or dh > 256:
             raise KernelError(f"attention kernels: head size {dh} is not supported (a multiple of 8, at most 256)")
@@ -1594,7 +1762,7 @@ class HipOps:
                     meta.meta["f32_tiles"] = tiles
             self._call("jle_attention_f32_tiles", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                        _p(block_table), block_table.shape[1], _p(tiles), tiles.numel() // 2, mode, param, float(scale),
-                       hq, hk, dh, ps)
+                       hq, hk, dh, ps, cap, _p(sink))
             return out
         if (not biased and q.dtype == torch.float32 and dh % 16 == 0 and ps % 16 == 0 and hq // hk <= 16
                 and ((meta is not None and meta.decode_bucket is not None)
@@ -1615,9 +1783,9 @@ class HipOps:
                 ws_o = torch.empty(n * hq * splits * dh, dtype=torch.float32, device=q.device)
             self._call("jle_attention_f32_heads", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                        _p(block_table), block_table.shape[1], n, mode, param, float(scale), hq, hk, dh, ps, splits,
-                       per, _p(ws_ml), _p(ws_o))
+                       per, _p(ws_ml), _p(ws_o), cap, _p(sink))
             if splits > 1:
-                self._call("jle_attention_merge", _p(ws_ml), _p(ws_o), _p(out), 0, n * hq, dh, splits)
+                self._call("jle_attention_merge", _p(ws_ml), _p(ws_o), _p(out), 0, n * hq, dh, splits, _p(sink), hq)
             return out
         # few tokens with many keys (decode): each query's keys are shared between several wavefronts
         splits, tiles_per_split, ws_ml, ws_o = 1, 0, None, None
@@ -1636,11 +1804,11 @@ class HipOps:
                 splits = -(-tiles // tiles_per_split)
                 ws_ml = torch.empty(waves * splits * 2, dtype=torch.float32, device=q.device)
                 ws_o = torch.empty(waves * splits * dh, dtype=torch.float32, device=q.device)
-        if biased:
+        if biased or sink is not None or cap > 0:
             self._call("jle_paged_attention_biased", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                        _p(block_table), block_table.shape[1], mode, param, float(scale), self._is_bf16(q), n, hq, hk,
                        dh, ps, splits, tiles_per_split, _p(ws_ml), _p(ws_o), _p(bias),
-                       bias_len, _p(sink))
+                       bias_len, _p(sink), cap)
             return out
         self._call("jle_paged_attention_generic", _p(q), _p(kv_cache), _p(out), _p(positions), _p(token_segment),
                    _p(block_table), block_table.shape[1], mode, param, float(scale), self._is_bf16(q), n, hq, hk, dh,

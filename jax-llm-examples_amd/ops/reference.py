@@ -195,6 +195,24 @@ class ReferenceOps:
             h = h * weight.float()
         return h.to(out_dtype), (h if want32 else None)
 
+    def add_layernorm(self, x, delta, weight, bias, eps: float, out_dtype, want32: bool = False):
+        """``x += delta`` (in place, float32), then ``h = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias``."""
+        delta = self.materialize(delta)
+        if delta is not None:
+            x.add_(delta.float())
+        d = x - x.mean(-1, keepdim=True)
+        h = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * weight.float() + bias.float()
+        return h.to(out_dtype), (h if want32 else None)
+
+    def joined_rows(self, x, delta, rows, out_dtype):
+        """``x + delta`` (not kept) and ``rows`` side by side: float32 ``[N, 2 D]``, or in bfloat16 ``[N, 3 D]``: the
+        leading term of ``x + delta``, ``rows``, and the remainder of ``x + delta``."""
+        y = x if delta is None else x + self.materialize(delta).float()
+        if out_dtype == torch.float32:
+            return torch.cat([y, rows], dim=1)
+        hi = y.to(out_dtype)
+        return torch.cat([hi, rows.to(out_dtype), (y - hi.float()).to(out_dtype)], dim=1)
+
     def add_residual(self, x, delta) -> None:
         x.add_(self.materialize(delta).float())
 
@@ -209,6 +227,10 @@ class ReferenceOps:
     def lm_head(self, h, w, tiled: bool = False):
         assert not tiled, "the plain ops read row-major weights"
         return h.float() @ w.float().t()
+
+    def linear_float32(self, h, w, tiled: bool = False):
+        """``h @ w.T`` with the float32 sums as they are."""
+        return self.lm_head(h, w, tiled)
 
     def linear_bias(self, h, w, bias, bias_run=None):
         """``h @ w.T + bias`` rounded once to the run dtype.  Returns ``(rows, bias still to be added or None)``:
@@ -411,6 +433,57 @@ class ReferenceOps:
         y = y.reshape(n, norm_groups, inner // norm_groups)
         y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)
         return (y.reshape(n, inner) * norm_weight.float()).to(rows.dtype)
+
+    def gated_unit(self, u, y, y_bias, w_ra, b_ra, w_ri, b_ri, lam, rate: float, state, ctx):
+        """``u``, ``y``: ``[N, W]`` in the run dtype (``y`` may be a view of wider rows).  Per block of ``W / blocks``
+        channels ``r = sigmoid(w_ra u + b_ra)``, ``i = sigmoid(w_ri u + b_ri)``; ``log a = -rate r softplus(lam)``; token by
+        token from the request's memory (``state[slot, phase]``: ``[W]``; the new one goes to ``state[slot, 1 - phase]``)
+        ``S <- a S + sqrt(1 - a^2) i u``.  Returns ``S * gelu_tanh(y + y_bias)`` in the run dtype; float32 inside."""
+        n, W = u.shape
+        blocks = w_ra.shape[0]
+        uf = u.float()
+        ub = uf.reshape(n, blocks, W // blocks)
+        gate = lambda w, b: torch.sigmoid(torch.einsum("nbk,bok->nbo", ub, w.float()) + b.float()).reshape(n, W)
+        log_a = -rate * gate(w_ra, b_ra) * torch.nn.functional.softplus(lam.float())
+        a = torch.exp(log_a)
+        take = torch.sqrt(-torch.expm1(2.0 * log_a)) * gate(w_ri, b_ri) * uf
+        S_all = torch.empty_like(uf)
+        cu = ctx.cu_seqlens.tolist()
+        slots, phase = ctx.state_slots.tolist(), ctx.state_phase.tolist()
+        for s in range(len(cu) - 1):
+            S = state[slots[s], phase[s]].float()
+            for t in range(cu[s], cu[s + 1]):
+                S = a[t] * S + take[t]
+                S_all[t] = S
+            state[slots[s], 1 - phase[s]] = S
+        z = y.float() + y_bias.float()
+        g = 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z * z * z)))
+        return (S_all * g).to(u.dtype)
+
+    def retention(self, rows, num_heads: int, head_dim: int, value_dim: int, rotation, decays, eps: float, state, ctx):
+        """``rows``: ``[N, 2 H dk + 2 H dv]`` = q | k | v | output gate, run dtype.  q and k per head turned by the
+        rotation, k times ``dk^(-1/2)``; per head, token by token from the request's memory (``state[slot, phase]``:
+        ``[H, dv, dk]``, the transposed ``S``; the new one goes to ``state[slot, 1 - phase]``) ``S <- decays[0] S + k v^T;
+        o = S^T q``; then ``o`` divided by its root mean square per head (``eps``), times ``silu`` of the output gate.
+        ``[N, H dv]`` in the run dtype; float32 inside."""
+        n = rows.shape[0]
+        H, dk, dv = num_heads, head_dim, value_dim
+        r = rows.float()
+        q = self._turn(r[:, : H * dk].reshape(n, H, dk), ctx.positions, rotation)
+        k = self._turn(r[:, H * dk: 2 * H * dk].reshape(n, H, dk), ctx.positions, rotation) * dk ** -0.5
+        v = r[:, 2 * H * dk: 2 * H * dk + H * dv].reshape(n, H, dv)
+        g = r[:, 2 * H * dk + H * dv:]
+        out = torch.empty(n, H, dv, dtype=torch.float32, device=rows.device)
+        cu = ctx.cu_seqlens.tolist()
+        slots, phase = ctx.state_slots.tolist(), ctx.state_phase.tolist()
+        for s in range(len(cu) - 1):
+            S = state[slots[s], phase[s]].float()
+            for t in range(cu[s], cu[s + 1]):
+                S = decays[0][:, None, None] * S + v[t][:, :, None] * k[t][:, None, :]
+                out[t] = torch.einsum("hvk,hk->hv", S, q[t])
+            state[slots[s], 1 - phase[s]] = S
+        o = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps)
+        return (o.reshape(n, H * dv) * (g * torch.sigmoid(g))).to(rows.dtype)
 
     def gated_delta(self, rows, gates, a_log, dt_bias, norm_weight, out_gate, num_heads: int, num_kv_heads: int,
                     head_dim: int, value_dim: int, eps: float, floor: float, state, ctx):
@@ -619,7 +692,7 @@ class ReferenceOps:
                          own_kv: bool, prep, positions, kv_cache, slot_mapping):
         """``rows``: ``[N, Hq dk]`` (queries only) or, with ``own_kv``, ``[N, Hq dk + Hk dk + Hk dv]``.  One RMS norm
         over all of a token's queries and one over all its keys (``prep.norm_weight_q`` / ``_k`` of those sizes,
-        ``prep.norm_eps``), the queries times ``prep.query_scale``'s position-dependent factor; keys and values
+        ``prep.norm_eps``), then the rotation (if ``prep`` has one), the queries times ``prep.query_scale``'s position-dependent factor; keys and values
         written into their pages (if ``kv_cache`` is given) with heads of ``page_dim`` elements, zeros behind the real
         ones.  Returns q ``[N, Hq, page_dim]`` in the run dtype."""
         n = rows.shape[0]
@@ -628,6 +701,7 @@ class ReferenceOps:
         r = rows.float()
         rms = lambda x, w: x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + prep.norm_eps) * w.float()
         q = rms(r[:, : hq * dk], prep.norm_weight_q)
+        q = self._turn(q.reshape(n, hq, dk), positions, prep.rotation).reshape(n, hq * dk)
         if prep.query_scale is not None:
             floor_scale, attn_scale = prep.query_scale
             q = q * (1.0 + attn_scale * torch.log1p(torch.floor((positions.float() + 1.0) / floor_scale)))[:, None]
@@ -636,6 +710,7 @@ class ReferenceOps:
             if not own_kv:
                 raise ValueError("rows without keys and values cannot fill pages")
             k = rms(r[:, hq * dk: (hq + hk) * dk], prep.norm_weight_k).reshape(n, hk, dk)
+            k = self._turn(k, positions, prep.rotation)
             v = r[:, (hq + hk) * dk:].reshape(n, hk, dv)
             ps = kv_cache.shape[3]
             page, off = (slot_mapping // ps).long(), (slot_mapping % ps).long()
@@ -651,13 +726,14 @@ class ReferenceOps:
         return self.paged_attention(q, kv_cache, block_table, positions, token_segment, retention, scale, meta)
 
     def paged_attention(self, q, kv_cache, block_table, positions, token_segment, retention, scale: float, meta=None,
-                        bias=None, sink=None, penalty=None):
+                        bias=None, sink=None, penalty=None, cap=None):
         """For each token: softmax over the keys of its own request at positions
         ``[start(pos), pos]``, read from the pages its block table names.  ``bias``: float32 ``[Hq, L]``; a key ``n``
         places back adds ``bias[h, min(n, L - 1)]`` to head ``h``'s scaled score.  ``sink``: float32 ``[Hq]``;
         ``exp(sink[h])`` is one more term of head ``h``'s denominator (no key, no value, not scaled, no bias).
         ``penalty``: float32 ``[Hq, 2]``; ``penalty[h, 0] * ln(1 + penalty[h, 1] * n)`` is taken off head ``h``'s scaled
-        score of a key ``n`` places back."""
+        score of a key ``n`` places back.  ``cap``: a scaled score ``s`` becomes ``cap tanh(s / cap)`` (before anything is
+        added to it)."""
         n, hq, dh = q.shape
         hk, ps = kv_cache.shape[2], kv_cache.shape[3]
         g = hq // hk
@@ -680,6 +756,8 @@ class ReferenceOps:
             v = values_t(kv_cache)[pages, :, :, off].float()
             qi = q[i].float().reshape(hk, g, dh)
             sc = torch.einsum("hgd,thd->hgt", qi, k) * scale
+            if cap is not None:
+                sc = cap * torch.tanh(sc / cap)
             if bias is not None:
                 back = (p - kpos).clamp_max(bias.shape[1] - 1)
                 sc = sc + bias.float()[:, back].reshape(hk, g, -1)

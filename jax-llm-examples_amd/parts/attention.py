@@ -15,7 +15,8 @@ the output projection skips the zeros).  A second family of options, off for Lla
 size), ``distance_bias`` (a learned number per head and distance added to the scaled score;
 ``log_buckets``: a table of ``rows`` rows, the first half one distance each, the other half spread evenly over the
 logarithm of the distance up to ``max_distance``, where the last row begins), ``sink`` (a learned number per head
-whose exponential is one more term of the softmax's denominator) and ``own_kv = False`` (the layer projects no keys
+whose exponential is one more term of the softmax's denominator), a rotation of half-split pairs behind that norm,
+``score_cap`` (``cap tanh(score / cap)`` on the scaled score) and ``own_kv = False`` (the layer projects no keys
 and values: its run reads the cache that another run writes).  With any of these the rows go through
 ``qkv_span_prepare`` (norms over the projections, query scale, pages with heads filled up with zeros) and the
 attention kernels that take a bias table and sinks.  A third family, off for Llama 4 too: ``score_maps``
@@ -27,7 +28,9 @@ a weighted q/k norm before the rotation together with a convolution, half-split 
 retention rule ``window_keep`` (a window plus the sequence's first tokens), ``head_temperature`` (a learned number per
 head that its scaled scores are multiplied by: it rides in the query norm's weight) and the ``distance_bias`` kind
 ``log_distance`` (two learned numbers per head: ``r1 ln(1 + r2 n)`` is taken off the score of a key ``n`` places back;
-formed inside the attention kernels).  With any of these the projected rows go
+formed inside the attention kernels), ``output_gate = "head"`` (one gate a head, ``sigmoid(W_g h)_head``, whose rows
+lie behind the projection's) and ``sink = "zero"`` (one more term ``exp(0)`` in the denominator, without a number of
+its own).  With any of these the projected rows go
 through ``conv_rows`` (bias, convolution, state), ``heads_prepare`` (norm, rotation, pages with filled-up heads; a
 value head written once per score map, so that the attention kernels see ``maps * kv_heads`` key/value heads, the
 queries re-ordered at load so that those of a key head lie together) and, for two maps, ``diff_combine``.  Formulas:
@@ -88,7 +91,11 @@ class Attention(Mixer):
         self.bias_max = None if db is None else int(db.max_distance)
         if db is not None and not 2 <= self.bias_rows // 2 < self.bias_max:
             raise ValueError("a log_buckets distance table needs at least 4 rows and a max_distance beyond half of them")
-        self.has_sink = bool(spec.get("sink", False))
+        if spec.get("sink", False) not in (False, True, "zero"):
+            raise ValueError(f"a sink is learned (True) or 'zero', not {spec.sink!r}")
+        self.has_sink = spec.get("sink", False) is True
+        self.zero_sink = spec.get("sink", False) == "zero"
+        self.score_cap = None if spec.get("score_cap") is None else float(spec.score_cap)
         self.own_kv = bool(spec.get("own_kv", True))
         # the path through the kernel that norms over whole projections, and the attention kernels with bias and sink
         self.spanned = (self.qk_norm_span == "projection" or db is not None or self.has_sink or not self.own_kv)
@@ -108,23 +115,36 @@ class Attention(Mixer):
         self.maps = 1 if maps is None else 2
         self.diff = None if maps is None else float(maps.diff)
         self.head_norm_eps = None if maps is None else float(maps.eps)
-        self.output_gate = bool(spec.get("output_gate", False))
+        self.output_gate = spec.get("output_gate", False)
+        if self.output_gate not in (False, True, "head"):
+            raise ValueError(f"an output gate is per element (True) or per 'head', not {self.output_gate!r}")
+        self.head_gate = self.output_gate == "head"
         # the path through conv_rows and heads_prepare (see the module's text)
-        self.general = (self.maps > 1 or self.output_gate or self.retention[0] == "window_keep" or self.log_distance
+        self.general = (self.maps > 1 or bool(self.output_gate) or self.zero_sink or self.retention[0] == "window_keep" or self.log_distance
                         or self.head_temperature
                         or (not self.spanned and (self.conv_taps > 0 or self.biased or self.value_dim != self.head_dim)
                             and (self.qk_norm_weighted or self.qk_norm_first
                                  or (rot is not None and rot.pairing != "adjacent"))))
         self.lam = None
         if self.spanned:
-            if self.qk_norm_span != "projection" or not self.qk_norm_weighted or self.qk_norm_first:
-                raise ValueError("distance_bias, sink and own_kv=False come with a weighted q/k norm over the projection")
-            if rot is not None or self.biased or self.conv_taps:
-                raise ValueError("the attention mixer's path with a q/k norm over the projection has no rotation, no "
-                                 "projection bias and no convolution")
+            if self.qk_norm_span != "projection" or not self.qk_norm_weighted or (self.qk_norm_first and rot is None):
+                raise ValueError("distance_bias, a learned sink and own_kv=False come with a weighted q/k norm over the "
+                                 "projection")
+            if rot is not None and not (self.qk_norm_first and rot.pairing == "half" and rot.magnitude == 1.0):
+                raise ValueError("a rotation with a q/k norm over the projection comes behind it and turns half-split pairs")
+            if self.biased or self.conv_taps:
+                raise ValueError("the attention mixer's path with a q/k norm over the projection has no projection bias "
+                                 "and no convolution")
         if self.general and (self.spanned or self.query_scale is not None or self.qk_norm_span != "head"):
             raise ValueError("score maps, an output gate, the window_keep rule and a weighted norm with a convolution "
                              "come without a norm over the projection, a distance table, sinks and a query scale")
+        if self.score_cap is not None and (not self.spanned or self.score_cap <= 0 or db is not None or self.has_sink):
+            raise ValueError("a positive score cap comes with a q/k norm over the projection, without a distance table and "
+                             "sinks")
+        if (self.head_gate or self.zero_sink) and (self.maps > 1 or self.biased or self.retention[0] == "window_keep"
+                                                   or self.log_distance):
+            raise ValueError("a gate per head and a sink of zero come without score maps, projection biases, kept first "
+                             "tokens and a distance penalty")
         if self.log_distance and (self.maps > 1 or self.retention[0] == "window_keep"):
             raise ValueError("a log_distance penalty comes without score maps and the window_keep rule")
         if self.head_temperature and not (self.qk_norm_weighted and self.qk_norm_first and self.maps == 1):
@@ -160,7 +180,7 @@ class Attention(Mixer):
             extra["bqkv"] = ParamSpec((channels,), policy="float32", init=("normal", 0.3))
         if self.conv_taps:
             extra["conv"] = ParamSpec((channels, self.conv_taps), policy="float32", init=("normal", 0.6))
-        if self.output_gate:
+        if self.output_gate and not self.head_gate:
             extra["wg"] = ParamSpec((hq * dv, d), init=("normal", d ** -0.5))
         if self.head_temperature:
             extra["head_temp"] = ParamSpec((hq,), policy="float32", init=("uniform", 0.5, 1.5))
@@ -171,8 +191,9 @@ class Attention(Mixer):
             for name in ("lam_q1", "lam_k1", "lam_q2", "lam_k2"):
                 extra[name] = ParamSpec((dh,), policy="float32", init=("normal", 0.3))
         return {
-            # rows: q heads (head by head, a head's score maps one after the other), then k heads, then v heads
-            "wqkv": ParamSpec((channels, d)),
+            # rows: q heads (head by head, a head's score maps one after the other), then k heads, then v heads (then the
+            # heads' gates)
+            "wqkv": ParamSpec((channels + (hq if self.head_gate else 0), d)),
             "wo": ParamSpec((d, hq * dv)),
             **extra,
             **({"q_norm": ParamSpec((dh,), policy="float32", init=("ones",)),
@@ -246,6 +267,9 @@ class Attention(Mixer):
                     P[name][:nq] = P[name][:nq][idx]
             self.bias_run = None if not self.biased else P["bqkv"].to(P["wqkv"].dtype)
             self.conv_by_tap = P["conv"].t().contiguous() if self.conv_taps else None
+        self.sink_zeros = None
+        if self.zero_sink:
+            self.sink_zeros = torch.zeros(self.num_heads, dtype=torch.float32, device=self.params["wqkv"].device)
         self.wo_padded = None
         if self.page_dim != self.value_dim and self.maps == 1:  # the attention's output has page_dim elements a head: zeros' columns
             wo = self.params["wo"]
@@ -263,21 +287,24 @@ class Attention(Mixer):
         if self.general:
             mp = self.maps
             proj, bias = ops.linear_bias(h, self.params["wqkv"], self.params.get("bqkv"), self.bias_run)
-            gate = ops.linear(h, self.params["wg"]) if self.output_gate else None
-            rows = proj
+            rows, gate = proj, None
+            if self.head_gate:
+                rows, gate = proj[:, : self.channels], proj[:, self.channels:]
+            elif self.output_gate:
+                gate = ops.linear(h, self.params["wg"])
             if self.conv_taps or bias is not None or proj.dtype != ctx.dtype:
-                rows = ops.conv_rows(proj, bias, self.conv_by_tap, self.conv_taps, cache.state, ctx)
+                rows = ops.conv_rows(rows, bias, self.conv_by_tap, self.conv_taps, cache.state, ctx)
             q = ops.heads_prepare(rows, self.num_heads * mp, self.num_kv_heads * mp, self.num_kv_heads, self.head_dim,
                                   self.value_dim, self.page_dim, self.prep, ctx.positions,
                                   cache.kv if cache.writes else None, cache.slot_mapping)
             o = ops.paged_attention(q, cache.kv, cache.block_table, ctx.positions, ctx.token_segment, self.retention,
-                                    self.softmax_scale, cache.attn_meta, penalty=self.penalty)
+                                    self.softmax_scale, cache.attn_meta, penalty=self.penalty, sink=self.sink_zeros)
             if mp > 1:
                 o = ops.diff_combine(o, self.lam, 1.0 - self.diff, self.head_norm_eps, gate, self.num_heads,
                                      self.num_kv_heads, self.page_dim, self.value_dim)
                 return ops.linear(o, self.params["wo"])
             if gate is not None:
-                if self.page_dim != self.value_dim:
+                if self.page_dim != self.value_dim and not self.head_gate:
                     raise ValueError("an output gate on heads that are filled up with zeros is not provided for")
                 o = ops.sigmoid_mul(o, gate)
             return ops.linear(o, self.params["wo"] if self.wo_padded is None else self.wo_padded)
@@ -290,7 +317,7 @@ class Attention(Mixer):
                                      cache.kv if cache.writes else None, cache.slot_mapping)
             o = ops.paged_attention(q, cache.kv, cache.block_table, ctx.positions, ctx.token_segment, self.retention,
                                     self.softmax_scale, cache.attn_meta, bias=self.bias_table,
-                                    sink=self.params.get("sink"))
+                                    sink=self.params.get("sink"), cap=self.score_cap)
             return ops.linear(o, self.params["wo"] if self.wo_padded is None else self.wo_padded)
         if self.convolved:
             # the projection (its bias added by the product where the library does it, else by the kernel that reads

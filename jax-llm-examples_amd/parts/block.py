@@ -140,6 +140,33 @@ class ParallelBlock:
         residual.add(BranchSum(y, None if ff is None else ff.forward(h_b, None, ctx)))
 
 
+@register_arrangement("parallel_one_norm")
+class ParallelOneNormBlock:
+    """Both branches read the same normed rows: ``h = norm(x)``, ``x = x + (mixer(h) + feed_forward(h))``.  The mixer may
+    return a :class:`~.residual.ScaledSum` (two mixers side by side); the feed-forward's output becomes one more term
+    of it, and the whole sum stays pending on the residual.  The layer may have no feed-forward."""
+
+    def __init__(self, spec: LayerSpec) -> None:
+        self.spec = spec
+        self.mixer = build_mixer(spec.mixer)
+        self.mixer_norm = build_norm(spec.mixer_norm)
+        self.feed_forward = None if spec.feed_forward is None else build_feed_forward(spec.feed_forward)
+
+    def parts(self):
+        out = {"mixer": self.mixer, "mixer_norm": self.mixer_norm}
+        if self.feed_forward is not None:
+            out["feed_forward"] = self.feed_forward
+        return out
+
+    def forward(self, residual, ctx, cache) -> None:
+        ff = self.feed_forward
+        mixer32 = bool(getattr(self.mixer, "wants_float32_input", False))
+        ff32 = ff is not None and ff.wants_float32_input
+        h, h32 = self.mixer_norm.forward(residual, ctx, want32=mixer32 or ff32)
+        y = ScaledSum.of(self.mixer.forward(h, ctx, cache, h32) if mixer32 else self.mixer.forward(h, ctx, cache))
+        residual.add(y if ff is None else y.plus(ff.forward(h, h32 if ff32 else None, ctx)))
+
+
 class SigmoidGate(Part):
     """``sigmoid(W h + b)`` per element of a branch's output; this part holds ``W`` and ``b``, the kernel that
     adds the branch to the residual applies the sigmoid and the product."""

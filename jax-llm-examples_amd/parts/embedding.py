@@ -8,8 +8,8 @@ cosine of the same angle (the rates formed once in float64 and rounded, the angl
 ``(prev * mul_prev + token * mul_cur) mod buckets``, and the table's extra last row for a sequence's first token.
 The token before is known to the step (``StepContext.prev_token_ids``; across steps the cache manager keeps it).
 ``linear_head`` (``model.py:1204``): float32 logits ``h @ W.T`` with a matrix of its own, or, with
-``tied``, with the embedding's table; optionally plus a ``bias`` and squashed by a soft cap
-(``cap * tanh(logits / cap)``).  Llama 4 uses neither option: its ends are the two kernels alone.
+``tied``, with the embedding's table; optionally times a ``scale``, plus a ``bias`` and squashed by a soft cap
+(``cap * tanh(logits / cap)``).  Llama 4 uses none of the options: its ends are the two kernels alone.
 """
 from __future__ import annotations
 
@@ -86,6 +86,7 @@ class LinearHead(OutputHead):
         self.biased = bool(spec.get("bias", False))
         cap = spec.get("softcap")
         self.softcap = None if cap is None else float(cap)
+        self.scale = float(spec.get("scale", 1.0))
         self.tiled = False
 
     graph_safe = True
@@ -115,6 +116,8 @@ class LinearHead(OutputHead):
 
     def forward(self, h: torch.Tensor, ctx, embedding) -> torch.Tensor:
         logits = ctx.ops.lm_head(h, self.matrix(embedding), tiled=self.tiled)
+        if self.scale != 1.0:
+            logits.mul_(self.scale)
         if self.biased:
             logits.add_(self.params["bias"])
         if self.softcap is not None:

@@ -41,15 +41,15 @@ class BranchSum:
 
 class ScaledSum:
     """A branch output that is not formed yet: ``vector * sum_i factor_i * term_i`` per row, formed in float32 by the
-    kernel that adds it to the residual.  ``terms``: up to two ``(rows, factor)`` pairs, rows ``[N, hidden]`` in the
+    kernel that adds it to the residual.  ``terms``: up to three ``(rows, factor)`` pairs, rows ``[N, hidden]`` in the
     run dtype or float32 (or a sum of expert outputs still in pieces), factors plain numbers; ``vector``: float32
     ``[hidden]`` or ``None``.  It is what a layer with a multiplier on its branches, a learned scale per channel, or
-    two mixers side by side with a weight each leaves pending."""
+    two mixers side by side with a weight each (and a feed-forward beside them) leaves pending."""
 
     def __init__(self, terms, vector=None) -> None:
         self.terms = [(t, float(f)) for t, f in terms]
-        if not 1 <= len(self.terms) <= 2:
-            raise ValueError("a scaled sum has one or two terms")
+        if not 1 <= len(self.terms) <= 3:
+            raise ValueError("a scaled sum has one to three terms")
         self.vector = vector
         self.shape, self.dtype = self.terms[0][0].shape, self.terms[0][0].dtype
 
@@ -61,6 +61,12 @@ class ScaledSum:
                 raise ValueError("a scaled sum with a vector cannot be scaled by another")
             return cls([(t, f * factor) for t, f in y.terms], vector)
         return cls([(y, factor)], vector)
+
+    def plus(self, y, factor: float = 1.0) -> "ScaledSum":
+        """This sum (which must have no vector) and one more term."""
+        if self.vector is not None:
+            raise ValueError("nothing is added to a scaled sum with a vector")
+        return ScaledSum(self.terms + [(y, factor)])
 
     def rows(self, ops, idx) -> "ScaledSum":
         return ScaledSum([(ops.gather_rows(t, idx), f) for t, f in self.terms], self.vector)
@@ -121,6 +127,21 @@ class Residual:
         h, h32 = ctx.ops.add_rmsnorm(self.x, self.pending, weight, eps, ctx.dtype, want32)
         self.pending = None
         return h, h32
+
+    def layer_normed(self, ctx, weight, bias, eps: float, want32: bool = False):
+        """Adds what is pending and forms the layer norm's rows (in the run dtype and, if asked, float32)."""
+        self._settle_injected(ctx)
+        h, h32 = ctx.ops.add_layernorm(self.x, self.pending, weight, bias, eps, ctx.dtype, want32)
+        self.pending = None
+        return h, h32
+
+    def project_with(self, ctx, rows, weight, tiled: bool) -> None:
+        """``x <- weight [x; rows]``: the stream (with what is pending added) becomes a product of itself and ``rows``
+        (float32 ``[N, hidden]``) side by side.  ``weight``: see the kernel set's ``joined_rows``."""
+        self._settle_injected(ctx)
+        joined = ctx.ops.joined_rows(self.x, self.pending, rows, ctx.dtype)
+        self.pending = None
+        self._x = ctx.ops.linear_float32(joined, weight, tiled=tiled)
 
     def normed_shifted(self, ctx, weight, eps: float, shift=None):
         """Adds what is pending, norms the rows and, with ``shift = (weight, state)``, also gives the rows mixed
