@@ -120,8 +120,26 @@ def design_configs(size: dict, layers: int):
     f_kinds = [("mamba2", f_mem), ("attention", f_attn), ("mamba2", f_mem), ("latent_attention", f_latent)]
     folivik = {"architecture": "Folivik", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5},
                "layers": [{"type": f_kinds[i % 4][0], "mixer": f_kinds[i % 4][1], "mlp": f_moe} for i in range(layers)]}
+    # Lifesun: an attention over a window with capped scores beside a retention (half the heads, values twice as wide), and
+    # an attention within chunks beside a gated recurrent unit of the model's width, in turn, a dense feed-forward on the
+    # same norm; the inner layers run twice.  Its closest models here: Llama 4 with dense layers, and for the recurrent
+    # mixers Sudilorn and Folivik
+    l_attn = {"heads": size["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+              "mask": {"size": size["span"]}}
+    l_capped = {"left": dict(l_attn, softcap=50.0, rot={"base": 500000.0, "dims": 64}),
+                "right": {"heads": size["heads"] // 2, "dim": 128, "vdim": 256, "rot": {"base": 10000.0, "dims": 128},
+                          "decay": [1.0 - 2.0 ** -(5 + i % 8) for i in range(size["heads"] // 2)]},
+                "left_scale": 0.9, "right_scale": 0.8}
+    l_chunk = {"left": l_attn, "right": {"width": size["width"], "blocks": size["width"] // 256, "conv": 4},
+               "left_scale": 0.9, "right_scale": 0.8}
+    lifesun = {"architecture": "Lifesun", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5},
+               "logit_scale": 0.5,
+               "layers": [{"type": "parallel" if i % 2 else "parallel_2", "mixer": l_chunk if i % 2 else l_capped,
+                           "mlp": {"kind": "dense", "ff": size["ff"]}} for i in range(layers)]}
+    if layers >= 3:
+        lifesun["loop"] = {"start": 1, "stop": layers - 1, "times": 2}
     return {"rovidra": rovidra, "tiradra": tiradra, "llama4-dense": llama, "mazotar": mazotar, "llama4-moe": llama_moe,
-            "sudilorn": sudilorn, "folivik": folivik}
+            "sudilorn": sudilorn, "folivik": folivik, "lifesun": lifesun}
 
 
 def bench_designs(args) -> int:
@@ -230,10 +248,10 @@ def main() -> int:
     ap.add_argument("--no-prefill", action="store_true")
     ap.add_argument("--design-points", default="1@2048,8@2048,64@2048", help="decode steps of --designs: batch@context")
     ap.add_argument("--designs", default="", help="instead of the default workload: prefill and decode of the Rovidra, "
-                    "Tiradra, Mazotar, Sudilorn and Folivik designs beside the Llama 4 layers of equal sizes, at the named sizes "
+                    "Tiradra, Mazotar, Sudilorn, Folivik and Lifesun designs beside the Llama 4 layers of equal sizes, at the named sizes "
                     "(comma-separated, of " + ", ".join(DESIGN_SIZES) + "; 'all')")
     ap.add_argument("--design-names", default="", help="with --designs: only these of rovidra, tiradra, llama4-dense, "
-                    "mazotar, llama4-moe, sudilorn, folivik")
+                    "mazotar, llama4-moe, sudilorn, folivik, lifesun")
     args = ap.parse_args()
     if args.designs:
         return bench_designs(args)

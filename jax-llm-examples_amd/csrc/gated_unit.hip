@@ -76,13 +76,28 @@ struct Step<float> {
   }
 };
 
-__device__ __forceinline__ float sigmoid_(float x) { return 1.0f / (1.0f + expf(-x)); }
+// exp, 1 / (1 + exp(-x)) and the square root: float32 runs by the library, bfloat16 ones by the hardware's instructions
+// (a unit in the last place each, and half a one of the exponent's argument)
+template <typename T>
+struct Math {
+  static __device__ __forceinline__ float exp(float x) { return expf(x); }
+  static __device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+  static __device__ __forceinline__ float root(float x) { return sqrtf(x); }
+};
+template <>
+struct Math<bf16_t> {
+  static __device__ __forceinline__ float exp(float x) { return __builtin_amdgcn_exp2f(1.4426950408889634f * x); }
+  static __device__ __forceinline__ float sigmoid(float x) { return __builtin_amdgcn_rcpf(1.0f + exp(-x)); }
+  static __device__ __forceinline__ float root(float x) { return __builtin_amdgcn_sqrtf(x); }
+};
 __device__ __forceinline__ float softplus_(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 // gelu in its tanh form: 0.5 (1 + tanh t) = sigmoid(2 t)
+template <typename T>
 __device__ __forceinline__ float gelu_(float z) {
-  return z * sigmoid_(1.5957691216057308f * __builtin_fmaf(0.044715f * z, z * z, z));
+  return z * Math<T>::sigmoid(1.5957691216057308f * __builtin_fmaf(0.044715f * z, z * z, z));
 }
 // sqrt(1 - a^2) for a = exp(l), l <= 0: 1 - exp(x), x = 2 l, by its series near zero, where the difference would cancel
+template <typename T>
 __device__ __forceinline__ float taken(float l, float a) {
   const float x = 2.0f * l;
   float e = 1.0f / 40320.0f;
@@ -94,7 +109,7 @@ __device__ __forceinline__ float taken(float l, float a) {
   e = __builtin_fmaf(e, x, 0.5f);
   e = __builtin_fmaf(e, x, 1.0f);
   const float near = -e * x, far = __builtin_fmaf(-a, a, 1.0f);
-  return sqrtf(x > -0.5f ? near : far);
+  return Math<T>::root(x > -0.5f ? near : far);
 }
 
 template <typename T>
@@ -126,8 +141,8 @@ struct Channel {  // a channel's constants
   __device__ __forceinline__ Channel(const UnitArgs<T>& p, int ch)
       : fall(-p.rate * softplus_(p.lam[ch])), br(p.br[ch]), bi(p.bi[ch]) {}
   __device__ __forceinline__ Map map(float pre_r, float pre_i, float u) const {
-    const float l = fall * sigmoid_(pre_r + br), a = expf(l);
-    return Map{a, taken(l, a) * sigmoid_(pre_i + bi) * u};
+    const float l = fall * Math<T>::sigmoid(pre_r + br), a = Math<T>::exp(l);
+    return Map{a, taken<T>(l, a) * Math<T>::sigmoid(pre_i + bi) * u};
   }
 };
 
@@ -175,7 +190,7 @@ __global__ __launch_bounds__(64) void gated_unit_tokens_kernel(UnitArgs<T> p, T*
       const int ph = p.phase[n];
       const float s = __builtin_fmaf(m.a, st[(size_t)ph * p.W], m.b);
       st[(size_t)(1 - ph) * p.W] = s;
-      Num<T>::store(out + (size_t)n * p.W + ch, s * gelu_(Num<T>::load(p.y + (size_t)n * p.y_ld + ch) + yb));
+      Num<T>::store(out + (size_t)n * p.W + ch, s * gelu_<T>(Num<T>::load(p.y + (size_t)n * p.y_ld + ch) + yb));
     }
 }
 
@@ -343,10 +358,10 @@ __global__ __launch_bounds__(256) void gated_unit_out_kernel(const int* __restri
       const f32x4_t a = load4<float>(wa + at), b = load4<float>(wb + at), z = load4<T>(yr);
       f32x4_t o;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = __builtin_fmaf(a[e], S[e < V ? e : 0], b[e]) * gelu_(z[e] + yb[e < V ? e : 0]);
+      for (int e = 0; e < 4; ++e) o[e] = __builtin_fmaf(a[e], S[e < V ? e : 0], b[e]) * gelu_<T>(z[e] + yb[e < V ? e : 0]);
       store4<T>(out + at, o);
     } else {
-      Num<T>::store(out + at, __builtin_fmaf(wa[at], S[0], wb[at]) * gelu_(Num<T>::load(yr) + yb[0]));
+      Num<T>::store(out + at, __builtin_fmaf(wa[at], S[0], wb[at]) * gelu_<T>(Num<T>::load(yr) + yb[0]));
     }
   }
 }

@@ -311,7 +311,9 @@ __device__ __forceinline__ uint32_t split(float v) {
 
 // The chunks' operands.  dkp, dvp: dk and dv filled up (zeros) to what the kernels below are laid out for.
 struct Operands {
-  bf16_t *qh, *ql, *kh, *kl;  // [N][H][dkp]: queries and keys, leading terms and remainders
+  // [nc][H][kChunk][dkp]: queries and keys, leading terms and remainders (a chunk's rows of a head side by side: rows that
+  // lie all heads apart fall on few of the caches' sets and channels)
+  bf16_t *qh, *ql, *kh, *kl;
   bf16_t *dh, *dl;            // [nc][H][dkp][kChunk]: keys times decay^(n-1-s), a row the chunk's tokens (zeros behind its last)
   bf16_t* vt;                 // [nc][H][dvp][kChunk]: values, the same way
   bf16_t *sh, *sl;            // [nc][H][dvp][dkp]: the memory in front of the chunk
@@ -319,7 +321,52 @@ struct Operands {
   int dkp, dvp;
 };
 
-// blockIdx: (chunk, half of it, head).  Shared memory: [kPrep][max(dkp + 1, dvp / 2 + 1)] words.
+__device__ __forceinline__ void unpack8(uint4 r, float* v) {
+  const uint32_t w[4] = {r.x, r.y, r.z, r.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    v[2 * i] = __uint_as_float(w[i] << 16);
+    v[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+  }
+}
+// eight numbers' leading terms and remainders, eight of each side by side
+__device__ __forceinline__ void deal8(const uint32_t* w, uint4& hi, uint4& lo) {
+  uint32_t h[4], l[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    h[j] = (w[2 * j] & 0xffffu) | (w[2 * j + 1] << 16);
+    l[j] = (w[2 * j] >> 16) | (w[2 * j + 1] & 0xffff0000u);
+  }
+  hi = uint4{h[0], h[1], h[2], h[3]};
+  lo = uint4{l[0], l[1], l[2], l[3]};
+}
+// Elements e .. e + 7 of a head's row x, turned.  VEC: dk and the half of the turned elements are multiples of 8, half-split
+// pairs, rows aligned; a: the token's angles.
+template <bool VEC>
+__device__ __forceinline__ void turned8(const bf16_t* x, int e, const Heads& z, const float2* a, float* v) {
+  if (VEC) {
+    unpack8(*reinterpret_cast<const uint4*>(x + e), v);
+    if (e < z.rd) {
+      const int hr = z.rd / 2;
+      const bool first = e < hr;
+      float o[8];
+      unpack8(*reinterpret_cast<const uint4*>(x + (first ? e + hr : e - hr)), o);
+      const float4* t = reinterpret_cast<const float4*>(a + (first ? e : e - hr));
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float4 c = t[i];  // (two pairs' cosines and sines)
+        v[2 * i] = first ? v[2 * i] * c.x - o[2 * i] * c.y : v[2 * i] * c.x + o[2 * i] * c.y;
+        v[2 * i + 1] = first ? v[2 * i + 1] * c.z - o[2 * i + 1] * c.w : v[2 * i + 1] * c.z + o[2 * i + 1] * c.w;
+      }
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = e + i < z.dk ? turned(x, e + i, z, [&](int j) { return a[j]; }) : 0.f;
+  }
+}
+
+// blockIdx: (chunk, half of it, head).  Shared memory: [kPrep][max(dkp + 4, dvp / 2 + 4)] words.
+template <bool VEC>
 __global__ __launch_bounds__(256) void retention_prepare_kernel(const bf16_t* __restrict__ rows,
                                                                 const float2* __restrict__ angles, Heads z,
                                                                 const float* __restrict__ decays,
@@ -329,32 +376,50 @@ __global__ __launch_bounds__(256) void retention_prepare_kernel(const bf16_t* __
   const int t0 = chunks[3 * c + 1], n = chunks[3 * c + 2], m = min(kPrep, n - s0);  // (m <= 0: zeros only)
   const int hd = z.H * z.dk, hr = z.rd / 2, W = z.width(), dkp = o.dkp, dvp = o.dvp;
   const float log2_decay = decays[z.H + h];
-  for (int i = threadIdx.x; i < m * dkp; i += 256) {
-    const int t = i / dkp, e = i - t * dkp;
+  const size_t own = ((size_t)c * z.H + h) * kChunk + s0;  // this block's first row of q and k
+  const int e8 = dkp / 8;  // (a power of two)
+  for (int i = threadIdx.x; i < m * e8; i += 256) {
+    const int t = i / e8, e = (i - t * e8) * 8;
     const size_t row = (size_t)(t0 + s0 + t);
-    uint32_t v = 0u;
-    if (e < z.dk) v = split(turned(rows + row * W + h * z.dk, e, z, [&](int j) { return angles[row * hr + j]; }));
-    const size_t at = (row * z.H + h) * dkp + e;
-    o.qh[at] = (bf16_t)(v & 0xffffu);
-    o.ql[at] = (bf16_t)(v >> 16);
+    uint32_t w[8] = {0u, 0u, 0u, 0u, 0u, 0u, 0u, 0u};
+    if (e < z.dk) {
+      float v[8];
+      turned8<VEC>(rows + row * W + h * z.dk, e, z, angles + row * hr, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) w[j] = split(v[j]);
+    }
+    uint4 hi, lo;
+    deal8(w, hi, lo);
+    const size_t at = (own + t) * dkp + e;
+    *reinterpret_cast<uint4*>(o.qh + at) = hi;
+    *reinterpret_cast<uint4*>(o.ql + at) = lo;
   }
-  const int ldk = dkp + 1;
-  for (int i = threadIdx.x; i < kPrep * dkp; i += 256) {
-    const int t = i / dkp, e = i - t * dkp;
-    uint32_t d = 0u;
+  const int ldk = dkp + 4;
+  for (int i = threadIdx.x; i < kPrep * e8; i += 256) {
+    const int t = i / e8, e = (i - t * e8) * 8;
+    uint32_t d[8] = {0u, 0u, 0u, 0u, 0u, 0u, 0u, 0u};
     if (t < m) {
       const size_t row = (size_t)(t0 + s0 + t);
-      uint32_t v = 0u;
+      uint32_t w[8] = {0u, 0u, 0u, 0u, 0u, 0u, 0u, 0u};
       if (e < z.dk) {
-        const float k = turned(rows + row * W + hd + h * z.dk, e, z, [&](int j) { return angles[row * hr + j]; }) * z.k_scale;
-        v = split(k);
-        d = split(k * __builtin_amdgcn_exp2f((float)(n - 1 - s0 - t) * log2_decay));
+        float v[8];
+        turned8<VEC>(rows + row * W + hd + h * z.dk, e, z, angles + row * hr, v);
+        const float fade = __builtin_amdgcn_exp2f((float)(n - 1 - s0 - t) * log2_decay);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float k = v[j] * z.k_scale;
+          w[j] = split(k);
+          d[j] = split(k * fade);
+        }
       }
-      const size_t at = (row * z.H + h) * dkp + e;
-      o.kh[at] = (bf16_t)(v & 0xffffu);
-      o.kl[at] = (bf16_t)(v >> 16);
+      uint4 hi, lo;
+      deal8(w, hi, lo);
+      const size_t at = (own + t) * dkp + e;
+      *reinterpret_cast<uint4*>(o.kh + at) = hi;
+      *reinterpret_cast<uint4*>(o.kl + at) = lo;
     }
-    words[t * ldk + e] = d;
+    *reinterpret_cast<uint4*>(words + t * ldk + e) = uint4{d[0], d[1], d[2], d[3]};
+    *reinterpret_cast<uint4*>(words + t * ldk + e + 4) = uint4{d[4], d[5], d[6], d[7]};
   }
   __syncthreads();
   const size_t kt = ((size_t)c * z.H + h) * dkp * kChunk + s0;
@@ -364,22 +429,29 @@ __global__ __launch_bounds__(256) void retention_prepare_kernel(const bf16_t* __
 #pragma unroll
     for (int j = 0; j < 8; ++j) w[j] = words[(tg + j) * ldk + e];
     uint4 hi, lo;
-    uint32_t* ph = &hi.x;
-    uint32_t* pl = &lo.x;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      ph[j] = (w[2 * j] & 0xffffu) | (w[2 * j + 1] << 16);
-      pl[j] = (w[2 * j] >> 16) | (w[2 * j + 1] & 0xffff0000u);
-    }
+    deal8(w, hi, lo);
     *reinterpret_cast<uint4*>(o.dh + kt + (size_t)e * kChunk + tg) = hi;
     *reinterpret_cast<uint4*>(o.dl + kt + (size_t)e * kChunk + tg) = lo;
   }
   __syncthreads();
   bf16_t* sv = reinterpret_cast<bf16_t*>(words);
-  const int ldv = dvp + 2;
-  for (int i = threadIdx.x; i < kPrep * dvp; i += 256) {
-    const int t = i / dvp, e = i - t * dvp;
-    sv[t * ldv + e] = (t < m && e < z.dv) ? rows[(size_t)(t0 + s0 + t) * W + 2 * hd + h * z.dv + e] : (bf16_t)0;
+  const int ldv = dvp + 8, v8 = dvp / 8;
+  for (int i = threadIdx.x; i < kPrep * v8; i += 256) {
+    const int t = i / v8, e = (i - t * v8) * 8;
+    uint4 v = {0u, 0u, 0u, 0u};
+    if (t < m && e < z.dv) {
+      const bf16_t* src = rows + (size_t)(t0 + s0 + t) * W + 2 * hd + h * z.dv + e;
+      if (VEC) {
+        v = *reinterpret_cast<const uint4*>(src);
+      } else {
+        uint32_t w[4] = {0u, 0u, 0u, 0u};
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          if (e + j < z.dv) w[j >> 1] |= (uint32_t)src[j] << (16 * (j & 1));
+        v = uint4{w[0], w[1], w[2], w[3]};
+      }
+    }
+    *reinterpret_cast<uint4*>(sv + t * ldv + e) = v;
   }
   __syncthreads();
   const size_t vt = ((size_t)c * z.H + h) * dvp * kChunk + s0;
@@ -496,7 +568,7 @@ __global__ __launch_bounds__(256) void retention_outputs_kernel(const bf16_t* __
 #pragma unroll
   for (int x = 0; x < QT; ++x) {
     t[x] = q0 + 16 * x + c16;
-    const size_t at = ((size_t)(t0 + min(t[x], n - 1)) * z.H + h) * dkp + 8 * g;
+    const size_t at = ((size_t)blockIdx.x * kChunk + min(t[x], n - 1)) * dkp + 8 * g;
 #pragma unroll
     for (int k = 0; k < DKS; ++k) {
       qh[x][k] = piece(o.qh + at + 32 * k);
@@ -538,7 +610,7 @@ __global__ __launch_bounds__(256) void retention_outputs_kernel(const bf16_t* __
     for (int tt = 0; tt < 2; ++tt) {
 #pragma unroll
       for (int x = 0; x < QT; ++x) st[x][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
-      const size_t at = ((size_t)(t0 + min(s0 + 16 * tt + c16, n - 1)) * z.H + h) * dkp + 8 * g;
+      const size_t at = ((size_t)blockIdx.x * kChunk + min(s0 + 16 * tt + c16, n - 1)) * dkp + 8 * g;
 #pragma unroll
       for (int k = 0; k < DKS; ++k) {
         const bf16x8 kh = piece(o.kh + at + 32 * k), kl = piece(o.kl + at + 32 * k);
@@ -563,13 +635,7 @@ __global__ __launch_bounds__(256) void retention_outputs_kernel(const bf16_t* __
           s[4 * tt + i] = split(p);
         }
       uint4 hi, lo;
-      uint32_t* wh = &hi.x;
-      uint32_t* wl = &lo.x;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        wh[j] = (s[2 * j] & 0xffffu) | (s[2 * j + 1] << 16);
-        wl[j] = (s[2 * j] >> 16) | (s[2 * j + 1] & 0xffff0000u);
-      }
+      deal8(s, hi, lo);
       ph[x] = __builtin_bit_cast(bf16x8, hi);
       pl[x] = __builtin_bit_cast(bf16x8, lo);
     }
@@ -629,7 +695,7 @@ int padded_values(int dv) { return dv <= 64 ? 64 : dv <= 128 ? 128 : dv <= 256 ?
 size_t align16(size_t n) { return (n + 15) / 16 * 16; }
 
 // the operands' places in the workspace; with base null: its size
-size_t place(Operands& o, char* base, int N, int nc, int H, int dk, int dv) {
+size_t place(Operands& o, char* base, int nc, int H, int dk, int dv) {
   o.dkp = padded_keys(dk);
   o.dvp = padded_values(dv);
   size_t at = 0;
@@ -638,11 +704,11 @@ size_t place(Operands& o, char* base, int N, int nc, int H, int dk, int dv) {
     at += align16(bytes);
     return p;
   };
-  const size_t q = (size_t)N * H * o.dkp * 2, kt = (size_t)nc * H * o.dkp * kChunk * 2, ch = (size_t)nc * H;
-  o.qh = (bf16_t*)take(q);
-  o.ql = (bf16_t*)take(q);
-  o.kh = (bf16_t*)take(q);
-  o.kl = (bf16_t*)take(q);
+  const size_t kt = (size_t)nc * H * o.dkp * kChunk * 2, ch = (size_t)nc * H;
+  o.qh = (bf16_t*)take(kt);
+  o.ql = (bf16_t*)take(kt);
+  o.kh = (bf16_t*)take(kt);
+  o.kl = (bf16_t*)take(kt);
   o.dh = (bf16_t*)take(kt);
   o.dl = (bf16_t*)take(kt);
   o.vt = (bf16_t*)take(ch * o.dvp * kChunk * 2);
@@ -655,7 +721,7 @@ size_t place(Operands& o, char* base, int N, int nc, int H, int dk, int dv) {
 template <int DKS, int DVT>
 int launch_outputs(const bf16_t* rows, const Operands& o, const Heads& z, const float* decays, const int* chunks, int nc,
                    bf16_t* out, float eps, bool vec, hipStream_t s) {
-  constexpr int QT = (DKS <= 4 && DVT <= 16) ? 2 : 1;
+  constexpr int QT = DVT <= 8 && DKS <= 4 ? 2 : 1;  // (what leaves registers for several wavefronts a SIMD)
   const dim3 grid(nc * z.H, kChunk / (64 * QT));
   if (vec)
     hipLaunchKernelGGL((retention_outputs_kernel<DKS, DVT, QT, true>), grid, dim3(256), 0, s, rows, o, z, decays, chunks, out, eps);
@@ -677,18 +743,21 @@ int pick_outputs(const bf16_t* rows, const Operands& o, const Heads& z, const fl
 }
 
 int run_chunks(const bf16_t* rows, const float2* angles, const Heads& z, const Memory& mem, const int* chunks, int nc,
-               const int* first, char* ws, bf16_t* out, int N, int R, float eps, hipStream_t s) {
+               const int* first, char* ws, bf16_t* out, int R, float eps, hipStream_t s) {
   Operands o;
-  place(o, ws, N, nc, z.H, z.dk, z.dv);
-  const size_t lds = sizeof(uint32_t) * kPrep * (size_t)(o.dkp + 1 > o.dvp / 2 + 1 ? o.dkp + 1 : o.dvp / 2 + 1);
-  static bool allowed = false;
-  if (!allowed) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&retention_prepare_kernel),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);
+  place(o, ws, nc, z.H, z.dk, z.dv);
+  const size_t lds = sizeof(uint32_t) * kPrep * (size_t)(o.dkp > o.dvp / 2 ? o.dkp + 4 : o.dvp / 2 + 4);
+  const bool vec8 = z.dk % 8 == 0 && z.dv % 8 == 0 && (z.rd == 0 || z.half_pairs) && (z.rd / 2) % 8 == 0 &&
+                    ((uintptr_t)rows | (uintptr_t)angles) % 16 == 0;  // (then a row's width is a multiple of 8 too)
+  auto prepare = vec8 ? retention_prepare_kernel<true> : retention_prepare_kernel<false>;
+  static bool allowed[2] = {false, false};
+  if (!allowed[vec8]) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prepare), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                       80 * 1024);
     if (e != hipSuccess) return (int)e;
-    allowed = true;
+    allowed[vec8] = true;
   }
-  hipLaunchKernelGGL(retention_prepare_kernel, dim3(nc, kChunk / kPrep, z.H), dim3(256), lds, s, rows, angles, z, mem.decays,
+  hipLaunchKernelGGL(prepare, dim3(nc, kChunk / kPrep, z.H), dim3(256), lds, s, rows, angles, z, mem.decays,
                      chunks, o);
   JLE_LAUNCH_CHECK();
   hipLaunchKernelGGL(retention_chunk_memory_kernel, dim3(nc * z.H, (o.dkp / 64) * (o.dvp / 64)), dim3(64), 0, s, o, z);
@@ -766,9 +835,9 @@ Heads heads_of(int H, int dk, int dv, const float* inv_freq, int rd, int half_pa
 JLE_API int jle_retention_chunk_tokens() { return kChunk; }
 JLE_API int jle_retention_chunked_supported(int dk, int dv) { return dk >= 1 && dv >= 1 && padded_keys(dk) && padded_values(dv); }
 // bytes of the chunk kernels' workspace, in units of 1,024
-JLE_API int jle_retention_workspace_kib(int N, int nc, int H, int dk, int dv) {
+JLE_API int jle_retention_workspace_kib(int nc, int H, int dk, int dv) {
   Operands o;
-  return (int)((place(o, nullptr, N, nc, H, dk, dv) + 1023) / 1024);
+  return (int)((place(o, nullptr, nc, H, dk, dv) + 1023) / 1024);
 }
 
 // cosines and sines of every token's angles: out [N][rd / 2][2] float32
@@ -811,5 +880,5 @@ JLE_API int jle_retention(const void* rows, int is_bf16, const int* positions, c
   if (how != 2 || !is_bf16 || nc < 1 || chunks == nullptr || first == nullptr || !jle_retention_chunked_supported(dk, dv) ||
       (uintptr_t)ws % 16)
     return JLE_BAD_ARG;
-  return run_chunks((const bf16_t*)rows, (const float2*)angles, z, mem, chunks, nc, first, (char*)ws, (bf16_t*)out, N, R, eps, s);
+  return run_chunks((const bf16_t*)rows, (const float2*)angles, z, mem, chunks, nc, first, (char*)ws, (bf16_t*)out, R, eps, s);
 }

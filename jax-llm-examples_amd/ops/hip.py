@@ -180,7 +180,7 @@ def _bind(path: str):
                        ("jle_mlstm_chunked_supported", [_i, _i]), ("jle_mlstm_chunk_tokens", []),
                        ("jle_gated_delta_padded", [_i]), ("jle_gated_unit_chunk_tokens", []),
                        ("jle_retention_chunk_tokens", []), ("jle_retention_chunked_supported", [_i, _i]),
-                       ("jle_retention_workspace_kib", [_i, _i, _i, _i, _i])):
+                       ("jle_retention_workspace_kib", [_i, _i, _i, _i])):
         fn = getattr(lib, name, None)
         if fn is not None:
             fn.argtypes = args
@@ -892,9 +892,11 @@ class HipOps:
         out = torch.matmul(h, w.t())
         return out if out_dtype is None or out_dtype == out.dtype else out.to(out_dtype)
 
-    def linear_float32(self, h, w, tiled: bool = False):
-        """``h @ w.T`` with the float32 sums as they are; ``tiled``: ``w`` is in the streaming layout."""
-        return self.lm_head(h, w, tiled)
+    def linear_float32(self, h, w):
+        """``h @ w.T`` with the float32 sums as they are: a library product where there are many rows."""
+        if h.dtype == torch.bfloat16 and (h.shape[0] > self.SKINNY_MAX_ROWS or h.shape[1] % 8):
+            return torch.mm(h, w.t(), out_dtype=torch.float32)
+        return self.lm_head(h, w)
 
     def linear_bias(self, h, w, bias, bias_run=None):
         """``h @ w.T + bias``.  Returns ``(rows, bias still to be added or None)``: the library's product adds the
@@ -1150,7 +1152,7 @@ class HipOps:
                     ctx.scratch[("retention_angles", id(inv), rd, magnitude)] = (angles, inv)
             if chunked:
                 chunks, firsts, nc = self._chunk_table(ctx, int(self._query("jle_retention_chunk_tokens")), rows.device)
-                kib = self._query("jle_retention_workspace_kib", n, nc, H, dk, dv)
+                kib = self._query("jle_retention_workspace_kib", nc, H, dk, dv)
                 ws = torch.empty(kib * 1024, dtype=torch.uint8, device=rows.device)
             else:
                 ws = torch.empty(n * H * (2 * dk + dv), dtype=torch.float32, device=rows.device)

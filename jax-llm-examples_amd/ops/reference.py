@@ -228,9 +228,9 @@ class ReferenceOps:
         assert not tiled, "the plain ops read row-major weights"
         return h.float() @ w.float().t()
 
-    def linear_float32(self, h, w, tiled: bool = False):
+    def linear_float32(self, h, w):
         """``h @ w.T`` with the float32 sums as they are."""
-        return self.lm_head(h, w, tiled)
+        return self.lm_head(h, w)
 
     def linear_bias(self, h, w, bias, bias_run=None):
         """``h @ w.T + bias`` rounded once to the run dtype.  Returns ``(rows, bias still to be added or None)``:

@@ -68,22 +68,17 @@ class PassProjection(Part):
     def __init__(self, spec) -> None:
         super().__init__()
         self.hidden, self.times = int(spec.hidden_size), int(spec.times)
-        self.joined, self.tiled = None, False
+        self.joined = None
 
     def param_specs(self):
         return {"weight": ParamSpec((self.hidden, 2 * self.hidden), init=("normal", (2 * self.hidden) ** -0.5))}
 
     def finalize(self) -> None:
-        from ..ops.layout import can_tile, tile_
-
         w = self.params["weight"]
         # [hidden, 3 hidden] in bfloat16: for x's leading part, x_0, and x's remainder
         self.joined = torch.cat([w, w[:, : self.hidden]], dim=1) if w.dtype == torch.bfloat16 else w
-        self.tiled = can_tile(self.joined)
-        if self.tiled:
-            tile_(self.joined)
 
     def enter(self, residual, embedded, number: int, ctx) -> None:
         if not 0 <= number < self.times:
             raise ValueError(f"pass {number} of a loop of {self.times}")
-        residual.project_with(ctx, embedded, self.joined, self.tiled)
+        residual.project_with(ctx, embedded, self.joined)

@@ -135,13 +135,13 @@ class Residual:
         self.pending = None
         return h, h32
 
-    def project_with(self, ctx, rows, weight, tiled: bool) -> None:
+    def project_with(self, ctx, rows, weight) -> None:
         """``x <- weight [x; rows]``: the stream (with what is pending added) becomes a product of itself and ``rows``
         (float32 ``[N, hidden]``) side by side.  ``weight``: see the kernel set's ``joined_rows``."""
         self._settle_injected(ctx)
         joined = ctx.ops.joined_rows(self.x, self.pending, rows, ctx.dtype)
         self.pending = None
-        self._x = ctx.ops.linear_float32(joined, weight, tiled=tiled)
+        self._x = ctx.ops.linear_float32(joined, weight)
 
     def normed_shifted(self, ctx, weight, eps: float, shift=None):
         """Adds what is pending, norms the rows and, with ``shift = (weight, state)``, also gives the rows mixed
