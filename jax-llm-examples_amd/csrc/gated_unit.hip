@@ -235,7 +235,7 @@ __global__ __launch_bounds__(kChunkWaves * 64) void gated_unit_chunk_kernel(Unit
     }
     __syncthreads();
     const int steps = min(8, (size - k0 + KS - 1) / KS);
-#pragma unroll 2
+#pragma unroll 4
     for (int s = 0; s < steps; ++s) {
       const int k = s * KS + KL * g, left = size - k0 - k;
       Frag fr[CT], fi[CT];
@@ -255,8 +255,10 @@ __global__ __launch_bounds__(kChunkWaves * 64) void gated_unit_chunk_kernel(Unit
         }
       }
     }
-    __syncthreads();
+    if (k0 + SLAB < size) __syncthreads();
   }
+  // (a block's part of a row that is no wider than the slab is still there)
+  const bool held = size <= SLAB;
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
     const int in_blk = c0 + 16 * ct + c16;
@@ -272,7 +274,9 @@ __global__ __launch_bounds__(kChunkWaves * 64) void gated_unit_chunk_kernel(Unit
       for (int i = 0; i < 4; ++i) {
         const int t = 16 * rt + 4 * g + i;
         m[i] = Map{1.f, 0.f};
-        if (t < n) m[i] = k.map(ar[ct][rt][i], ai[ct][rt][i], Num<T>::load(p.u + (size_t)(t0 + t) * p.W + ch));
+        if (t < n)
+          m[i] = k.map(ar[ct][rt][i], ai[ct][rt][i],
+                       held ? Num<T>::load(su + t * ROW + min(in_blk, size - 1)) : Num<T>::load(p.u + (size_t)(t0 + t) * p.W + ch));
         if (i > 0) m[i] = then(m[i - 1], m[i]);
       }
       // across the channel's four lanes

@@ -28,6 +28,7 @@ namespace {
 
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) unsigned int u32x4;  // (register arrays of HIP's uint4 may end up in scratch)
 
 struct Heads {
   int H, dk, dv, rd, half_pairs;
@@ -546,144 +547,193 @@ __global__ __launch_bounds__(256) void retention_walk_kernel(Operands o, Heads z
   if (there) mem.state[(slot + 1 - ph) * half + h * head + e] = S;
 }
 
-// The outputs of 16 QT tokens of a chunk for one head, a wavefront.  Everything is kept transposed (rows: keys or value
-// elements, columns: tokens), so that the weighted scores are the second product's operand where the first left them: of
-// 32 keys the inner index (g, j) is key 4 g + j of the first 16 for j < 4, of the second for j >= 4.
-// DKS: dkp / 32, DVT: dvp / 16.  VEC: gate and output rows are aligned for four neighbours.
-// blockIdx: (chunk * H + head, 64 QT tokens)
-template <int DKS, int DVT, int QT, bool VEC>
-__global__ __launch_bounds__(256) void retention_outputs_kernel(const bf16_t* __restrict__ rows, Operands o, Heads z,
-                                                                const float* __restrict__ decays,
-                                                                const int* __restrict__ chunks, bf16_t* __restrict__ out,
-                                                                float eps) {
-  constexpr int dkp = 32 * DKS, dvp = 16 * DVT;
-  const int lane = threadIdx.x & 63, w = wave_index(), c16 = lane & 15, g = lane >> 4;
+// The outputs of a chunk for one head: a block of eight wavefronts, 16 tokens each.  Everything is kept transposed (rows:
+// keys or value elements, columns: tokens), so that the weighted scores are the second product's operand where the first
+// left them: row r of the scores' key tile tt is key 8 (r / 4) + 4 tt + r % 4 of a step's 32, so a lane's eight scores are
+// those of eight consecutive keys.
+// All wavefronts read the same memory, keys and values: they come through shared memory, once per block, in stages - 32
+// value columns of the memory, then 32 keys with their values -, the next stage's on its way in registers while one is
+// worked on; two buffers, one barrier a stage.
+// DKS: dkp / 32, DVT: dvp / 16.  VEC: gate and output rows are aligned for four neighbours.  blockIdx: chunk * H + head
+constexpr int kOutThreads = kChunk * 4;
+
+template <int DKS, int DVT>
+constexpr size_t output_lds() {  // bytes of the two buffers
+  return 2 * sizeof(bf16_t) * (2 * 32 * (32 * DKS + 8) + 16 * DVT * 40);
+}
+
+template <int DKS, int DVT, bool VEC>
+__global__ __launch_bounds__(kOutThreads) void retention_outputs_kernel(const bf16_t* __restrict__ rows, Operands o, Heads z,
+                                                                        const float* __restrict__ decays,
+                                                                        const int* __restrict__ chunks,
+                                                                        bf16_t* __restrict__ out, float eps) {
+  constexpr int dkp = 32 * DKS, dvp = 16 * DVT, TH = kOutThreads;
+  constexpr int LK = dkp + 8, LV = 40;                      // from one row to the next in shared memory
+  constexpr int HALF = 32 * LK, BUF = 2 * HALF + dvp * LV;  // leading terms, remainders, values
+  constexpr int RP = 32 * dkp / 8, KP = 2 * RP / TH;        // eights of a stage's rows (one kind), and a thread's of both
+  constexpr int VE = dvp * 4, VP = (VE + TH - 1) / TH;      // the same of its values
+  constexpr int SS = DVT / 2;                               // stages of the memory
+  static_assert(2 * RP % TH == 0, "whole rounds of rows");
+  extern __shared__ __attribute__((aligned(16))) bf16_t buffers[];
+  const int tid = threadIdx.x, lane = tid & 63, w = wave_index(), c16 = lane & 15, g = lane >> 4;
   const int c = blockIdx.x / z.H, h = blockIdx.x - c * z.H;
   const int t0 = chunks[3 * c + 1], n = chunks[3 * c + 2];
-  const int q0 = (blockIdx.y * 4 + w) * 16 * QT;  // the wavefront's first place in the chunk
-  if (q0 >= n) return;                            // (no barrier below)
+  const int q0 = w * 16;        // the wavefront's first place in the chunk
+  const bool live = q0 < n;
   const float log2_decay = decays[z.H + h];
-  int t[QT];
-  bf16x8 qh[QT][DKS], ql[QT][DKS];
+  const int t = q0 + c16;
+  const size_t own = (size_t)blockIdx.x * kChunk * dkp;
+  const bf16_t* vt = o.vt + (size_t)blockIdx.x * dvp * kChunk;
+  const size_t mem_at = (size_t)blockIdx.x * dvp * dkp;
+  const int stages = SS + (n + 31) / 32;
+
+  u32x4 reg[KP + VP];
+  auto fetch = [&](int stage) {
+    const bool keys = stage >= SS;
+    const size_t at = keys ? own + (size_t)(stage - SS) * 32 * dkp : mem_at + (size_t)stage * 32 * dkp;
+    const bf16_t *hi = (keys ? o.kh : o.sh) + at, *lo = (keys ? o.kl : o.sl) + at;
 #pragma unroll
-  for (int x = 0; x < QT; ++x) {
-    t[x] = q0 + 16 * x + c16;
-    const size_t at = ((size_t)blockIdx.x * kChunk + min(t[x], n - 1)) * dkp + 8 * g;
+    for (int i = 0; i < KP; ++i) {
+      const int idx = tid + TH * i;
+      reg[i] = *reinterpret_cast<const u32x4*>((idx < RP ? hi : lo) + (size_t)(idx < RP ? idx : idx - RP) * 8);
+    }
+    if (keys) {
+#pragma unroll
+      for (int i = 0; i < VP; ++i) {
+        const int idx = min(tid + TH * i, VE - 1);
+        reg[KP + i] = *reinterpret_cast<const u32x4*>(vt + (size_t)(idx >> 2) * kChunk + (stage - SS) * 32 + (idx & 3) * 8);
+      }
+    }
+  };
+  auto put = [&](int stage) {
+    bf16_t* b = buffers + (stage & 1) * BUF;
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int idx = tid + TH * i, in = idx < RP ? idx : idx - RP;
+      *reinterpret_cast<u32x4*>(b + (idx < RP ? 0 : HALF) + (in / (dkp / 8)) * LK + (in % (dkp / 8)) * 8) = reg[i];
+    }
+    if (stage >= SS) {
+#pragma unroll
+      for (int i = 0; i < VP; ++i) {
+        const int idx = tid + TH * i;
+        if (idx < VE) *reinterpret_cast<u32x4*>(b + 2 * HALF + (idx >> 2) * LV + (idx & 3) * 8) = reg[KP + i];
+      }
+    }
+    __syncthreads();
+    if (stage + 1 < stages) fetch(stage + 1);
+  };
+
+  fetch(0);
+  bf16x8 qh[DKS], ql[DKS];
+  {
+    const size_t at = own + (size_t)min(t, n - 1) * dkp + 8 * g;
 #pragma unroll
     for (int k = 0; k < DKS; ++k) {
-      qh[x][k] = piece(o.qh + at + 32 * k);
-      ql[x][k] = piece(o.ql + at + 32 * k);
+      qh[k] = piece(o.qh + at + 32 * k);
+      ql[k] = piece(o.ql + at + 32 * k);
     }
   }
-  f32x4 acc[QT][DVT];
+  f32x4 acc[DVT];
+#pragma unroll
+  for (int d = 0; d < DVT; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
   // the memory's part
-  {
-    const size_t s_at = (size_t)blockIdx.x * dvp * dkp + (size_t)c16 * dkp + 8 * g;
 #pragma unroll
-    for (int d = 0; d < DVT; ++d) {
+  for (int st = 0; st < SS; ++st) {
+    put(st);
+    if (!live) continue;
+    const bf16_t* b = buffers + (st & 1) * BUF + c16 * LK + 8 * g;
 #pragma unroll
-      for (int x = 0; x < QT; ++x) acc[x][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < DKS; ++k) {
+      bf16x8 sh[2], sl[2];
 #pragma unroll
-      for (int k = 0; k < DKS; ++k) {
-        const bf16x8 sh = piece(o.sh + s_at + (size_t)16 * d * dkp + 32 * k), sl = piece(o.sl + s_at + (size_t)16 * d * dkp + 32 * k);
-#pragma unroll
-        for (int x = 0; x < QT; ++x) {
-          acc[x][d] = mma(sl, qh[x][k], acc[x][d]);
-          acc[x][d] = mma(sh, ql[x][k], acc[x][d]);
-          acc[x][d] = mma(sh, qh[x][k], acc[x][d]);
-        }
+      for (int x = 0; x < 2; ++x) {
+        sh[x] = piece(b + 16 * x * LK + 32 * k);
+        sl[x] = piece(b + HALF + 16 * x * LK + 32 * k);
       }
-    }
 #pragma unroll
-    for (int x = 0; x < QT; ++x) {
-      const float f = __builtin_amdgcn_exp2f((float)(t[x] + 1) * log2_decay);
+      for (int x = 0; x < 2; ++x) acc[2 * st + x] = mma(sl[x], qh[k], acc[2 * st + x]);
 #pragma unroll
-      for (int d = 0; d < DVT; ++d) acc[x][d] *= f;
+      for (int x = 0; x < 2; ++x) acc[2 * st + x] = mma(sh[x], ql[k], acc[2 * st + x]);
+#pragma unroll
+      for (int x = 0; x < 2; ++x) acc[2 * st + x] = mma(sh[x], qh[k], acc[2 * st + x]);
     }
+  }
+  {
+    const float f = __builtin_amdgcn_exp2f((float)(t + 1) * log2_decay);
+#pragma unroll
+    for (int d = 0; d < DVT; ++d) acc[d] *= f;
   }
   // the chunk's own tokens
-  const int last = min(q0 + 16 * QT, n) - 1;
-  const bf16_t* vt = o.vt + (size_t)blockIdx.x * dvp * kChunk + (size_t)c16 * kChunk + 4 * g;
-  for (int s0 = 0; s0 <= last; s0 += 32) {
-    f32x4 st[QT][2];
+  for (int stage = SS; stage < stages; ++stage) {
+    put(stage);
+    const int s0 = (stage - SS) * 32;
+    if (!live || s0 > q0 + 15) continue;
+    const bf16_t* b = buffers + (stage & 1) * BUF;
+    f32x4 st[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    const bf16_t* kr = b + (8 * (c16 >> 2) + (c16 & 3)) * LK + 8 * g;
 #pragma unroll
-    for (int tt = 0; tt < 2; ++tt) {
+    for (int k = 0; k < DKS; ++k) {
+      bf16x8 kh[2], kl[2];
 #pragma unroll
-      for (int x = 0; x < QT; ++x) st[x][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
-      const size_t at = ((size_t)blockIdx.x * kChunk + min(s0 + 16 * tt + c16, n - 1)) * dkp + 8 * g;
-#pragma unroll
-      for (int k = 0; k < DKS; ++k) {
-        const bf16x8 kh = piece(o.kh + at + 32 * k), kl = piece(o.kl + at + 32 * k);
-#pragma unroll
-        for (int x = 0; x < QT; ++x) {
-          st[x][tt] = mma(kl, qh[x][k], st[x][tt]);
-          st[x][tt] = mma(kh, ql[x][k], st[x][tt]);
-          st[x][tt] = mma(kh, qh[x][k], st[x][tt]);
-        }
+      for (int tt = 0; tt < 2; ++tt) {
+        kh[tt] = piece(kr + 4 * tt * LK + 32 * k);
+        kl[tt] = piece(kr + HALF + 4 * tt * LK + 32 * k);
       }
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt) st[tt] = mma(kl[tt], qh[k], st[tt]);
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt) st[tt] = mma(kh[tt], ql[k], st[tt]);
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt) st[tt] = mma(kh[tt], qh[k], st[tt]);
     }
-    bf16x8 ph[QT], pl[QT];
+    uint32_t s[8];
 #pragma unroll
-    for (int x = 0; x < QT; ++x) {
-      uint32_t s[8];
+    for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-      for (int tt = 0; tt < 2; ++tt)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int back = t[x] - (s0 + 16 * tt + 4 * g + i);
-          const float p = back >= 0 ? st[x][tt][i] * __builtin_amdgcn_exp2f((float)back * log2_decay) : 0.f;
-          s[4 * tt + i] = split(p);
-        }
-      uint4 hi, lo;
-      deal8(s, hi, lo);
-      ph[x] = __builtin_bit_cast(bf16x8, hi);
-      pl[x] = __builtin_bit_cast(bf16x8, lo);
-    }
+      for (int i = 0; i < 4; ++i) {
+        const int back = t - (s0 + 8 * g + 4 * tt + i);
+        s[4 * tt + i] = split(back >= 0 ? st[tt][i] * __builtin_amdgcn_exp2f((float)back * log2_decay) : 0.f);
+      }
+    uint4 hi, lo;
+    deal8(s, hi, lo);
+    const bf16x8 ph = __builtin_bit_cast(bf16x8, hi), pl = __builtin_bit_cast(bf16x8, lo);
+    const bf16_t* vr = b + 2 * HALF + c16 * LV + 8 * g;
 #pragma unroll
     for (int d = 0; d < DVT; ++d) {
-      const bf16_t* v = vt + (size_t)16 * d * kChunk + s0;
-      const uint2 a = *reinterpret_cast<const uint2*>(v), b = *reinterpret_cast<const uint2*>(v + 16);
-      const bf16x8 vv = __builtin_bit_cast(bf16x8, uint4{a.x, a.y, b.x, b.y});
-#pragma unroll
-      for (int x = 0; x < QT; ++x) {
-        acc[x][d] = mma(vv, pl[x], acc[x][d]);
-        acc[x][d] = mma(vv, ph[x], acc[x][d]);
-      }
+      const bf16x8 v = piece(vr + 16 * d * LV);
+      acc[d] = mma(v, pl, acc[d]);
+      acc[d] = mma(v, ph, acc[d]);
     }
   }
+  if (!live) return;
   // norm and gate: a token's elements lie in the four lanes of its column
+  float ss = 0.f;
 #pragma unroll
-  for (int x = 0; x < QT; ++x) {
-    float ss = 0.f;
+  for (int d = 0; d < DVT; ++d)
 #pragma unroll
-    for (int d = 0; d < DVT; ++d)
+    for (int i = 0; i < 4; ++i) ss = __builtin_fmaf(acc[d][i], acc[d][i], ss);  // (zeros behind the real elements)
+  ss += __shfl_xor(ss, 16, 64);
+  ss += __shfl_xor(ss, 32, 64);
+  if (t >= n) return;
+  const float inv = 1.0f / sqrtf(ss / (float)z.dv + eps);
+  const size_t row = (size_t)(t0 + t);
+  const bf16_t* gr = rows + row * z.width() + 2 * z.H * z.dk + z.H * z.dv + h * z.dv + 4 * g;
+  bf16_t* dst = out + (row * z.H + h) * z.dv + 4 * g;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) ss = __builtin_fmaf(acc[x][d][i], acc[x][d][i], ss);  // (zeros behind the real elements)
-    ss += __shfl_xor(ss, 16, 64);
-    ss += __shfl_xor(ss, 32, 64);
-    if (t[x] >= n) continue;
-    const float inv = 1.0f / sqrtf(ss / (float)z.dv + eps);
-    const size_t row = (size_t)(t0 + t[x]);
-    const bf16_t* gr = rows + row * z.width() + 2 * z.H * z.dk + z.H * z.dv + h * z.dv + 4 * g;
-    bf16_t* dst = out + (row * z.H + h) * z.dv + 4 * g;
-#pragma unroll
-    for (int d = 0; d < DVT; ++d) {
-      const int e = 16 * d + 4 * g;
-      if (VEC) {
-        if (e < z.dv) {
-          const uint2 r = *reinterpret_cast<const uint2*>(gr + 16 * d);
-          const float g0 = __uint_as_float(r.x << 16), g1 = __uint_as_float(r.x & 0xffff0000u);
-          const float g2 = __uint_as_float(r.y << 16), g3 = __uint_as_float(r.y & 0xffff0000u);
-          *reinterpret_cast<uint2*>(dst + 16 * d) =
-              uint2{pack_bf16(acc[x][d][0] * inv * silu_(g0), acc[x][d][1] * inv * silu_(g1)),
-                    pack_bf16(acc[x][d][2] * inv * silu_(g2), acc[x][d][3] * inv * silu_(g3))};
-        }
-      } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (e + i < z.dv)
-            dst[16 * d + i] = float_to_bf16(acc[x][d][i] * inv * silu_(bf16_to_float(gr[16 * d + i])));
+  for (int d = 0; d < DVT; ++d) {
+    const int e = 16 * d + 4 * g;
+    if (VEC) {
+      if (e < z.dv) {
+        const uint2 r = *reinterpret_cast<const uint2*>(gr + 16 * d);
+        const float g0 = __uint_as_float(r.x << 16), g1 = __uint_as_float(r.x & 0xffff0000u);
+        const float g2 = __uint_as_float(r.y << 16), g3 = __uint_as_float(r.y & 0xffff0000u);
+        *reinterpret_cast<uint2*>(dst + 16 * d) = uint2{pack_bf16(acc[d][0] * inv * silu_(g0), acc[d][1] * inv * silu_(g1)),
+                                                        pack_bf16(acc[d][2] * inv * silu_(g2), acc[d][3] * inv * silu_(g3))};
       }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (e + i < z.dv) dst[16 * d + i] = float_to_bf16(acc[d][i] * inv * silu_(bf16_to_float(gr[16 * d + i])));
     }
   }
 }
@@ -718,15 +768,20 @@ size_t place(Operands& o, char* base, int nc, int H, int dk, int dv) {
   return at;
 }
 
-template <int DKS, int DVT>
+template <int DKS, int DVT, bool VEC>
 int launch_outputs(const bf16_t* rows, const Operands& o, const Heads& z, const float* decays, const int* chunks, int nc,
-                   bf16_t* out, float eps, bool vec, hipStream_t s) {
-  constexpr int QT = DVT <= 8 && DKS <= 4 ? 2 : 1;  // (what leaves registers for several wavefronts a SIMD)
-  const dim3 grid(nc * z.H, kChunk / (64 * QT));
-  if (vec)
-    hipLaunchKernelGGL((retention_outputs_kernel<DKS, DVT, QT, true>), grid, dim3(256), 0, s, rows, o, z, decays, chunks, out, eps);
-  else
-    hipLaunchKernelGGL((retention_outputs_kernel<DKS, DVT, QT, false>), grid, dim3(256), 0, s, rows, o, z, decays, chunks, out, eps);
+                   bf16_t* out, float eps, hipStream_t s) {
+  constexpr size_t lds = output_lds<DKS, DVT>();
+  static_assert(lds <= 160 * 1024, "the two buffers fit a compute unit");
+  static bool allowed = false;
+  if (!allowed) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&retention_outputs_kernel<DKS, DVT, VEC>),
+                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+    allowed = true;
+  }
+  hipLaunchKernelGGL((retention_outputs_kernel<DKS, DVT, VEC>), dim3(nc * z.H), dim3(kOutThreads), lds, s, rows, o, z, decays,
+                     chunks, out, eps);
   JLE_LAUNCH_CHECK();
   return 0;
 }
@@ -734,12 +789,16 @@ int launch_outputs(const bf16_t* rows, const Operands& o, const Heads& z, const 
 template <int DKS>
 int pick_outputs(const bf16_t* rows, const Operands& o, const Heads& z, const float* decays, const int* chunks, int nc,
                  bf16_t* out, float eps, bool vec, hipStream_t s) {
+#define OUTPUTS(DVT)                                                                                          \
+  return vec ? launch_outputs<DKS, DVT, true>(rows, o, z, decays, chunks, nc, out, eps, s)                    \
+             : launch_outputs<DKS, DVT, false>(rows, o, z, decays, chunks, nc, out, eps, s)
   switch (o.dvp) {
-    case 64: return launch_outputs<DKS, 4>(rows, o, z, decays, chunks, nc, out, eps, vec, s);
-    case 128: return launch_outputs<DKS, 8>(rows, o, z, decays, chunks, nc, out, eps, vec, s);
-    case 256: return launch_outputs<DKS, 16>(rows, o, z, decays, chunks, nc, out, eps, vec, s);
-    default: return launch_outputs<DKS, 32>(rows, o, z, decays, chunks, nc, out, eps, vec, s);
+    case 64: OUTPUTS(4);
+    case 128: OUTPUTS(8);
+    case 256: OUTPUTS(16);
+    default: OUTPUTS(32);
   }
+#undef OUTPUTS
 }
 
 int run_chunks(const bf16_t* rows, const float2* angles, const Heads& z, const Memory& mem, const int* chunks, int nc,
