@@ -377,8 +377,10 @@ int run_tokens(const UnitArgs<T>& p, T* out, int N, int blocks, bool vec, hipStr
   hipLaunchKernelGGL((gated_unit_tokens_kernel<T, RT, VEC>), dim3(blocks * tiles, (N + 16 * RT - 1) / (16 * RT)), \
                      dim3(64), 0, s, p, out, N, tiles)
   if (vec) {
-    if (N <= 16) TOKENS(1, true);
-    else if (N <= 32) TOKENS(2, true);
+    // (more rows a wavefront read the matrices less often; up to two wavefronts a SIMD it is their number that counts)
+    const long long waves = (long long)blocks * tiles * ((N + 15) / 16);
+    if (waves <= 2048) TOKENS(1, true);
+    else if (waves <= 4096) TOKENS(2, true);
     else TOKENS(4, true);
   } else {
     TOKENS(1, false);

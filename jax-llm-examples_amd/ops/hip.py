@@ -894,7 +894,7 @@ class HipOps:
 
     def linear_float32(self, h, w):
         """``h @ w.T`` with the float32 sums as they are: a library product where there are many rows."""
-        if h.dtype == torch.bfloat16 and (h.shape[0] > self.SKINNY_MAX_ROWS or h.shape[1] % 8):
+        if h.dtype == torch.bfloat16 and (h.shape[0] > self.SKINNY_DENSE_ROWS or h.shape[1] % 8):
             return torch.mm(h, w.t(), out_dtype=torch.float32)
         return self.lm_head(h, w)
 
